@@ -159,12 +159,26 @@ class CacheManager:
 
     def layer_cache(self, position: int, reader: bool = False) -> LayerCache:
         """The cache of schedule position `position`; `reader` marks a layer that
-        only reads it."""
+        only reads it (of a cache made of several parts, its pages: state belongs to the
+        run that keeps it)."""
         where = self._where[position]
         if isinstance(where, dict):
             return LayerCache(group=-1, owned=not reader, page_size=self.page_size,
-                              parts={name: self._one_cache(w, reader) for name, w in where.items()})
+                              parts={name: self._one_cache(w, reader) for name, w in where.items()
+                                     if not reader or w[0] == "pages"})
         return self._one_cache(where, reader)
+
+    def reading_cache(self, position: int, owner: int) -> LayerCache:
+        """The cache of a run at `position` that reads the one of position `owner`: what it
+        reads, and beside that what the run keeps for itself (where its mixer keeps anything)."""
+        cache = self.layer_cache(owner, reader=True)
+        if position in self._where:
+            own = self.layer_cache(position)
+            if not own.parts or (set(own.parts) & set(cache.parts)) or (not cache.parts and cache.group >= 0):
+                raise PageError(f"schedule position {position}: what a reading run keeps must be a composite cache "
+                                "whose entries have names of their own, beside a composite cache that it reads")
+            cache.parts.update(own.parts)
+        return cache
 
     def _one_cache(self, where: tuple, reader: bool) -> LayerCache:
         family, gi, li = where
@@ -220,7 +234,7 @@ class CacheManager:
 
     def trim(self, seq: SequenceCache, num_computed: int) -> int:
         """Give back the pages of groups with a window or a block-local mask that no
-        later query can reach.
+        later query can reach (those of the first `keep_first` tokens stay).
 
         After `num_computed` tokens the next query sits at position >=
         num_computed.  With a window it reads keys > num_computed - window; with
@@ -235,7 +249,8 @@ class CacheManager:
                 continue
             first_needed = g.spec.first_needed(num_computed)
             done = min(first_needed // self.page_size, len(table))
-            for i in range(seq._trimmed[gi], done):
+            kept = -(-g.spec.keep_first // self.page_size)  # pages of the first tokens stay
+            for i in range(max(seq._trimmed[gi], kept), done):
                 if table[i] >= 0:
                     g.pool.release(table[i])
                     table[i] = -1

@@ -42,12 +42,26 @@ class LayerNormSpec:
 
 
 @dataclass(frozen=True)
+class DynamicTanhSpec:
+    """y = tanh(alpha * x) * weight + bias, alpha a tensor of one number: a bounded elementwise map
+    in the place of a norm (no mean, no variance)."""
+
+    kind: ClassVar[str] = "dynamic_tanh"
+    names: Names = ()
+
+
+@dataclass(frozen=True)
 class RotarySpec:
-    """Rotation of element pairs (i, i + rotary_dim/2) by position * theta**(-2i/rotary_dim)."""
+    """Rotation of element pairs (i, i + rotary_dim/2) by position * theta**(-2i/rotary_dim).
+    ``scaling`` = (factor, original, fast, slow), YaRN: rates that make fewer than `slow` full
+    turns within `original` positions are divided by `factor`, rates that make more than `fast`
+    stay, those between are blended linearly in i; cosine and sine are multiplied by 0.1 *
+    ln(factor) + 1."""
 
     kind: ClassVar[str] = "rotary_half"
     theta: float
     rotary_dim: int
+    scaling: tuple | None = None
 
 
 @dataclass(frozen=True)
@@ -124,6 +138,47 @@ class AttentionSpec:
 
 
 @dataclass(frozen=True)
+class DifferentialAttentionSpec:
+    """Grouped-query attention whose heads are each the difference of two attentions ("maps") over
+    the same values, with a short convolution behind its projections and a window that keeps a
+    sequence's first tokens.
+
+    q = W_q x + b ([heads, 2, head_dim]), k = W_k x + b ([kv_heads, 2, head_dim]), v = W_v x + b
+    ([kv_heads, value_dim]); every channel of each passes a causal convolution over time (``conv``
+    taps, the last meets the current token, no bias; 0: none); ``position`` (a rotation spec or
+    None) turns each map of each head of q and k.  Map m of head h: softmax over the visible keys of
+    (q[h, m] . k[g, m]) * scale, times v[g], g = h // (heads / kv_heads).  With a1, a2 the two maps'
+    results and lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff (four learned vectors of head_dim):
+    o = a1 - lambda a2, o <- o / sqrt(mean(o^2) + eps) * (1 - diff), the mean over the head's
+    elements.  ``diff`` None: one map a head, ordinary attention, without lambda and that norm.
+    ``head_gate``: head h's result is multiplied by sigmoid(W_g x)_h, one number a head.  Then W_o.
+    ``window``: a query at i reads keys j <= i with i - j < window or j < keep_first; None reads
+    every key.  ``shared_kv``: the layer has no key and value tensors and reads the cache of another
+    run (ScheduleEntry.cache_of) with queries, convolution of the queries and mask of its own.
+    ``cache_window`` / ``cache_keep``: what the layer's cache keeps where a reader looks further
+    back than the layer ("own": the layer's window and keep_first; None: everything)."""
+
+    kind: ClassVar[str] = "differential_attention"
+    num_heads: int
+    num_kv_heads: int
+    head_dim: int
+    value_dim: int
+    scale: float
+    diff: float | None
+    eps: float
+    qkv_bias: bool = True
+    conv: int = 0
+    window: int | None = None
+    keep_first: int = 0
+    position: object = None
+    head_gate: bool = True
+    shared_kv: bool = False
+    cache_window: object = "own"
+    cache_keep: int | None = None
+    names: Names = ()
+
+
+@dataclass(frozen=True)
 class LatentAttentionSpec:
     """Attention whose queries, keys and values come through low-rank latents.
 
@@ -196,11 +251,13 @@ class SelectiveScanSpec:
 @dataclass(frozen=True)
 class RetentionSpec:
     """Linear attention with a fixed decay per head, no softmax and no denominator.  q = W_q x,
-    k = W_k x ([heads, head_dim]), v = W_v x ([heads, value_dim]); ``position`` (a rotation
-    spec or None) is applied to q and k; k is multiplied by head_dim ** -0.5;
-    S_t = decay[h] S_(t-1) + k_t v_t^T, o_t = S_t^T q_t.  Each head's o is divided by its root
-    mean square (``eps``, no weight), the heads side by side are multiplied by silu(W_g x),
-    then W_o.  Per request: S (float32)."""
+    k = W_k x ([heads, head_dim]), v = W_v x ([heads, value_dim]); ``activation`` "silu" is applied
+    to all three, ``position`` (a rotation spec or None) to q and k; k is multiplied by
+    ``key_scale`` (None: head_dim ** -0.5); S_t = decay[h] S_(t-1) + k_t v_t^T, o_t = S_t^T q_t.
+    Each head's o is divided by its root mean square (``eps``), or with ``norm_heads`` False the
+    heads side by side by theirs; with ``norm_weight`` (a tensor) they are multiplied by a weight of
+    their common size; then by the ``gate`` activation of W_g x ("silu", "sigmoid"), then W_o.  Per
+    request: S (float32)."""
 
     kind: ClassVar[str] = "retention"
     num_heads: int
@@ -210,6 +267,11 @@ class RetentionSpec:
     eps: float
     position: object = None
     names: Names = ()
+    activation: str | None = None
+    key_scale: float | None = None
+    norm_heads: bool = True
+    norm_weight: bool = False
+    gate: str = "silu"
 
 
 @dataclass(frozen=True)
@@ -256,7 +318,7 @@ class MoESpec:
 class DenseFFNSpec:
     """down(act(up(x))) without biases.  ``activation`` "xielu": for z > 0, softplus(p) z^2
     + z / 2; else (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2, with the layer's own two
-    numbers (p, q) in a tensor of two elements."""
+    numbers (p, q) in a tensor of two elements.  "relu_squared": max(z, 0)^2."""
 
     kind: ClassVar[str] = "dense_act"
     intermediate_size: int
@@ -300,8 +362,9 @@ class TokenSideSpec:
 
 @dataclass(frozen=True)
 class BlockSpec:
-    """x += mixer(mixer_norm(x)); x += ffn(ffn_norm(x)).  ``ffn`` may be None: the
-    layer then has no feed-forward and no second norm.
+    """x += mixer(mixer_norm(x)); x += ffn(ffn_norm(x)), both addends multiplied by
+    ``residual_scale``.  ``ffn`` may be None: the layer then has no feed-forward and no
+    second norm.
 
     ``name`` is the prefix of the block's tensors in the weight file; the
     ``*_name`` fields are the sub-names of its parts below that prefix.
@@ -317,6 +380,7 @@ class BlockSpec:
     ffn_name: str = "mlp"
     mixer_norm_name: str = "input_layernorm"
     ffn_norm_name: str = "post_attention_layernorm"
+    residual_scale: float = 1.0
 
 
 @dataclass(frozen=True)

@@ -109,7 +109,8 @@ int shk_interleave_gate_up(const void* gate_t, const void* up_t, int m, int k, v
                            void* stream);
 
 // out[n, m] (+)= a[n, k] @ w^T + bias with w given in the tiled layout; a is
-// bfloat16 row-major with row stride lda; out is bfloat16 or float32.
+// bfloat16 row-major with row stride lda; out is bfloat16 or float32.  accumulate 1
+// adds to a float32 out; accumulate 2 stores max(v, 0)^2 of every result v.
 // gated != 0: wt is an interleaved gate/up pair and out[n, m] = act(a @ gate^T) *
 // (a @ up^T), without bias or accumulation; gated is the activation, 1 for SiLU,
 // 2 for GELU in its tanh form, 3 for ReLU, 4 for g * sigmoid(1.702 g).  A gated product's
@@ -152,12 +153,13 @@ int shk_mfma_alone(const void* operands, float* out, int workgroups, int iters, 
 // pairing 1 pairs the neighbours (2i, 2i + 1) instead, with the same angle for pair i.
 // v_from_k != 0: there are no value columns, qkv is [n, (heads + kv_heads) * head_dim],
 // and a token's values are its keys as they were projected, before the rotation.
+// magnitude: what cosine and sine are multiplied by (1 for a plain rotation).
 int shk_rope_kv_store(void* qkv, int dtype, int n, int heads, int kv_heads, int head_dim,
                       int rot_dim, const float* inv_freq, const int32_t* positions,
                       const int32_t* token_seq, const int32_t* tables, int table_stride,
                       void* k_pool, void* v_pool, int page_size, int num_pages, int write_kv,
                       const float* parts, int splits, const float* bias, int pairing,
-                      int v_from_k, void* stream);
+                      int v_from_k, float magnitude, void* stream);
 
 // Causal attention of n query tokens over their sequences' paged caches.
 // Token t (position p, sequence s) reads keys j in (p - window, p] (all j <= p
@@ -378,7 +380,8 @@ int shk_selective_scan(const float* dt, const void* x, const float* bc, int ld_b
                        void* out, int dtype, int num_seqs, void* stream);
 
 // Retention (ssm.hip): per head S_t = decay[h] S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, over float32
-// projections at columns q_off, k_off ([heads, dim]) and v_off ([heads, v_dim]) of proj; a slot
+// projections at columns q_off, k_off ([heads, dim]) and v_off ([heads, v_dim]) of proj (act 1: SiLU
+// of each of them, 0: as they are); a slot
 // holds S as [heads, v_dim, dim].  shk_rotate_half_rows turns the pairs (i, i + rot_dim / 2) of
 // every head of float32 rows in place by positions[t] * inv_freq[i] and multiplies the head by mult.
 long long shk_retention_state_floats(int heads, int dim, int v_dim);
@@ -387,7 +390,65 @@ int shk_rotate_half_rows(float* x, int ld, int off, int heads, int dim, int rot_
 int shk_retention_scan(const float* proj, int ld, int q_off, int k_off, int v_off, const float* decay,
                        int num_seqs, int heads, int dim, int v_dim, const int32_t* positions,
                        const int32_t* cu_q, const int32_t* slots, float* state, long long slot_stride,
-                       float* out, void* stream);
+                       float* out, int act, void* stream);
+
+// tanh(alpha * x) * weight + bias in the place of a norm (dynamic_tanh.hip).  resid[row] gains scale *
+// delta[row] first (delta of `dtype`, or delta_splits float32 partial sums [splits][resid_rows][hidden];
+// null: nothing) and is stored back with write_resid; out[r] (null: none) belongs to row rows[r] (rows
+// null: row r).
+int shk_add_dynamic_tanh(float* resid, const void* delta, int delta_splits, float scale, float alpha,
+                         const float* weight, const float* bias, void* out, int dtype, const int32_t* rows, int n,
+                         int hidden, int write_resid, int resid_rows, void* stream);
+
+// Short convolution, rotation, cache write, gates (conv_store.hip).  A row of the projections (proj [n, ldp]
+// of `dtype`, or `splits` float32 partial sums [splits][n][ldp] plus bias [ldp] or null) holds q_heads * dim
+// query elements, k_heads * dim keys, v_heads * v_dim values, `gates` gate numbers, padding.  With taps
+// ([num_taps, channels] float32, channels = queries, keys and values; null: no convolution, num_taps 1)
+// every channel becomes y_t = sum_j taps[j] u_(t - num_taps + 1 + j), zeros before the sequence's start;
+// the first rot_dim elements of every query and key head turn in pairs (i, i + rot_dim / 2) by position *
+// inv_freq[i], cosine and sine times magnitude.  Queries go to q_out [n, q_heads * dim]; keys and values to
+// their pages as in shk_rope_kv_store, `maps` neighbouring key heads as one cached row of maps * dim
+// elements; gate_out [n, gates] = sigmoid.  state + slots[seq] * slot_stride holds the last num_taps - 1
+// inputs [num_taps - 1][channels] and is updated.  The first num_single sequences have one token each;
+// tile_lists holds num_tiles sequences, then num_tiles first queries within their portions, covering the
+// other sequences in steps of shk_conv_store_tile(num_taps) tokens.
+int shk_conv_store_tile(int taps);
+long long shk_conv_store_state_floats(int channels, int taps);
+int shk_conv_store(const void* proj, int ldp, const float* parts, int splits, const float* bias, int dtype, int n,
+                   const float* taps, int num_taps, int q_heads, int k_heads, int maps, int dim, int rot_dim,
+                   const float* inv_freq, float magnitude, int v_heads, int v_dim, int gates,
+                   const int32_t* positions, const int32_t* cu_q, const int32_t* slots, const int32_t* tables,
+                   int table_stride, float* state, long long slot_stride, const int32_t* tile_lists, int num_single,
+                   int num_tiles, void* q_out, float* gate_out, void* k_pool, void* v_pool, int page_size,
+                   int num_pages, void* stream);
+
+// Differential attention (attention_diff.hip, attention_diff_mfma.hip): q [n, heads, maps * dim] over a key
+// cache whose rows are [map 1, map 2]; with maps 2 a head's result is a1 - lambda a2, divided by
+// sqrt(mean^2 + eps) over its v_dim elements and multiplied by `rest`; gate (float32 [n, heads] or null)
+// multiplies it.  The query at position p reads keys j <= p with p - j < window (0: any) or j < keep_first.
+// shk_diff_attention serves any sizes up to 256; the bfloat16 kernels rows (maps * dim) and values in
+// multiples of 32 up to 128 and pages in multiples of 16.  Single tokens: the first num_seqs sequences;
+// partial: num_seqs * heads * maps * nsplit * (v_dim + 2) floats.  Portions: wg_lists holds num_wgs
+// sequences, then num_wgs first queries, in steps of 16 * shk_diff_attention_tiles(...); with nsplit > 1
+// partial: prompt_tokens * heads * maps * nsplit * (v_dim + 2) floats.
+int shk_diff_attention(const void* q, void* out, int dtype, int n, int heads, int kv_heads, int maps, int dim, int v_dim,
+                       const int32_t* positions, const int32_t* token_seq, const int32_t* tables, int table_stride,
+                       int num_seqs, const void* k_pool, const void* v_pool, int page_size, int num_pages, int window,
+                       int keep_first, float scale, float lambda, float rest, float eps, const float* gate,
+                       void* stream);
+int shk_diff_attention_supports_mfma(int heads, int kv_heads, int maps, int row_dim, int v_dim, int page_size);
+int shk_diff_attention_tiles(int heads, int kv_heads, int small);
+int shk_diff_attention_decode_bf16(const void* q, void* out, int num_seqs, int heads, int kv_heads, int maps, int row_dim,
+                                   int v_dim, const int32_t* positions, const int32_t* tables, int table_stride,
+                                   const void* k_pool, const void* v_pool, int page_size, int window, int keep_first,
+                                   float scale, float lambda, float rest, float eps, const float* gate, float* partial,
+                                   int nsplit, int streaming, void* stream);
+int shk_diff_attention_prefill_bf16(const void* q, void* out, int num_wgs, int heads, int kv_heads, int maps, int row_dim,
+                                    int v_dim, const int32_t* cu_q, const int32_t* ctx_lens, const int32_t* wg_lists,
+                                    const int32_t* tables, int table_stride, const void* k_pool, const void* v_pool,
+                                    int page_size, int window, int keep_first, float scale, float lambda, float rest,
+                                    float eps, const float* gate, int small, float* partial, int nsplit,
+                                    int first_token, int prompt_tokens, void* stream);
 
 // A routed mixture of gated experts (moe.hip).  shk_moe_route: softmax over the experts' logits
 // (float32 [n, ld]); the `top` largest of score + correction (null: none) are chosen [n, top],
@@ -460,7 +521,7 @@ long long shk_sample_scratch_floats(int rows, int vocab);
 // `stream` is passed instead.  The calls run in order on `stream`; the first that
 // refuses its arguments ends the run with its status and message (those before it
 // have been launched).
-#define SHK_CALL_MAX_ARGS 32
+#define SHK_CALL_MAX_ARGS 40
 typedef struct shk_call {
   int32_t launcher;
   int32_t reserved;

@@ -43,6 +43,7 @@ HIPCC_FLAGS = [
 # would cost a copy out and a copy back.
 FILE_FLAGS = {
     "attention_mfma.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
+    "attention_diff_mfma.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form=1"],
 }
 
 

@@ -79,6 +79,15 @@ __device__ __forceinline__ float gate_act(float g, int act) {
   return silu(g);
 }
 
+// The activation of a plain product: such a product's `accumulate` argument is 0 (store), 1 (add to a
+// float32 output) or kPlainReluSquared: the square of max(v, 0) is stored, v the sum with its bias.
+constexpr int kPlainReluSquared = 2;
+__device__ __forceinline__ float plain_act(float v, int accumulate) {
+  if (accumulate != kPlainReluSquared) return v;
+  const float r = fmaxf(v, 0.f);
+  return r * r;
+}
+
 // act(g) * u of a gated product.  A gate with constants brings them where other products bring their bias
 // (a gated product has none): args[0] > 0 bounds the gate from above and the other factor from both sides
 // before anything else, args[1] is added to that factor.
@@ -289,10 +298,11 @@ __global__ void __launch_bounds__(WAVES* kWave)
     }
     if (GATED) v = gate_times_up(v, up, accumulate, bias);
     if (!GATED && bias) v += bias[row];
+    if (!GATED) v = plain_act(v, accumulate);
     const size_t idx = static_cast<size_t>(token) * ldo + row;
     if (out_f32) {
       float* o = static_cast<float*>(out);
-      o[idx] = (accumulate && !GATED) ? o[idx] + v : v;
+      o[idx] = (accumulate == 1 && !GATED) ? o[idx] + v : v;
     } else {
       static_cast<bf16*>(out)[idx] = from_float<bf16>(v);
     }
@@ -420,6 +430,7 @@ __global__ void __launch_bounds__(WAVES* kWave)
     for (int r = 0; r < 4; ++r) {
       v[r] = GATED ? gate_times_up(acc[0][b][r], acc[RB - 1][b][r], accumulate, bias) : acc[0][b][r];
       if (!GATED && bias && row0 + r < m) v[r] += bias[row0 + r];
+      if (!GATED) v[r] = plain_act(v[r], accumulate);
     }
     if (ksplit > 1) {
       float* o = static_cast<float*>(out) + (static_cast<size_t>(blockIdx.y) * n + token) * ldo + row0;
@@ -433,7 +444,7 @@ __global__ void __launch_bounds__(WAVES* kWave)
       float* o = static_cast<float*>(out) + idx;
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        if (row0 + r < m) o[r] = (accumulate && !GATED) ? o[r] + v[r] : v[r];
+        if (row0 + r < m) o[r] = (accumulate == 1 && !GATED) ? o[r] + v[r] : v[r];
     } else {
       bf16* o = static_cast<bf16*>(out) + idx;
       if (row0 + 3 < m && (ldo & 3) == 0) {
@@ -484,14 +495,14 @@ __device__ __forceinline__ void big_store(const f32x4 (&acc)[WM][WN], int lane, 
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         v[r] = GATED ? gate_times_up(acc[i][jn][r], acc[i + (GATED ? 1 : 0)][jn][r], accumulate, bias)
-                     : acc[i][jn][r] + add[GATED ? 0 : i][r];
+                     : plain_act(acc[i][jn][r] + add[GATED ? 0 : i][r], accumulate);
       }
       const size_t idx = (static_cast<size_t>(share) * n + token) * ldo + row0;
       if (out_f32) {
         float* o = static_cast<float*>(out) + idx;
 #pragma unroll
         for (int r = 0; r < 4; ++r)
-          if (row0 + r < m) o[r] = (accumulate && !GATED) ? o[r] + v[r] : v[r];
+          if (row0 + r < m) o[r] = (accumulate == 1 && !GATED) ? o[r] + v[r] : v[r];
       } else {
         bf16* o = static_cast<bf16*>(out) + idx;
         if (row0 + 3 < m && (ldo & 3) == 0) {
@@ -1076,6 +1087,7 @@ __global__ void __launch_bounds__(16 * kWave)
     for (int r = 0; r < 4; ++r) {
       v[r] = acc[b][r];
       if (!GATED && bias && row0 + r < m) v[r] += bias[row0 + r];
+      if (!GATED) v[r] = plain_act(v[r], accumulate);
     }
     if (ksplit > 1) {
       float* o = static_cast<float*>(out) + (static_cast<size_t>(blockIdx.y) * n + token) * ldo + row0;
@@ -1089,7 +1101,7 @@ __global__ void __launch_bounds__(16 * kWave)
       float* o = static_cast<float*>(out) + idx;
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        if (row0 + r < m) o[r] = (accumulate && !GATED) ? o[r] + v[r] : v[r];
+        if (row0 + r < m) o[r] = (accumulate == 1 && !GATED) ? o[r] + v[r] : v[r];
     } else {
       bf16* o = static_cast<bf16*>(out) + idx;
       if (row0 + 3 < m && (ldo & 3) == 0) {
@@ -1402,7 +1414,8 @@ extern "C" int shk_gemm_bf16_tiled_weight(const void* a, const void* wt, const f
               out_dtype);
   SHK_REQUIRE(n >= 0 && m > 0 && k > 0, "gemm_bf16: bad sizes n=%d m=%d k=%d", n, m, k);
   SHK_REQUIRE(lda >= k && ldo >= m, "gemm_bf16: row strides lda=%d ldo=%d too small", lda, ldo);
-  SHK_REQUIRE(!accumulate || out_dtype == kF32, "gemm_bf16: accumulate needs a float32 output");
+  SHK_REQUIRE(accumulate >= 0 && accumulate <= kPlainReluSquared, "gemm_bf16: unknown epilogue %d", accumulate);
+  SHK_REQUIRE(accumulate != 1 || out_dtype == kF32, "gemm_bf16: accumulate needs a float32 output");
   if (n == 0) return 0;
   if (gated) accumulate = gated;  // the gated kernels read the activation from this argument
   SHK_REQUIRE(a && wt && out, "gemm_bf16: null pointer");

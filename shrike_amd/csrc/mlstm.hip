@@ -190,6 +190,44 @@ __global__ void __launch_bounds__(256)
   }
 }
 
+// The same for wide rows (many heads normed together): a workgroup per (token, head), the row held in
+// registers between its mean square and its write.
+constexpr int kWideRow = 512;   // wider rows take the workgroup
+constexpr int kWideHeld = 16;   // elements a thread holds (rows of up to 4096); beyond that they are read again
+template <typename T>
+__global__ void __launch_bounds__(256)
+    headnorm_gate_wide_kernel(const float* __restrict__ o, const float* __restrict__ gate, int gate_ld,
+                              const float* __restrict__ weight, float eps, T* __restrict__ out, int heads, int v_dim,
+                              int gate_act) {
+  __shared__ float scratch[16];
+  const int t = blockIdx.x / heads, h = blockIdx.x % heads;
+  const float* x = o + (static_cast<size_t>(t) * heads + h) * v_dim;
+  const float* g = gate + static_cast<size_t>(t) * gate_ld + h * v_dim;
+  float held[kWideHeld], gates[kWideHeld];
+  float sq = 0.f;
+#pragma unroll
+  for (int i = 0; i < kWideHeld; ++i) {
+    const int d = threadIdx.x + i * 256;
+    held[i] = d < v_dim ? x[d] : 0.f;
+    gates[i] = d < v_dim ? g[d] : 0.f;
+  }
+#pragma unroll
+  for (int i = 0; i < kWideHeld; ++i) sq = fmaf(held[i], held[i], sq);
+  for (int d = threadIdx.x + kWideHeld * 256; d < v_dim; d += 256) sq = fmaf(x[d], x[d], sq);
+  const float r = 1.f / sqrtf(block_sum(sq, scratch) / static_cast<float>(v_dim) + eps);
+  T* y = out + (static_cast<size_t>(t) * heads + h) * v_dim;
+  auto put = [&](int d, float xv, float gv) {
+    const float s = (gate_act == 1 ? gv : 1.f) / (1.f + expf(-gv));
+    y[d] = from_float<T>(xv * r * (weight ? weight[h * v_dim + d] : 1.f) * s);
+  };
+#pragma unroll
+  for (int i = 0; i < kWideHeld; ++i) {
+    const int d = threadIdx.x + i * 256;
+    if (d < v_dim) put(d, held[i], gates[i]);
+  }
+  for (int d = threadIdx.x + kWideHeld * 256; d < v_dim; d += 256) put(d, x[d], g[d]);
+}
+
 }  // namespace shk
 
 using namespace shk;
@@ -244,6 +282,17 @@ extern "C" int shk_headnorm_gate(const float* o, const float* gate, int gate_ld,
   SHK_REQUIRE(o && gate && out, "headnorm_gate: null pointer");
   hipStream_t s = static_cast<hipStream_t>(stream);
   const long long units = static_cast<long long>(n) * heads;
+  if (v_dim > kWideRow) {
+    SHK_REQUIRE(units < (1LL << 31), "headnorm_gate: too many rows");
+    if (dtype == kF32)
+      headnorm_gate_wide_kernel<float><<<static_cast<unsigned>(units), 256, 0, s>>>(
+          o, gate, gate_ld, weight, eps, static_cast<float*>(out), heads, v_dim, gate_act);
+    else
+      headnorm_gate_wide_kernel<bf16><<<static_cast<unsigned>(units), 256, 0, s>>>(
+          o, gate, gate_ld, weight, eps, static_cast<bf16*>(out), heads, v_dim, gate_act);
+    SHK_LAUNCH_CHECK("headnorm_gate");
+    return 0;
+  }
   const int grid = static_cast<int>((units + 3) / 4);
   if (dtype == kF32)
     headnorm_gate_kernel<float><<<grid, 256, 0, s>>>(o, gate, gate_ld, weight, eps, static_cast<float*>(out), n, heads, v_dim, gate_act);

@@ -1,7 +1,7 @@
 // Rotary position encoding of queries and keys fused with the write of keys
 // and values into their cache pages.  One thread per element pair (queries and
 // keys) or element (values); a workgroup first tabulates the cosines and sines
-// of its token in LDS.  Angles are float32 products as in the reference.  The projections may arrive as the float32 partial sums of a
+// of its token in LDS (both times `magnitude`).  Angles are float32 products as in the reference.  The projections may arrive as the float32 partial sums of a
 // product that was split along k; they are added here, in order, with the bias.
 #include "api.h"
 #include "common.h"
@@ -20,7 +20,7 @@ __global__ void __launch_bounds__(kRopeThreads)
                          int table_stride, T* __restrict__ k_pool, T* __restrict__ v_pool,
                          int page_size, int num_pages, int write_kv,
                          const float* __restrict__ parts, int splits,
-                         const float* __restrict__ bias, int adjacent, int v_from_k) {
+                         const float* __restrict__ bias, int adjacent, int v_from_k, float magnitude) {
   __shared__ float cs[kMaxHalf];
   __shared__ float sn[kMaxHalf];
   const int t = blockIdx.x;
@@ -109,8 +109,8 @@ __global__ void __launch_bounds__(kRopeThreads)
     const float reduced = static_cast<float>(fma(turns, -6.283185307179586, a));
     float sv, cv;
     sincosf(reduced, &sv, &cv);
-    cs[f] = cv;
-    sn[f] = sv;
+    cs[f] = cv * magnitude;
+    sn[f] = sv * magnitude;
   }
   __syncthreads();
 
@@ -155,7 +155,7 @@ __global__ void __launch_bounds__(kRopeThreads)
                              const int32_t* __restrict__ tables, int table_stride,
                              bf16* __restrict__ k_pool, bf16* __restrict__ v_pool, int page_size,
                              int num_pages, int write_kv, const float* __restrict__ parts, int splits,
-                             const float* __restrict__ bias) {
+                             const float* __restrict__ bias, float magnitude) {
   __shared__ float cs[kMaxHalf];
   __shared__ float sn[kMaxHalf];
   const int t = blockIdx.x;
@@ -243,8 +243,8 @@ __global__ void __launch_bounds__(kRopeThreads)
     const float reduced = static_cast<float>(fma(turns, -6.283185307179586, wide));
     float sv, cv;
     sincosf(reduced, &sv, &cv);
-    cs[f] = cv;
-    sn[f] = sv;
+    cs[f] = cv * magnitude;
+    sn[f] = sv * magnitude;
   }
   __syncthreads();
 
@@ -288,7 +288,7 @@ __global__ void __launch_bounds__(kRopeThreads)
                                       const int32_t* __restrict__ tables, int table_stride,
                                       bf16* __restrict__ k_pool, bf16* __restrict__ v_pool, int page_size,
                                       int num_pages, int write_kv, const float* __restrict__ parts,
-                                      int splits, const float* __restrict__ bias, int v_from_k) {
+                                      int splits, const float* __restrict__ bias, int v_from_k, float magnitude) {
   __shared__ float cs[kMaxHalf];
   __shared__ float sn[kMaxHalf];
   const int t = blockIdx.x;
@@ -371,8 +371,8 @@ __global__ void __launch_bounds__(kRopeThreads)
     const float reduced = static_cast<float>(fma(turns, -6.283185307179586, wide));
     float sv, cv;
     sincosf(reduced, &sv, &cv);
-    cs[f] = cv;
-    sn[f] = sv;
+    cs[f] = cv * magnitude;
+    sn[f] = sv * magnitude;
   }
   __syncthreads();
 
@@ -419,7 +419,7 @@ extern "C" int shk_rope_kv_store(void* qkv, int dtype, int n, int heads, int kv_
                                  const int32_t* tables, int table_stride, void* k_pool,
                                  void* v_pool, int page_size, int num_pages, int write_kv,
                                  const float* parts, int splits, const float* bias,
-                                 int pairing, int v_from_k, void* stream) {
+                                 int pairing, int v_from_k, float magnitude, void* stream) {
   SHK_REQUIRE(dtype == kF32 || dtype == kBF16, "rope_kv_store: unknown dtype %d", dtype);
   SHK_REQUIRE(pairing == 0 || pairing == 1, "rope_kv_store: unknown pairing %d", pairing);
   SHK_REQUIRE(n >= 0 && heads > 0 && kv_heads > 0 && head_dim > 0,
@@ -453,7 +453,7 @@ extern "C" int shk_rope_kv_store(void* qkv, int dtype, int n, int heads, int kv_
     rope_kv_store_vec_kernel<<<n, kRopeThreads, 0, s>>>(
         static_cast<bf16*>(qkv), n, heads, kv_heads, head_dim, inv_freq, positions, token_seq, tables,
         table_stride, static_cast<bf16*>(k_pool), static_cast<bf16*>(v_pool), page_size, num_pages,
-        write_kv, parts, splits, bias);
+        write_kv, parts, splits, bias, magnitude);
     SHK_LAUNCH_CHECK("rope_kv_store");
     return 0;
   }
@@ -465,7 +465,7 @@ extern "C" int shk_rope_kv_store(void* qkv, int dtype, int n, int heads, int kv_
     rope_kv_store_adjacent_vec_kernel<<<n, kRopeThreads, 0, s>>>(
         static_cast<bf16*>(qkv), n, heads, kv_heads, head_dim, inv_freq, positions, token_seq, tables,
         table_stride, static_cast<bf16*>(k_pool), static_cast<bf16*>(v_pool), page_size, num_pages,
-        write_kv, parts, splits, bias, v_from_k);
+        write_kv, parts, splits, bias, v_from_k, magnitude);
     SHK_LAUNCH_CHECK("rope_kv_store");
     return 0;
   }
@@ -476,12 +476,12 @@ extern "C" int shk_rope_kv_store(void* qkv, int dtype, int n, int heads, int kv_
     rope_kv_store_kernel<float><<<grid, kRopeThreads, 0, s>>>(
         static_cast<float*>(qkv), n, heads, kv_heads, head_dim, rot_dim, inv_freq, positions,
         token_seq, tables, table_stride, static_cast<float*>(k_pool), static_cast<float*>(v_pool),
-        page_size, num_pages, write_kv, parts, splits, bias, pairing, v_from_k);
+        page_size, num_pages, write_kv, parts, splits, bias, pairing, v_from_k, magnitude);
   else
     rope_kv_store_kernel<bf16><<<grid, kRopeThreads, 0, s>>>(
         static_cast<bf16*>(qkv), n, heads, kv_heads, head_dim, rot_dim, inv_freq, positions,
         token_seq, tables, table_stride, static_cast<bf16*>(k_pool), static_cast<bf16*>(v_pool),
-        page_size, num_pages, write_kv, parts, splits, bias, pairing, v_from_k);
+        page_size, num_pages, write_kv, parts, splits, bias, pairing, v_from_k, magnitude);
   SHK_LAUNCH_CHECK("rope_kv_store");
   return 0;
 }

@@ -13,7 +13,8 @@
 // A request's slot holds S [inner, state] and then the convolution's last taps - 1
 // inputs [(taps - 1), inner], oldest first.
 //
-// Retention, per head:  S_t = decay S_(t-1) + k_t v_t^T;  o_t = S_t^T q_t.
+// Retention, per head:  S_t = decay S_(t-1) + k_t v_t^T;  o_t = S_t^T q_t, q, k and v as projected or
+// with SiLU applied to each.
 // A request's slot holds S as [heads, v_dim, dim].
 #include "api.h"
 #include "common.h"
@@ -262,7 +263,7 @@ __global__ void __launch_bounds__(256)
                           const float* __restrict__ decay, int heads, int dim, int v_dim,
                           const int32_t* __restrict__ positions, const int32_t* __restrict__ cu_q,
                           const int32_t* __restrict__ slots, float* __restrict__ state, long long slot_stride,
-                          float* __restrict__ out, int block) {
+                          float* __restrict__ out, int block, int act) {
   // Tokens go by in blocks of `block` (at most kRetBlock): the queries and keys of the heads that this workgroup's columns
   // belong to are staged in LDS by the workgroup ([token][head][q | k]), a lane fetches its column's
   // values of the block at once: the walk waits for memory once a block.
@@ -296,12 +297,17 @@ __global__ void __launch_bounds__(256)
       const int tt = i / (nh * 2 * dim), rest = i % (nh * 2 * dim);
       const int hh = rest / (2 * dim), j = rest % (2 * dim);
       const float* row = proj + static_cast<size_t>(t0 + tt) * ld;
-      qks[i] = j < dim ? row[q_off + (h_lo + hh) * dim + j] : row[k_off + (h_lo + hh) * dim + j - dim];
+      const float x = j < dim ? row[q_off + (h_lo + hh) * dim + j] : row[k_off + (h_lo + hh) * dim + j - dim];
+      qks[i] = act ? silu_f(x) : x;
     }
     float vs[kRetBlock];
 #pragma unroll
     for (int k = 0; k < kRetBlock; ++k)
       vs[k] = proj[static_cast<size_t>(t0 + (k < count ? k : 0)) * ld + v_off + h * v_dim + col];
+    if (act) {
+#pragma unroll
+      for (int k = 0; k < kRetBlock; ++k) vs[k] = silu_f(vs[k]);
+    }
     __syncthreads();
 #pragma unroll
     for (int k = 0; k < kRetBlock; ++k) {
@@ -458,7 +464,8 @@ extern "C" long long shk_retention_state_floats(int heads, int dim, int v_dim) {
 extern "C" int shk_retention_scan(const float* proj, int ld, int q_off, int k_off, int v_off, const float* decay,
                                   int num_seqs, int heads, int dim, int v_dim, const int32_t* positions,
                                   const int32_t* cu_q, const int32_t* slots, float* state, long long slot_stride,
-                                  float* out, void* stream) {
+                                  float* out, int act, void* stream) {
+  SHK_REQUIRE(act == 0 || act == 1, "retention_scan: unknown activation %d (0: none, 1: SiLU)", act);
   SHK_REQUIRE(num_seqs >= 0 && heads > 0 && dim > 0 && dim <= 1024 && v_dim > 0,
               "retention_scan: bad sizes seqs=%d heads=%d dim=%d v_dim=%d", num_seqs, heads, dim, v_dim);
   SHK_REQUIRE(q_off >= 0 && k_off >= 0 && v_off >= 0 && q_off + heads * dim <= ld && k_off + heads * dim <= ld &&
@@ -479,7 +486,7 @@ extern "C" int shk_retention_scan(const float* proj, int ld, int q_off, int k_of
   const size_t lds = block * a_token;
 #define SHK_GO(L)                                                                                              \
   retention_scan_kernel<L, (L == 64 ? 16 : kRowsPerLane)><<<dim3((units + 256 / L - 1) / (256 / L), num_seqs), 256, lds, s>>>(                \
-      proj, ld, q_off, k_off, v_off, decay, heads, dim, v_dim, positions, cu_q, slots, state, slot_stride, out, block)
+      proj, ld, q_off, k_off, v_off, decay, heads, dim, v_dim, positions, cu_q, slots, state, slot_stride, out, block, act)
   switch (lanes) {
     case 1: SHK_GO(1); break;
     case 2: SHK_GO(2); break;

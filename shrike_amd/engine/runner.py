@@ -103,8 +103,10 @@ class ModelRunner:
         self.layer_caches = []
         for pos, entry in enumerate(model.spec.schedule):
             owner = pos if entry.cache_of is None else entry.cache_of
-            if cache.owns_cache(owner):
-                self.layer_caches.append(cache.layer_cache(owner, reader=entry.cache_of is not None))
+            if cache.owns_cache(owner) and entry.cache_of is not None:
+                self.layer_caches.append(cache.reading_cache(pos, owner))
+            elif cache.owns_cache(owner):
+                self.layer_caches.append(cache.layer_cache(owner))
             else:
                 self.layer_caches.append(None)
         # state that the embedding keeps per request follows the schedule's positions
@@ -155,8 +157,10 @@ class ModelRunner:
                     )
                 # the pages this step writes, and the oldest page it reads
                 first = g.spec.first_needed(e.start) // ps
+                kept = min(-(-g.spec.keep_first // ps), last_page + 1)  # pages of the first tokens, which stay
                 touched = table[e.start // ps : last_page + 1]
-                if min(touched) < 0 or max(touched) >= self.cache.num_pages or table[first] < 0:
+                if min(touched) < 0 or max(touched) >= self.cache.num_pages or table[first] < 0 \
+                        or any(page < 0 for page in table[:kept]):
                     raise StepError("block table names a page outside the pool")
 
     def _meta(self, entries: list[StepEntry], order: list[int], pad_to: int = 0,

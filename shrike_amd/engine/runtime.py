@@ -66,12 +66,16 @@ class Runtime:
         self.linear(x, w, gate_up)
         ops.act_mul(gate_up, out, activation, limit, up_shift)
 
-    def linear(self, x, w: LinearWeight, out, bias=None, accumulate=False) -> None:
-        """out (+)= x @ w.T + bias."""
+    def linear(self, x, w: LinearWeight, out, bias=None, accumulate=False, activation: str | None = None) -> None:
+        """out (+)= x @ w.T + bias; with `activation` ("relu_squared") out = act(x @ w.T + bias), in the
+        product's epilogue for bfloat16, by a kernel of its own for float32."""
         if w.tiled is not None:
-            ops.gemm_tiled_weight(x, w.tiled, w.rows, w.cols, out, bias=bias, accumulate=accumulate)
-        else:
-            ops.gemm(x, w.dense, out, bias=bias, accumulate=accumulate)
+            ops.gemm_tiled_weight(x, w.tiled, w.rows, w.cols, out, bias=bias, accumulate=accumulate,
+                                  activation=activation)
+            return
+        ops.gemm(x, w.dense, out, bias=bias, accumulate=accumulate)
+        if activation is not None:
+            ops.activate(out, out, activation)
 
     def linear_deferred(self, ctx, name: str, x, w: LinearWeight, bias=None, reader="norm",
                         keep_float32: bool = False):

@@ -15,7 +15,7 @@ from ctypes import c_char_p, c_float, c_int, c_longlong, c_void_p
 
 _LIB = None
 _RECORDING: list | None = None  # (launcher id, argument tuple) while a step is being recorded
-CALL_MAX_ARGS = 32
+CALL_MAX_ARGS = 40
 
 
 class KernelError(RuntimeError):
@@ -47,7 +47,7 @@ _SIGNATURES = {
     "shk_gemm_bf16_parts": [_I, _I, _I, _I],
     "shk_mfma_alone": [_P, _P, _I, _I, _P],
     "shk_rope_kv_store": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _P, _I, _P, _I, _I,
-                          _P],
+                          _F, _P],
     "shk_attention": [_P, _I, _P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _I, _F, _P, _P,
                       _I, _P],
     "shk_qkv_store": [_P, _I, _I, _I, _I, _I, _I, _F, _I, _F, _F, _P, _P, _I, _P, _P, _P, _I, _P, _P, _I, _I, _I, _P],
@@ -71,7 +71,19 @@ _SIGNATURES = {
     "shk_selective_scan": [_P, _P, _P, _I, _I, _I, _P, _I, _P, _P, _I, _I, _I, _P, _I, _P, _P, _P, _P, c_longlong,
                            _P, _I, _I, _P],
     "shk_rotate_half_rows": [_P, _I, _I, _I, _I, _I, _P, _P, _F, _I, _P],
-    "shk_retention_scan": [_P, _I, _I, _I, _I, _P, _I, _I, _I, _I, _P, _P, _P, _P, c_longlong, _P, _P],
+    "shk_retention_scan": [_P, _I, _I, _I, _I, _P, _I, _I, _I, _I, _P, _P, _P, _P, c_longlong, _P, _I, _P],
+    "shk_add_dynamic_tanh": [_P, _P, _I, _F, _F, _P, _P, _P, _I, _P, _I, _I, _I, _I, _P],
+    "shk_conv_store": [_P, _I, _P, _I, _P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _P, _F, _I, _I, _I, _P, _P, _P, _P, _I, _P,
+                       c_longlong, _P, _I, _I, _P, _P, _P, _P, _I, _I, _P],
+    "shk_conv_store_tile": [_I],
+    "shk_diff_attention": [_P, _P, _I, _I, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _F, _F, _F,
+                           _P, _P],
+    "shk_diff_attention_supports_mfma": [_I, _I, _I, _I, _I, _I],
+    "shk_diff_attention_tiles": [_I, _I, _I],
+    "shk_diff_attention_decode_bf16": [_P, _P, _I, _I, _I, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _I, _F, _F, _F, _F, _P,
+                                       _P, _I, _I, _P],
+    "shk_diff_attention_prefill_bf16": [_P, _P, _I, _I, _I, _I, _I, _I, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _F, _F, _F,
+                                        _F, _P, _I, _P, _I, _I, _I, _P],
     "shk_moe_route": [_P, _I, _P, _I, _I, _P, _P, _I, _P],
     "shk_moe_experts": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
     "shk_moe_experts_grouped": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
@@ -144,6 +156,7 @@ def load():
         for name, argtypes in (("shk_attention_talking_scratch_floats", [_I, _I, _I, _I]),
                                ("shk_selective_scan_state_floats", [_I, _I, _I]),
                                ("shk_retention_state_floats", [_I, _I, _I]),
+                               ("shk_conv_store_state_floats", [_I, _I]),
                                ("shk_moe_grouped_scratch_bytes", [_I, _I, _I, _I]),
                                ("shk_attention_talking_mfma_scratch_floats", [_I, _I, _I, _I, _I, _I])):
             fn = getattr(raw, name)

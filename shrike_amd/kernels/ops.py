@@ -395,15 +395,19 @@ def mfma_alone(operands: torch.Tensor, workgroups: int, iters: int) -> float:
 
 
 def gemm_tiled_weight(a, wt, m: int, k: int, out, bias=None, accumulate=False, gated=False,
-                      splits: int = 1, gate_args=None) -> None:
+                      splits: int = 1, gate_args=None, activation: str | None = None) -> None:
     """out (+)= a @ w.T + bias with wt = retile_weight(w): up to 64 rows of a
     stream the weights once; more rows run the LDS-staged MFMA kernel (tiles of
     128 x 128 to 256 x 256, chosen by how many the product has).
     splits > 1: out is float32 [splits, n, m] and receives partial sums.
     gated: False, or the gate's activation (one of GATE_ACTIVATIONS; True is "silu") for
     an interleaved gate/up weight.  gate_args: float32 [2] on the device, (limit, up_shift) of
-    such a gate: act(min(g, limit)) * (clamp(u, -limit, limit) + up_shift), limit 0: no bounds."""
+    such a gate: act(min(g, limit)) * (clamp(u, -limit, limit) + up_shift), limit 0: no bounds.
+    activation "relu_squared": max(v, 0)^2 of every result is stored (no gate, no accumulation,
+    no shares of k)."""
     _rows(a, "gemm a")
+    if activation is not None and (activation != "relu_squared" or gated or accumulate or splits > 1):
+        raise KernelError(f"gemm_tiled_weight: activation {activation!r} of a plain whole product must be 'relu_squared'")
     n = a.shape[0]
     if a.shape[1] != k or a.dtype != torch.bfloat16:
         raise KernelError(f"gemm_tiled_weight: a must be bfloat16 [n, {k}], got {tuple(a.shape)}")
@@ -427,7 +431,7 @@ def gemm_tiled_weight(a, wt, m: int, k: int, out, bias=None, accumulate=False, g
             _dev(a, "a"), _dev(wt, "wt"),
             None if bias is None else _dev(bias, "bias", torch.float32),
             _dev(out, "out"), n, m, k, a.stride(0), out.stride(-2), dtype_code(out.dtype),
-            int(bool(accumulate)), activation_code(gated), int(splits), _stream(),
+            2 if activation else int(bool(accumulate)), activation_code(gated), int(splits), _stream(),
         )
     )
 
@@ -465,13 +469,13 @@ def _check_pools(who, q, tables, k_pool, v_pool, kv_heads, head_dim, page_size, 
 
 def rope_kv_store(qkv, heads, kv_heads, head_dim, rot_dim, inv_freq, positions, token_seq,
                   tables, k_pool, v_pool, page_size, write_kv=True, split_sum=None,
-                  adjacent_pairs: bool = False, values_from_keys: bool = False) -> None:
+                  adjacent_pairs: bool = False, values_from_keys: bool = False, magnitude: float = 1.0) -> None:
     """Rotate q and k of qkv [n, (heads + 2 kv_heads) head_dim] in float32 and put
     k, v into their pages (keys in slabs, see key_pool_shape; values transposed
     [pages, kv_heads, head_dim, page_size]).  adjacent_pairs: element 2i turns with
     2i + 1 instead of i with i + rot_dim / 2.  values_from_keys: qkv has no value
     columns, [n, (heads + kv_heads) head_dim], and a token's values are its keys as
-    they come in (before the rotation)."""
+    they come in (before the rotation).  magnitude: a factor on cosine and sine."""
     n = qkv.shape[0]
     if not qkv.is_contiguous() or qkv.shape[1] != (heads + (1 if values_from_keys else 2) * kv_heads) * head_dim:
         raise KernelError("rope_kv_store: qkv must be contiguous [n, (heads + 2 kv_heads) head_dim] "
@@ -502,7 +506,7 @@ def rope_kv_store(qkv, heads, kv_heads, head_dim, rot_dim, inv_freq, positions, 
             page_size, num_pages, int(bool(write_kv)),
             None if parts is None else _dev(parts, "parts", torch.float32), splits,
             None if bias is None else _dev(bias, "bias", torch.float32),
-            int(bool(adjacent_pairs)), int(bool(values_from_keys)), _stream(),
+            int(bool(adjacent_pairs)), int(bool(values_from_keys)), float(magnitude), _stream(),
         )
     )
 
@@ -806,6 +810,29 @@ def add_layernorm(resid, delta=None, dnorm=None, weight=None, bias=None, eps: fl
         resid.shape[0], _stream()))
 
 
+def add_dynamic_tanh(resid, delta=None, scale: float = 1.0, alpha: float = 1.0, weight=None, bias=None, out=None,
+                     rows=None, write_resid: bool = True, dtype=None) -> None:
+    """resid [N, hidden] (float32) gains scale * delta (a product's output, tensor or SplitSum); `out`
+    [n, hidden] receives tanh(alpha * x) * weight + bias of the sums.  rows: int32 row indices, out[r]
+    then belongs to resid[rows[r]]."""
+    hidden = resid.shape[1]
+    if resid.dtype != torch.float32 or not resid.is_contiguous():
+        raise KernelError("add_dynamic_tanh: resid must be contiguous float32")
+    n = resid.shape[0] if rows is None else rows.shape[0]
+    if out is not None:
+        dtype = out.dtype
+        if tuple(out.shape) != (n, hidden) or not out.is_contiguous():
+            raise KernelError("add_dynamic_tanh: out must be contiguous [rows, hidden]")
+    if dtype is None:
+        raise KernelError("add_dynamic_tanh: give out or dtype")
+    d_ptr, d_splits = (None, 0) if delta is None else _delta_any(delta, resid.shape[0], hidden, dtype, "add_dynamic_tanh")
+    check(load().shk_add_dynamic_tanh(
+        _dev(resid, "resid"), d_ptr, d_splits, float(scale), float(alpha), _f32vec(weight, hidden, "weight"),
+        _f32vec(bias, hidden, "bias"), None if out is None else _dev(out, "out"), dtype_code(dtype),
+        None if rows is None else _dev(rows, "rows", torch.int32), n, hidden, int(bool(write_resid)), resid.shape[0],
+        _stream()))
+
+
 def mix_history(history, coef, count: int, out, delta=None, dnorm=None, dtype=None) -> None:
     """out = sum_j coef[j] * history[j], j < count (float32 [slots, n, hidden] -> [n, hidden]); with
     delta and dnorm = (weight, bias, eps), history[count - 1] first gains the normed addend."""
@@ -989,9 +1016,11 @@ def retention_state_floats(heads: int, dim: int, v_dim: int) -> int:
 
 
 def retention_scan(proj, q_off, k_off, v_off, decay, num_seqs, heads, dim, v_dim, positions, cu_q, slots, state,
-                   out) -> None:
+                   out, activation: str | None = None) -> None:
     """S_t = decay S_(t-1) + k v^T, o = S^T q per head over the step's tokens; proj float32 rows,
-    out float32 [n, heads * v_dim]."""
+    out float32 [n, heads * v_dim]; activation "silu": of q, k and v."""
+    if activation not in (None, "silu"):
+        raise KernelError(f"retention_scan: unknown activation {activation!r}")
     _rows(proj, "retention_scan proj")
     n = proj.shape[0]
     if proj.dtype != torch.float32 or out.dtype != torch.float32 or tuple(out.shape) != (n, heads * v_dim) \
@@ -1005,7 +1034,7 @@ def retention_scan(proj, q_off, k_off, v_off, decay, num_seqs, heads, dim, v_dim
     check(load().shk_retention_scan(
         _dev(proj, "proj"), proj.stride(0), q_off, k_off, v_off, _dev(decay, "decay"), num_seqs, heads, dim, v_dim,
         _dev(positions, "positions", torch.int32), _dev(cu_q, "cu_q", torch.int32), _dev(slots, "slots", torch.int32),
-        _dev(state, "state"), state.stride(0), _dev(out, "out"), _stream()))
+        _dev(state, "state"), state.stride(0), _dev(out, "out"), int(activation == "silu"), _stream()))
 
 
 def moe_route(logits, correction, top: int, chosen, weights) -> None:
@@ -1253,3 +1282,140 @@ def sample(logits, out, temperature, top_p, uniforms, scratch, nucleus: bool = T
             scratch.numel(), rows, vocab, logits.stride(0), int(bool(nucleus)), _stream(),
         )
     )
+
+
+def conv_store_tile(taps: int) -> int:
+    """Tokens of a prompt portion that one workgroup of conv_store takes."""
+    return int(load().shk_conv_store_tile(int(taps)))
+
+
+def conv_store_state_floats(channels: int, taps: int) -> int:
+    return int(load().shk_conv_store_state_floats(int(channels), int(taps)))
+
+
+def conv_store(proj, heads: int, kv_heads: int, maps: int, dim: int, v_dim: int, gates: int, taps, rot_dim: int, inv_freq,
+               magnitude: float, positions, cu_q, slots, tables, state, tiles, num_single: int, q_out, gate_out,
+               k_pool=None, v_pool=None, page_size: int = 0) -> None:
+    """Convolution over time, rotation and cache write of the projections [n, width >= heads * maps * dim +
+    kv_heads * (maps * dim + v_dim) + gates] (a tensor of q_out's dtype, or a SplitSum): queries to q_out [n,
+    heads * maps * dim], keys (maps * dim elements a head) and values to their pages, sigmoid of the gates to
+    gate_out (float32 [n, gates]).  kv_heads 0: rows of queries and gates alone.  taps: float32 [K, channels]
+    or None; state: float32 [slots, >= (K - 1) * channels].  tiles: int32 sequences then first queries of the
+    portions' tiles (conv_store_tile tokens each), or None; the first num_single sequences have one token."""
+    parts, splits, bias = None, 0, None
+    if isinstance(proj, SplitSum):
+        parts, bias = proj.parts, proj.bias
+        splits, n, width = parts.shape
+        if parts.dtype != torch.float32 or not parts.is_contiguous() or (bias is not None and bias.numel() != width):
+            raise KernelError("conv_store: partial sums must be contiguous float32 [splits, n, width]")
+    else:
+        n, width = proj.shape
+        if not proj.is_contiguous() or proj.dtype != q_out.dtype:
+            raise KernelError("conv_store: the projections must be contiguous and of q_out's dtype")
+    channels = heads * maps * dim + kv_heads * (maps * dim + v_dim)
+    if tuple(q_out.shape) != (n, heads * maps * dim) or not q_out.is_contiguous():
+        raise KernelError("conv_store: q_out must be contiguous [n, heads * maps * dim]")
+    if gates and (tuple(gate_out.shape) != (n, gates) or gate_out.dtype != torch.float32 or not gate_out.is_contiguous()):
+        raise KernelError("conv_store: gate_out must be contiguous float32 [n, gates]")
+    num_taps = 1
+    if taps is not None:
+        num_taps = taps.shape[0]
+        if tuple(taps.shape) != (num_taps, channels) or taps.dtype != torch.float32 or not taps.is_contiguous():
+            raise KernelError(f"conv_store: taps must be contiguous float32 [K, {channels}]")
+    stride = 0
+    if num_taps > 1:
+        if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1:
+            raise KernelError("conv_store: state must be float32 [slots, floats]")
+        stride = state.stride(0)
+    num_tiles = 0 if tiles is None else tiles.numel() // 2
+    if positions.shape[0] < n or cu_q.shape[0] < 2 or slots.shape[0] < num_single:
+        raise KernelError("conv_store: positions, cu_q or slots are shorter than the step")
+    if kv_heads:
+        _check_pools("conv_store", q_out, tables, k_pool, v_pool, kv_heads, maps * dim, page_size, v_dim)
+    check(load().shk_conv_store(
+        None if splits else _dev(proj, "proj"), width, None if parts is None else _dev(parts, "parts"), splits,
+        None if bias is None else _dev(bias, "bias", torch.float32), dtype_code(q_out.dtype), n,
+        None if taps is None else _dev(taps, "taps"), num_taps, heads * maps, kv_heads * maps, maps, dim, rot_dim,
+        None if inv_freq is None else _dev(inv_freq, "inv_freq", torch.float32), float(magnitude), kv_heads, v_dim, gates,
+        _dev(positions, "positions", torch.int32), _dev(cu_q, "cu_q", torch.int32), _dev(slots, "slots", torch.int32),
+        _dev(tables, "tables", torch.int32) if kv_heads else None, tables.shape[1] if kv_heads else 0,
+        _dev(state, "state") if num_taps > 1 else None, stride,
+        None if tiles is None else _dev(tiles, "tiles", torch.int32), num_single, num_tiles, _dev(q_out, "q_out"),
+        _dev(gate_out, "gate_out") if gates else None, _dev(k_pool, "k_pool") if kv_heads else None,
+        _dev(v_pool, "v_pool") if kv_heads else None, page_size, k_pool.shape[0] if kv_heads else 0, _stream()))
+
+
+def _diff_shapes(who, q, out, heads, maps, dim, v_dim, gate):
+    n = q.shape[0]
+    if tuple(q.shape) != (n, heads * maps * dim) or not q.is_contiguous():
+        raise KernelError(f"{who}: q must be contiguous [n, heads * maps * dim]")
+    if tuple(out.shape) != (n, heads * v_dim) or not out.is_contiguous() or out.dtype != q.dtype:
+        raise KernelError(f"{who}: out must be contiguous [n, heads * v_dim] of q's dtype")
+    if gate is not None and (tuple(gate.shape) != (n, heads) or gate.dtype != torch.float32 or not gate.is_contiguous()):
+        raise KernelError(f"{who}: gate must be contiguous float32 [n, heads]")
+
+
+def diff_attention(q, out, heads, kv_heads, maps, dim, v_dim, positions, token_seq, tables, k_pool, v_pool, page_size,
+                   window, keep_first, scale, lam: float, rest: float, eps: float, gate=None) -> None:
+    """Attention of heads of `maps` maps over one set of values, any sizes up to 256: q [n, heads * maps * dim],
+    keys cached as rows of maps * dim.  Two maps: (a1 - lam a2) brought to unit root mean square (eps), times
+    rest.  The query at p reads keys j <= p with p - j < window (None: any) or j < keep_first.  gate: float32
+    [n, heads] or None."""
+    _diff_shapes("diff_attention", q, out, heads, maps, dim, v_dim, gate)
+    _check_pools("diff_attention", q, tables, k_pool, v_pool, kv_heads, maps * dim, page_size, v_dim)
+    check(load().shk_diff_attention(
+        _dev(q, "q"), _dev(out, "out"), dtype_code(q.dtype), q.shape[0], heads, kv_heads, maps, dim, v_dim,
+        _dev(positions, "positions", torch.int32), _dev(token_seq, "token_seq", torch.int32),
+        _dev(tables, "tables", torch.int32), tables.shape[1], tables.shape[0], _dev(k_pool, "k_pool"),
+        _dev(v_pool, "v_pool"), page_size, k_pool.shape[0], int(window or 0), int(keep_first), float(scale), float(lam),
+        float(rest), float(eps), None if gate is None else _dev(gate, "gate"), _stream()))
+
+
+def diff_attention_supports_mfma(heads, kv_heads, maps, dim, v_dim, page_size) -> bool:
+    return bool(load().shk_diff_attention_supports_mfma(heads, kv_heads, maps, maps * dim, v_dim, page_size))
+
+
+def diff_attention_tiles(heads, kv_heads, small: bool = False) -> int:
+    """Query tiles of 16 that one workgroup of the prompt kernel serves (0: not served)."""
+    return int(load().shk_diff_attention_tiles(heads, kv_heads, int(bool(small))))
+
+
+def diff_attention_decode(q, out, num_seqs, heads, kv_heads, maps, dim, v_dim, positions, tables, k_pool, v_pool,
+                          page_size, window, keep_first, scale, lam, rest, eps, gate, partial, nsplit,
+                          streaming: bool = False) -> None:
+    """diff_attention for the first num_seqs rows, one token each (bfloat16, on the matrix units); partial:
+    float32, num_seqs * heads * maps * nsplit * (v_dim + 2)."""
+    _diff_shapes("diff_attention_decode", q, out, heads, maps, dim, v_dim, gate)
+    _check_pools("diff_attention_decode", q, tables, k_pool, v_pool, kv_heads, maps * dim, page_size, v_dim)
+    if q.dtype != torch.bfloat16 or num_seqs > min(q.shape[0], tables.shape[0]):
+        raise KernelError("diff_attention_decode: bfloat16 rows, one per sequence")
+    if partial.dtype != torch.float32 or partial.numel() < num_seqs * heads * maps * nsplit * (v_dim + 2):
+        raise KernelError("diff_attention_decode: partial is too small")
+    check(load().shk_diff_attention_decode_bf16(
+        _dev(q, "q"), _dev(out, "out"), num_seqs, heads, kv_heads, maps, maps * dim, v_dim,
+        _dev(positions, "positions", torch.int32), _dev(tables, "tables", torch.int32), tables.shape[1],
+        _dev(k_pool, "k_pool"), _dev(v_pool, "v_pool"), page_size, int(window or 0), int(keep_first), float(scale),
+        float(lam), float(rest), float(eps), None if gate is None else _dev(gate, "gate"), _dev(partial, "partial"),
+        int(nsplit), int(bool(streaming)), _stream()))
+
+
+def diff_attention_prefill(q, out, wg_lists, heads, kv_heads, maps, dim, v_dim, cu_q, ctx_lens, tables, k_pool, v_pool,
+                           page_size, window, keep_first, scale, lam, rest, eps, gate, small: bool = False, partial=None,
+                           nsplit: int = 1, first_token: int = 0) -> None:
+    """diff_attention for prompt portions (bfloat16, on the matrix units).  wg_lists: int32, the sequences of
+    the workgroups' runs of 16 * diff_attention_tiles(...) queries, then the runs' first queries."""
+    _diff_shapes("diff_attention_prefill", q, out, heads, maps, dim, v_dim, gate)
+    _check_pools("diff_attention_prefill", q, tables, k_pool, v_pool, kv_heads, maps * dim, page_size, v_dim)
+    if q.dtype != torch.bfloat16:
+        raise KernelError("diff_attention_prefill: bfloat16 rows only")
+    prompt = q.shape[0] - first_token
+    if nsplit > 1 and (partial is None or partial.dtype != torch.float32
+                       or partial.numel() < prompt * heads * maps * nsplit * (v_dim + 2)):
+        raise KernelError("diff_attention_prefill: partial is too small")
+    check(load().shk_diff_attention_prefill_bf16(
+        _dev(q, "q"), _dev(out, "out"), wg_lists.numel() // 2, heads, kv_heads, maps, maps * dim, v_dim,
+        _dev(cu_q, "cu_q", torch.int32), _dev(ctx_lens, "ctx_lens", torch.int32), _dev(wg_lists, "wg_lists", torch.int32),
+        _dev(tables, "tables", torch.int32), tables.shape[1], _dev(k_pool, "k_pool"), _dev(v_pool, "v_pool"), page_size,
+        int(window or 0), int(keep_first), float(scale), float(lam), float(rest), float(eps),
+        None if gate is None else _dev(gate, "gate"), int(bool(small)),
+        None if partial is None else _dev(partial, "partial"), int(nsplit), int(first_token), prompt, _stream()))

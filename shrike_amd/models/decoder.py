@@ -82,14 +82,14 @@ class DecoderModel:
         return all(part.launches_follow_shape for part in self.parts())
 
     def cache_specs(self) -> list:
-        """Cache need of every schedule position (None for a position that
-        reads another position's cache or whose mixer keeps nothing), and after
+        """Cache need of every schedule position (for a position that reads another
+        position's cache, what its mixer keeps beside that; None where nothing is kept), and after
         them, where the embedding keeps state per request, one more entry for it
         (position len(schedule))."""
         out = []
         for entry in self.spec.schedule:
             mixer = self.blocks[entry.block].mixer
-            out.append(None if entry.cache_of is not None else mixer.cache_spec())
+            out.append(mixer.reader_spec() if entry.cache_of is not None else mixer.cache_spec())
         if self.embedding_state is not None:
             out.append(self.embedding_state)
         return out

@@ -31,7 +31,7 @@ def compute_units() -> int:
 
 
 def kv_cache_spec(num_kv_heads: int, head_dim: int, window: int | None = None,
-                  chunk: int | None = None, value_dim: int | None = None) -> PagedSpec:
+                  chunk: int | None = None, value_dim: int | None = None, keep_first: int = 0) -> PagedSpec:
     """The cache of grouped-query attention, laid out for this file's kernels: per
     page and key/value head the keys in slabs of 32 elements, [head_dim / 32,
     page_size, 32] (a wavefront's operand load for the matrix instruction then
@@ -46,6 +46,7 @@ def kv_cache_spec(num_kv_heads: int, head_dim: int, window: int | None = None,
                  PageTensor("v", (num_kv_heads, head_dim if value_dim is None else value_dim, PAGE))),
         window=window,
         chunk=chunk,
+        keep_first=keep_first,
     )
 
 
@@ -546,6 +547,7 @@ class PagedAttention(Mixer):
             write_kv=cache.owned, split_sum=split_sum,
             adjacent_pairs=bool(table is not None and getattr(self.position, "adjacent_pairs", False)),
             values_from_keys=s.values_from_keys,
+            magnitude=float(getattr(self.position, "magnitude", 1.0)),
         )
         attn = ctx.buffer("attn_out", (n, s.num_heads * s.head_dim), ctx.dtype)
         self.attend(ctx, qkv, attn, tables, cache)

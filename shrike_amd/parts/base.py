@@ -97,16 +97,19 @@ class PagedSpec:
     """Cache need of a mixer: something per token, kept in pages, for all earlier
     tokens (window None) or for the last `window` of them; with `chunk`, only for
     the tokens of the current block of `chunk` positions (blocks counted from
-    position 0).  The cache manager allocates every listed tensor as [layers,
+    position 0).  The first `keep_first` tokens of a sequence stay whatever the window
+    has passed.  The cache manager allocates every listed tensor as [layers,
     pages + 1, *dims] and hands a layer its slice under the tensor's name; it
     knows nothing else about them."""
 
     tensors: tuple[PageTensor, ...]
     window: int | None = None
     chunk: int | None = None
+    keep_first: int = 0
 
     def first_needed(self, position: int) -> int:
-        """The oldest position that a query at `position` (or any later one) still reads."""
+        """The oldest position that a query at `position` (or any later one) still reads,
+        the first `keep_first` apart."""
         lo = 0
         if self.window is not None:
             lo = max(lo, position - self.window + 1)
@@ -156,15 +159,17 @@ class HiddenState:
     `pending_norm` = (weight float32 [width], eps) says that `pending` joins the
     stream as pending * rsqrt(mean(pending^2) + eps) * weight, row by row;
     (weight, bias, eps) that it joins as its layer norm, (pending - mean) /
-    sqrt(var + eps) * weight + bias.  `cast`: the stream as it stands (nothing pending) in the
+    sqrt(var + eps) * weight + bias.  `pending_scale`: what `pending` (without a norm of its
+    own) is multiplied by as it joins.  `cast`: the stream as it stands (nothing pending) in the
     compute dtype, where the kernel that wrote `resid` last left such a copy."""
 
-    __slots__ = ("resid", "pending", "pending_norm", "cast")
+    __slots__ = ("resid", "pending", "pending_norm", "pending_scale", "cast")
 
     def __init__(self, resid: torch.Tensor, pending: torch.Tensor | None = None, pending_norm=None):
         self.resid = resid
         self.pending = pending
         self.pending_norm = pending_norm
+        self.pending_scale = 1.0
         self.cast = None
 
     def settle(self, ctx) -> None:
@@ -179,9 +184,12 @@ class HiddenState:
         elif self.pending_norm is not None:
             weight, eps = self.pending_norm
             ops.add_normed_rmsnorm(self.resid, self.pending, weight, eps, dtype=ctx.dtype)
+        elif self.pending_scale != 1.0:
+            ops.add_dynamic_tanh(self.resid, self.pending, self.pending_scale, dtype=ctx.dtype)
         else:
             ops.add_deltas(self.resid, self.pending, dtype=ctx.dtype)
         self.pending = self.pending_norm = None
+        self.pending_scale = 1.0
 
 
 class Part:
@@ -234,7 +242,8 @@ class Norm(Part):
 class PositionEncoding(Part):
     def rotary_table(self):
         """(inv_freq float32 [rot_dim/2], rot_dim) when the encoding is a
-        half-split rotation that the cache-write kernel applies; else None."""
+        half-split rotation that the cache-write kernel applies; else None.  An encoding
+        whose cosines and sines have a factor names it as `magnitude`."""
         return None
 
     def apply(self, ctx, qkv: torch.Tensor, heads: int, kv_heads: int, head_dim: int) -> None:
@@ -250,7 +259,12 @@ class Mixer(Part):
     state_graph_safe = False
 
     def cache_spec(self):
-        """PagedSpec, StateSpec or None."""
+        """PagedSpec, StateSpec, CompositeSpec or None."""
+        return None
+
+    def reader_spec(self):
+        """What a run that reads another run's cache keeps of its own beside it: None, or a
+        CompositeSpec whose entries join those that are read in the LayerCache's `parts`."""
         return None
 
     def forward(self, ctx, x: torch.Tensor, cache) -> torch.Tensor:

@@ -1,4 +1,5 @@
-"""Pre-norm residual block: x += mixer(norm(x)); x += ffn(norm(x))."""
+"""Pre-norm residual block, x += mixer(norm(x)); x += ffn(norm(x)), and the other arrangements of
+norms and sublayers around the stream."""
 
 from __future__ import annotations
 
@@ -7,7 +8,8 @@ from .base import Block, HiddenState, build_part, register_block
 
 class PreNormResidualBlock(Block):
     """Reference: shrike/models/qwen.py:147-150.  The additions are not done
-    here: each part's output is left pending and the next norm adds it."""
+    here: each part's output is left pending and the next norm adds it, multiplied by the
+    spec's residual_scale."""
 
     def __init__(self, spec, width, name):
         super().__init__(spec, width, name)
@@ -40,12 +42,15 @@ class PreNormResidualBlock(Block):
             part.load(tensors, runtime)
 
     def forward(self, ctx, hidden: HiddenState, cache) -> None:
+        scale = float(getattr(self.spec, "residual_scale", 1.0))
         x = self.mixer_norm.forward(ctx, hidden)
         hidden.pending = self.mixer.forward(ctx, x, cache)
+        hidden.pending_scale = scale
         if self.ffn is None:
             return
         x = self.ffn_norm.forward(ctx, hidden)
         hidden.pending = self.ffn.forward(ctx, x)
+        hidden.pending_scale = scale
 
 
 register_block("prenorm_residual", PreNormResidualBlock)

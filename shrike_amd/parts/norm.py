@@ -1,4 +1,4 @@
-"""RMSNorm fused with the residual add that precedes it."""
+"""Norms (and a bounded map in the place of one) fused with the residual add that precedes them."""
 
 from __future__ import annotations
 
@@ -30,8 +30,9 @@ class RMSNorm(Norm):
     def forward(self, ctx, hidden: HiddenState, rows=None, write_resid=True) -> torch.Tensor:
         n = hidden.resid.shape[0] if rows is None else rows.shape[0]
         out = ctx.buffer(f"normed", (n, self.width), ctx.dtype)
-        if hidden.pending is not None and hidden.pending_norm is not None and len(hidden.pending_norm) == 3:
-            hidden.settle(ctx)  # an addend with a layer norm of its own joins by that norm's kernel
+        if hidden.pending is not None and (hidden.pending_scale != 1.0 or (
+                hidden.pending_norm is not None and len(hidden.pending_norm) == 3)):
+            hidden.settle(ctx)  # a scaled addend, or one with a layer norm of its own, joins by its own kernel
         if hidden.pending is not None and hidden.pending_norm is not None:
             dweight, deps = hidden.pending_norm
             ops.add_normed_rmsnorm(hidden.resid, hidden.pending, dweight, deps, self.weight, self.eps, out,
@@ -79,8 +80,8 @@ class LayerNorm(Norm):
         n = hidden.resid.shape[0] if rows is None else rows.shape[0]
         out = ctx.buffer("normed", (n, self.width), ctx.dtype)
         dnorm = hidden.pending_norm
-        if hidden.pending is not None and dnorm is not None and len(dnorm) != 3:
-            hidden.settle(ctx)  # an addend with a norm of another kind joins by that norm's kernel
+        if hidden.pending is not None and (hidden.pending_scale != 1.0 or (dnorm is not None and len(dnorm) != 3)):
+            hidden.settle(ctx)  # a scaled addend, or one with a norm of another kind, joins by its own kernel
         ops.add_layernorm(hidden.resid, hidden.pending, dnorm=dnorm if hidden.pending is not None else None,
                           weight=self.weight, bias=self.bias, eps=self.eps, out=out, rows=rows,
                           write_resid=write_resid, dtype=ctx.dtype)
@@ -92,3 +93,38 @@ class LayerNorm(Norm):
 
 
 register_norm("layernorm", LayerNorm)
+
+
+class DynamicTanh(Norm):
+    """y = tanh(alpha * x) * weight + bias in float32, alpha one learned number: a bounded
+    elementwise map that stands where a norm would.  What is pending joins the stream in the same
+    kernel, multiplied by hidden.pending_scale."""
+
+    launches_follow_shape = True
+
+    def params(self):
+        return [ParamSpec(self.tensor_name("weight"), (self.width,), init="norm", keep_float32=True),
+                ParamSpec(self.tensor_name("bias"), (self.width,), init="bias", keep_float32=True),
+                ParamSpec(self.tensor_name("alpha"), (), init="norm", keep_float32=True)]
+
+    def load(self, tensors, runtime):
+        self.weight = tensors[self.tensor_name("weight")].contiguous()
+        self.bias = tensors[self.tensor_name("bias")].contiguous()
+        self.alpha = float(tensors[self.tensor_name("alpha")])
+
+    def forward(self, ctx, hidden: HiddenState, rows=None, write_resid=True) -> torch.Tensor:
+        n = hidden.resid.shape[0] if rows is None else rows.shape[0]
+        out = ctx.buffer("normed", (n, self.width), ctx.dtype)
+        if hidden.pending is not None and hidden.pending_norm is not None:
+            hidden.settle(ctx)  # an addend with a norm of its own joins by that norm's kernel
+        ops.add_dynamic_tanh(hidden.resid, hidden.pending, hidden.pending_scale, self.alpha, self.weight, self.bias,
+                             out, rows, write_resid)
+        if write_resid:
+            if hidden.pending is not None:
+                hidden.cast = None  # the stream has changed under a copy that an earlier kernel left
+            hidden.pending = hidden.pending_norm = None
+            hidden.pending_scale = 1.0
+        return out
+
+
+register_norm("dynamic_tanh", DynamicTanh)

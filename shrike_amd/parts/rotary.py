@@ -1,10 +1,32 @@
-"""Rotary position encoding with the half-split pairing (i, i + rot_dim/2)."""
+"""Rotary position encoding with the half-split pairing (i, i + rot_dim/2), its rates by the base
+alone or stretched for longer contexts (YaRN), and with neighbouring pairs."""
 
 from __future__ import annotations
+
+import math
 
 import torch
 
 from .base import PositionEncoding, register_position
+
+
+def yarn_rates(theta: float, dims: int, factor: float, original: float, fast: float, slow: float):
+    """(rates [dims / 2], magnitude) in double precision.  A pair i that makes t full turns within
+    `original` positions has 2 i = dims * ln(original / (2 pi t)) / ln theta; the pairs from the one of
+    `fast` turns (rounded down) to the one of `slow` turns (rounded up) pass linearly from theta ** (-2i /
+    dims) to that rate over `factor`."""
+
+    def pair_of(turns: float) -> float:
+        return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(theta))
+
+    lo = max(math.floor(pair_of(fast)), 0)
+    hi = min(math.ceil(pair_of(slow)), dims - 1)
+    rates = []
+    for i in range(dims // 2):
+        ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+        rate = theta ** (-2.0 * i / dims)
+        rates.append(rate / factor * ramp + rate * (1.0 - ramp))
+    return rates, 0.1 * math.log(factor) + 1.0
 
 
 class RotaryHalf(PositionEncoding):
@@ -15,10 +37,16 @@ class RotaryHalf(PositionEncoding):
 
     launches_follow_shape = True
     adjacent_pairs = False  # pairs are (i, i + rot_dim / 2)
+    magnitude = 1.0  # what cosine and sine are multiplied by
 
     def load(self, tensors, runtime):
         d = int(self.spec.rotary_dim)
-        inv_freq = 1.0 / (float(self.spec.theta) ** (torch.arange(0, d, 2).float() / d))
+        scaling = getattr(self.spec, "scaling", None)
+        if scaling is not None:
+            rates, self.magnitude = yarn_rates(float(self.spec.theta), d, *scaling)
+            inv_freq = torch.tensor(rates, dtype=torch.float64).to(torch.float32)
+        else:
+            inv_freq = 1.0 / (float(self.spec.theta) ** (torch.arange(0, d, 2).float() / d))
         self.inv_freq = inv_freq.to(runtime.device)
         self.rot_dim = d
 
@@ -37,6 +65,7 @@ class RotaryAdjacent(PositionEncoding):
 
     launches_follow_shape = True
     adjacent_pairs = True
+    magnitude = 1.0
 
     def load(self, tensors, runtime):
         d = int(self.spec.rotary_dim)

@@ -93,11 +93,12 @@ register_mixer("selective_scan", SelectiveScan)
 
 
 class Retention(Mixer):
-    """One product yields queries, keys, values and the output gate of a token in float32;
-    queries and keys are rotated (the spec's position encoding, applied to float32 rows) and
-    the keys scaled; the scan carries S per head in the request's state slot (float32); the
-    readout is brought to unit root mean square per head, gated by SiLU of the gate
-    projection, and projected."""
+    """One product yields queries, keys, values and the output gate of a token in float32; by the
+    spec SiLU is applied to the first three; queries and keys are rotated (the spec's position
+    encoding, applied to float32 rows) and the keys scaled; the scan carries S per head in the
+    request's state slot (float32); the readout is brought to unit root mean square (per head, or
+    the heads together), weighted, gated by SiLU or the sigmoid of the gate projection, and
+    projected."""
 
     launches_follow_shape = True
     state_graph_safe = True
@@ -112,8 +113,11 @@ class Retention(Mixer):
     def params(self):
         s, h = self.spec, self.width
         qk, v = s.num_heads * s.head_dim, s.num_heads * s.value_dim
-        return [ParamSpec(self._t("q"), (qk, h)), ParamSpec(self._t("k"), (qk, h)), ParamSpec(self._t("v"), (v, h)),
-                ParamSpec(self._t("g"), (v, h)), ParamSpec(self._t("o"), (h, v))]
+        out = [ParamSpec(self._t("q"), (qk, h)), ParamSpec(self._t("k"), (qk, h)), ParamSpec(self._t("v"), (v, h)),
+               ParamSpec(self._t("g"), (v, h)), ParamSpec(self._t("o"), (h, v))]
+        if s.norm_weight:
+            out.append(ParamSpec(self._t("norm"), (v,), init="norm", keep_float32=True))
+        return out
 
     def state_floats(self) -> int:
         s = self.spec
@@ -132,8 +136,15 @@ class Retention(Mixer):
             raise ValueError(f"{self.name}: {len(s.decay)} decays for {s.num_heads} heads")
         if self.position is not None:
             if type(self.position).rotary_table is PositionEncoding.rotary_table \
-                    or getattr(self.position, "adjacent_pairs", False):
-                raise ValueError(f"{self.name}: retention rotates pairs (i, i + rot_dim / 2) only")
+                    or getattr(self.position, "adjacent_pairs", False) or getattr(s.position, "scaling", None):
+                raise ValueError(f"{self.name}: retention rotates pairs (i, i + rot_dim / 2) only, without scaling")
+            if s.activation is not None:
+                raise ValueError(f"{self.name}: retention applies an activation to queries and keys only where "
+                                 "they are not rotated")
+        if s.activation not in (None, "silu") or s.gate not in ("silu", "sigmoid"):
+            raise ValueError(f"{self.name}: unknown activation {s.activation!r} or gate {s.gate!r}")
+        if s.activation is not None and s.key_scale != 1.0:
+            raise ValueError(f"{self.name}: activated keys are not scaled (key_scale 1)")
         if ops.retention_state_floats(s.num_heads, s.head_dim, s.value_dim) != self.state_floats():
             raise RuntimeError(f"{self.name}: the kernel's state layout and the cache's size disagree")
 
@@ -145,6 +156,8 @@ class Retention(Mixer):
         self.in_width = 2 * qk + 2 * v
         self.decay = torch.tensor([float(d) for d in s.decay], dtype=torch.float32, device=runtime.device)
         self.w_o = runtime.weight(tensors[self._t("o")])
+        self.norm_weight = tensors[self._t("norm")].contiguous() if s.norm_weight else None
+        self.key_scale = float(s.head_dim) ** -0.5 if s.key_scale is None else float(s.key_scale)
         if self.position is not None:
             self.position.load(tensors, runtime)
         self.linear = runtime.linear
@@ -158,14 +171,15 @@ class Retention(Mixer):
         inv_freq, rot_dim = self.position.rotary_table() if self.position is not None else (None, 0)
         if rot_dim:
             ops.rotate_half_rows(proj, off["q"], s.num_heads, s.head_dim, rot_dim, inv_freq, ctx.positions, 1.0)
-        ops.rotate_half_rows(proj, off["k"], s.num_heads, s.head_dim, rot_dim, inv_freq, ctx.positions,
-                             float(s.head_dim) ** -0.5)
+        if rot_dim or self.key_scale != 1.0:
+            ops.rotate_half_rows(proj, off["k"], s.num_heads, s.head_dim, rot_dim, inv_freq, ctx.positions, self.key_scale)
         read = ctx.buffer("retention_read", (n, s.num_heads * s.value_dim), torch.float32)
         state = cache.state_padded if cache.state_padded is not None else cache.state
         ops.retention_scan(proj, off["q"], off["k"], off["v"], self.decay, ctx.num_seqs, s.num_heads, s.head_dim,
-                           s.value_dim, ctx.positions, ctx.cu_q, ctx.state_slots, state, read)
+                           s.value_dim, ctx.positions, ctx.cu_q, ctx.state_slots, state, read, activation=s.activation)
         gated = ctx.buffer("retention_gated", (n, s.num_heads * s.value_dim), ctx.dtype)
-        ops.headnorm_gate(read, proj[:, off["g"]:], None, s.eps, gated, s.num_heads, s.value_dim, gate_act="silu")
+        heads, size = (s.num_heads, s.value_dim) if s.norm_heads else (1, s.num_heads * s.value_dim)
+        ops.headnorm_gate(read, proj[:, off["g"]:], self.norm_weight, s.eps, gated, heads, size, gate_act=s.gate)
         return self.linear_deferred(ctx, "retention_out", gated, self.w_o)
 
 

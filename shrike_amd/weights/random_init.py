@@ -26,7 +26,9 @@ _STD = {"matrix": 0.02, "embedding": 0.02, "bias": 0.02, "norm": 0.1, "norm_zero
         # near the identity, and coefficients of an average (1 / count + N(0, 0.05))
         "positive": 0.5, "log_rate": 0.5, "near_identity": 0.1, "average": 0.05,
         # a table of numbers that are added to attention scores: N(0, 1) in both modes
-        "score_bias": 1.0}
+        "score_bias": 1.0,
+        # the taps of a short convolution: N(0, 0.3), and 1 added to the last (the current token's)
+        "taps": 0.3}
 
 #: "reference": the distributions above.  "unit": matrices N(0, 1/fan_in) (the
 #: embedding table N(0, 1)), biases N(0, 0.1): every part's output is as large
@@ -68,6 +70,8 @@ def random_tensor(p: ParamSpec, seed: int, dtype: torch.dtype, device="cpu",
         t += torch.eye(shape[0], shape[1], device=device)
     elif p.init == "average":
         t += 1.0 / shape[0]
+    elif p.init == "taps":
+        t[:, -1] += 1.0
     return t.to(dtype)
 
 
