@@ -327,8 +327,9 @@ def kernel_breakdown(engine, steps: int = 3, before_step=None) -> dict:
              "add_deltas", "add_normed_rmsnorm", "act_mul_rows", "add_rows", "embed_pairs", "qkv_store",
              "latent_prepare", "rotate_heads", "latent_attention", "latent_attention_mfma", "gemm_batched", "mlstm_scan", "headnorm_gate",
              "xielu", "layernorm", "add_layernorm", "attention_talking", "attention_talking_mfma", "conv_silu", "dt_softplus", "selective_scan",
-             "rotate_half_rows", "retention_scan", "moe_route", "moe_experts", "mix_history", "scale_softcap",
-             "postnorm", "cast_rows", "activate", "gate_mul"]
+             "rotate_half_rows", "retention_scan", "retention_chunk", "moe_route", "moe_experts", "mix_history", "scale_softcap",
+             "postnorm", "cast_rows", "activate", "gate_mul", "add_dynamic_tanh", "conv_store", "diff_attention",
+             "diff_attention_decode", "diff_attention_prefill"]
     names = [n for n in names if hasattr(ops, n)]
     spans: list[tuple[str, object, object]] = []
     saved = {n: getattr(ops, n) for n in names}
@@ -589,6 +590,53 @@ def poresun_like(qcfg, window: int, pattern: str, experts: int, top: int):
     return pcfg, sizes
 
 
+def fozedra_like(qcfg, window: int, pattern: str):
+    """A Fozedra configuration with the layer sizes of a Qwen2 one (same width, vocabulary and number
+    of layers).  `pattern` says which mixer each layer has, letter by letter, repeated: a, differential
+    attention with Qwen2's heads, each two maps of half a Qwen2 head (so queries, keys and values are as
+    wide as Qwen2's), rotated whole with stretched rates, a convolution of 4 taps, a window of `window`
+    keys that keeps the first 4; s, such a layer that reads the keys and values of the last a layer
+    before it; l, lightning attention with width / 256 heads of 128 query/key and 256 value elements (as
+    Ligipel's retention).  Every layer has the dense feed-forward with two matrices as wide as Qwen2's.
+    With it an object that names the sizes as the formulas of this program expect them."""
+    from types import SimpleNamespace
+
+    from shrike_amd.models.fozedra import FozedraConfig, FozedraLayer, Lightning, MappedAttention, Rotation
+
+    h, d, H, KV = qcfg.hidden_size, qcfg.head_dim, qcfg.num_attention_heads, qcfg.num_key_value_heads
+    inter, lheads = qcfg.intermediate_size, max(1, qcfg.hidden_size // 256)
+    rot = Rotation(base=qcfg.rope_theta, dims=d // 2, scaling=(4.0, 4096.0, 32.0, 1.0))
+    light = Lightning(heads=lheads, dim=128, vdim=256, decay=tuple(1.0 - 2.0 ** (-5 - i % 8) for i in range(lheads)))
+    layers, last_a = [], None
+    for i in range(qcfg.num_hidden_layers):
+        letter = pattern[i % len(pattern)]
+        if letter == "s" and last_a is None:
+            letter = "a"
+        if letter == "l":
+            layers.append((letter, FozedraLayer("lightning", light, inter)))
+        elif letter in "as":
+            mixer = MappedAttention(heads=H, kv_heads=KV, dim=d // 2, vdim=d, scale=(d // 2) ** -0.5, diff=0.5, conv=4,
+                                    window=window, keep_first=4, rot=rot, kv_from=last_a if letter == "s" else None)
+            last_a = i if letter == "a" else last_a
+            layers.append((letter, FozedraLayer("attention", mixer, inter)))
+        else:
+            raise SystemExit(f"--pattern: unknown letter {letter!r} for --fozedra (a, s, l)")
+    fcfg = FozedraConfig(vocab=qcfg.vocab_size, width=h, norm_eps=qcfg.rms_norm_eps,
+                         layers=tuple(layer for _, layer in layers), residual_mult=0.3)
+    n = len(layers)
+    elements = {"a": 2 * (H + KV) * d * h + H * h, "s": 2 * H * d * h + H * h, "l": (2 * 128 + 3 * 256) * lheads * h}
+    cached = {"a": 2 * KV * d, "s": 0, "l": 0}
+    states = {"a": 3 * (H + 2 * KV) * d, "s": 3 * H * d, "l": lheads * 128 * 256}
+    sizes = SimpleNamespace(
+        hidden_size=h, head_dim=d, num_attention_heads=H, num_key_value_heads=KV, intermediate_size=inter,
+        num_hidden_layers=n, vocab_size=qcfg.vocab_size, attention_layers=sum(letter != "l" for letter, _ in layers),
+        layer_elements=sum(elements[letter] for letter, _ in layers) // n + 2 * h * inter,
+        # (a layer that reads another's keys and values streams them once more)
+        kv_elements_per_token=sum(2 * KV * d for letter, _ in layers if letter != "l"),
+        state_bytes_per_seq=2 * 4 * sum(states[letter] for letter, _ in layers))
+    return fcfg, sizes
+
+
 def run_designs(args, qcfg) -> dict:
     """Another design beside Qwen2 at equal layer sizes, random weights: a prompt of 2,048
     tokens in one step, decode steps at batch 1, 8 and 64 from that context, and what each
@@ -598,9 +646,12 @@ def run_designs(args, qcfg) -> dict:
     import torch
 
     from shrike_amd import SamplingParams
-    from shrike_amd.models import ligipel, minilorn, mofarax, poresun, qwen2
+    from shrike_amd.models import fozedra, ligipel, minilorn, mofarax, poresun, qwen2
 
-    if args.poresun:
+    if args.fozedra:
+        fcfg, fsizes = fozedra_like(qcfg, args.window, args.pattern if set(args.pattern) <= set("asl") else "asl")
+        other = ("fozedra", fozedra.build_spec(fcfg), fsizes)
+    elif args.poresun:
         pcfg, psizes = poresun_like(qcfg, args.window, args.pattern if set(args.pattern) <= set("absl") else "absl",
                                     args.experts, args.top)
         other = ("poresun", poresun.build_spec(pcfg), psizes)
@@ -796,17 +847,21 @@ def main() -> int:
                     help="Ligipel beside Qwen2 at equal layer sizes: prompt, decode at batch 1/8/64, time per kernel")
     ap.add_argument("--poresun", action="store_true",
                     help="the Poresun design beside Qwen2 at the layer sizes of --shape, random weights")
+    ap.add_argument("--fozedra", action="store_true",
+                    help="the Fozedra design beside Qwen2 at the layer sizes of --shape, random weights")
     ap.add_argument("--experts", type=int, default=8, metavar="N", help="--ligipel, --poresun: routed experts a layer")
     ap.add_argument("--top", type=int, default=2, metavar="N", help="--ligipel, --poresun: experts a token uses")
     ap.add_argument("--pattern", default="alml", metavar="LETTERS",
                     help="--minilorn: the layers' mixers in order, repeated: a(ttention), l(atent attention), m(atrix memory); "
                          "--ligipel: p(arallel attention and scan), r(etention), default pppr; --poresun: a(ttention "
                          "with a window), b (causal attention), s (reads the last b layer's keys and values), "
-                         "l(atent attention), default absl")
+                         "l(atent attention), default absl; --fozedra: a (differential attention), s (reads the last a "
+                         "layer's keys and values), l(ightning attention), default asl")
     ap.add_argument("--window", type=int, default=4096, metavar="N",
                     help="--minilorn: sliding window of its latent attention (4096: no fewer keys than Qwen2 reads)")
-    ap.add_argument("--design-only", choices=["qwen2", "mofarax", "minilorn", "ligipel", "poresun"], default=None,
-                    help="--mofarax / --minilorn / --ligipel / --poresun: run only this one of the two (for a profile of "
+    ap.add_argument("--design-only", choices=["qwen2", "mofarax", "minilorn", "ligipel", "poresun", "fozedra"],
+                    default=None,
+                    help="--mofarax / --minilorn / --ligipel / --poresun / --fozedra: run only this one of the two (for a profile of "
                          "one model's kernels)")
     ap.add_argument("--mask-size", type=int, default=8192, metavar="N",
                     help="--mofarax: positions per block of its attention (8192: no fewer keys than Qwen2 reads)")
@@ -840,12 +895,14 @@ def main() -> int:
         raw["num_hidden_layers"] = args.layers
     cfg = Qwen2Config.from_dict(raw)
     spec = build_spec(cfg)
-    if args.mofarax or args.minilorn or args.ligipel or args.poresun:
+    if args.mofarax or args.minilorn or args.ligipel or args.poresun or args.fozedra:
         designs = run_designs(args, cfg)
-        design = "Poresun" if args.poresun else "Ligipel" if args.ligipel else "Minilorn" if args.minilorn else "Mofarax"
+        design = "Fozedra" if args.fozedra else "Poresun" if args.poresun else "Ligipel" if args.ligipel else "Minilorn" if args.minilorn else "Mofarax"
         config = {"shape": args.shape, "layers": cfg.num_hidden_layers, "prompt": PROMPT_LEN,
                   "decode_steps": args.design_steps}
-        config.update({"pattern": args.pattern if set(args.pattern) <= set("absl") else "absl", "window": args.window,
+        config.update({"pattern": args.pattern if set(args.pattern) <= set("asl") else "asl", "window": args.window}
+                      if args.fozedra
+                      else {"pattern": args.pattern if set(args.pattern) <= set("absl") else "absl", "window": args.window,
                        "experts": args.experts, "top": args.top} if args.poresun
                       else {"pattern": args.pattern if set(args.pattern) <= set("pr") else "pppr", "window": args.window,
                             "experts": args.experts, "top": args.top} if args.ligipel

@@ -110,7 +110,8 @@ int shk_interleave_gate_up(const void* gate_t, const void* up_t, int m, int k, v
 
 // out[n, m] (+)= a[n, k] @ w^T + bias with w given in the tiled layout; a is
 // bfloat16 row-major with row stride lda; out is bfloat16 or float32.  accumulate 1
-// adds to a float32 out; accumulate 2 stores max(v, 0)^2 of every result v.
+// adds to a float32 out; accumulate 2 stores max(v, 0)^2 of every result v; accumulate
+// 4 * r stores SiLU(v) for the first r of the m columns of out, v for the others.
 // gated != 0: wt is an interleaved gate/up pair and out[n, m] = act(a @ gate^T) *
 // (a @ up^T), without bias or accumulation; gated is the activation, 1 for SiLU,
 // 2 for GELU in its tanh form, 3 for ReLU, 4 for g * sigmoid(1.702 g).  A gated product's
@@ -304,7 +305,7 @@ int shk_mlstm_scan(const float* proj, int ld, int q_off, int k_off, int v_off, i
 // out[t, h, :] = o[t, h, :] * rsqrt(mean(o[t, h, :]^2) + eps) * weight[h, :] * g(gate[t, h, :]);
 // o float32 [n, heads * v_dim], gate float32 rows gate_ld apart, out of `dtype`.  weight may be
 // null (none); gate_act 0: g is the sigmoid, 1: SiLU.
-int shk_headnorm_gate(const float* o, const float* gate, int gate_ld, const float* weight, float eps,
+int shk_headnorm_gate(const float* o, const void* gate, int gate_dtype, int gate_ld, const float* weight, float eps,
                       void* out, int dtype, int n, int heads, int v_dim, int gate_act, void* stream);
 
 // Layer norm with weight and bias around the float32 stream (layernorm.hip).  For each of n
@@ -379,18 +380,27 @@ int shk_selective_scan(const float* dt, const void* x, const float* bc, int ld_b
                        const int32_t* cu_q, const int32_t* slots, float* state, long long slot_stride,
                        void* out, int dtype, int num_seqs, void* stream);
 
-// Retention (ssm.hip): per head S_t = decay[h] S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, over float32
-// projections at columns q_off, k_off ([heads, dim]) and v_off ([heads, v_dim]) of proj (act 1: SiLU
+// Retention (ssm.hip): per head S_t = decay[h] S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, over
+// projections (of `dtype`) at columns q_off, k_off ([heads, dim]) and v_off ([heads, v_dim]) of proj (act 1: SiLU
 // of each of them, 0: as they are); a slot
 // holds S as [heads, v_dim, dim].  shk_rotate_half_rows turns the pairs (i, i + rot_dim / 2) of
 // every head of float32 rows in place by positions[t] * inv_freq[i] and multiplies the head by mult.
 long long shk_retention_state_floats(int heads, int dim, int v_dim);
 int shk_rotate_half_rows(float* x, int ld, int off, int heads, int dim, int rot_dim, const float* inv_freq,
                          const int32_t* positions, float mult, int n, void* stream);
-int shk_retention_scan(const float* proj, int ld, int q_off, int k_off, int v_off, const float* decay,
+int shk_retention_scan(const void* proj, int dtype, int ld, int q_off, int k_off, int v_off, const float* decay,
                        int num_seqs, int heads, int dim, int v_dim, const int32_t* positions,
                        const int32_t* cu_q, const int32_t* slots, float* state, long long slot_stride,
                        float* out, int act, void* stream);
+// The same for prompt portions over bfloat16 projections as they are, in chunks on the matrix units
+// (retention_chunk.hip), for sequences first_seq .. first_seq + num_seqs - 1; dim 32, 64, 96, 128, 192 or
+// 256, v_dim in multiples of 32, columns in runs of 8.  A float32 operand of a product enters as the sum
+// of two bfloat16 numbers; sums and the state are float32.
+int shk_retention_chunk_supports(int dim, int v_dim);
+int shk_retention_chunk_bf16(const void* proj, int ld, int q_off, int k_off, int v_off, const float* decay,
+                             int first_seq, int num_seqs, int heads, int dim, int v_dim, const int32_t* positions,
+                             const int32_t* cu_q, const int32_t* slots, float* state, long long slot_stride, float* out,
+                             void* stream);
 
 // tanh(alpha * x) * weight + bias in the place of a norm (dynamic_tanh.hip).  resid[row] gains scale *
 // delta[row] first (delta of `dtype`, or delta_splits float32 partial sums [splits][resid_rows][hidden];

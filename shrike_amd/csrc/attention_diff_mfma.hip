@@ -327,9 +327,13 @@ __global__ void __launch_bounds__(kWave) diff_merge_kernel(const DiffArgs a, int
 // A workgroup of WAVES wavefronts serves every query head of one key/value head for a run of 16 * tiles
 // queries of one sequence; wavefront w owns head w % group, query tile w / group, both maps.  The chunk
 // of 32 keys (all of the row's slices, and the values) is staged once in LDS in operand layout.
+// Two maps' sums take twice the registers of one: with 8 wavefronts a workgroup they get 256 each (two
+// wavefronts on a SIMD, whose two maps are two independent chains); held to 128 the kernel spills and
+// takes 2.7 times as long (28 heads over 4, maps of 64, 2,048 queries: 305 us against 113), which is
+// what more than 8 heads a key/value head, in 16 wavefronts, still have to live with.
 // grid: entries of wg_seq / wg_q0 x kv_heads x splits.
 template <int D, int DV, int MAPS, int WAVES>
-__global__ void __launch_bounds__(WAVES* kWave) __attribute__((amdgpu_waves_per_eu(4)))
+__global__ void __launch_bounds__(WAVES* kWave) __attribute__((amdgpu_waves_per_eu(WAVES >= 16 || MAPS == 1 ? 4 : 2)))
     diff_prefill_kernel(const DiffArgs a, int tiles, const int32_t* __restrict__ cu_q,
                         const int32_t* __restrict__ ctx_lens, const int32_t* __restrict__ wg_seq,
                         const int32_t* __restrict__ wg_q0, int first_token, int partial_rows) {

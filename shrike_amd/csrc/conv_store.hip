@@ -410,6 +410,8 @@ extern "C" int shk_conv_store(const void* proj, int ldp, const float* parts, int
                         static_cast<const void*>(state), static_cast<const void*>(q_out), static_cast<const void*>(k_pool),
                         static_cast<const void*>(v_pool)})
     four = four && reinterpret_cast<uintptr_t>(p) % 16 == 0;
+  // few single tokens: a channel a thread, so that their launch has workgroups enough (the same sums either way)
+  if (a.tile == 1 && static_cast<long long>(num_single) * (channels / 4) < 128 * kConvThreads) four = false;
   const int V = four ? 4 : 1;
   const int items = channels / V - (q_heads + k_heads) * (rot_dim / 2) / V + gates;
   const dim3 grid(num_single + num_tiles, (items + kConvThreads - 1) / kConvThreads);

@@ -80,12 +80,21 @@ __device__ __forceinline__ float gate_act(float g, int act) {
 }
 
 // The activation of a plain product: such a product's `accumulate` argument is 0 (store), 1 (add to a
-// float32 output) or kPlainReluSquared: the square of max(v, 0) is stored, v the sum with its bias.
-constexpr int kPlainReluSquared = 2;
-__device__ __forceinline__ float plain_act(float v, int accumulate) {
-  if (accumulate != kPlainReluSquared) return v;
-  const float r = fmaxf(v, 0.f);
-  return r * r;
+// float32 output), kPlainReluSquared: the square of max(v, 0) is stored, v the sum with its bias, or 4 *
+// rows: the first `rows` output rows (weight rows) pass SiLU, the others are stored as they are.
+constexpr int kPlainReluSquared = 2, kPlainSiluRows = 4;
+__device__ __forceinline__ float plain_act(float v, int accumulate, int row) {
+  if (accumulate == kPlainReluSquared) {
+    const float r = fmaxf(v, 0.f);
+    return r * r;
+  }
+  return accumulate >= kPlainSiluRows && row < accumulate / kPlainSiluRows ? silu(v) : v;
+}
+// the same argument for the rows from `first` on
+inline int plain_act_from(int accumulate, int first) {
+  if (accumulate < kPlainSiluRows) return accumulate;
+  const int left = accumulate / kPlainSiluRows - first;
+  return left > 0 ? left * kPlainSiluRows : 0;
 }
 
 // act(g) * u of a gated product.  A gate with constants brings them where other products bring their bias
@@ -298,7 +307,7 @@ __global__ void __launch_bounds__(WAVES* kWave)
     }
     if (GATED) v = gate_times_up(v, up, accumulate, bias);
     if (!GATED && bias) v += bias[row];
-    if (!GATED) v = plain_act(v, accumulate);
+    if (!GATED) v = plain_act(v, accumulate, row);
     const size_t idx = static_cast<size_t>(token) * ldo + row;
     if (out_f32) {
       float* o = static_cast<float*>(out);
@@ -430,7 +439,7 @@ __global__ void __launch_bounds__(WAVES* kWave)
     for (int r = 0; r < 4; ++r) {
       v[r] = GATED ? gate_times_up(acc[0][b][r], acc[RB - 1][b][r], accumulate, bias) : acc[0][b][r];
       if (!GATED && bias && row0 + r < m) v[r] += bias[row0 + r];
-      if (!GATED) v[r] = plain_act(v[r], accumulate);
+      if (!GATED) v[r] = plain_act(v[r], accumulate, row0 + r);
     }
     if (ksplit > 1) {
       float* o = static_cast<float*>(out) + (static_cast<size_t>(blockIdx.y) * n + token) * ldo + row0;
@@ -495,7 +504,7 @@ __device__ __forceinline__ void big_store(const f32x4 (&acc)[WM][WN], int lane, 
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         v[r] = GATED ? gate_times_up(acc[i][jn][r], acc[i + (GATED ? 1 : 0)][jn][r], accumulate, bias)
-                     : plain_act(acc[i][jn][r] + add[GATED ? 0 : i][r], accumulate);
+                     : plain_act(acc[i][jn][r] + add[GATED ? 0 : i][r], accumulate, row0 + r);
       }
       const size_t idx = (static_cast<size_t>(share) * n + token) * ldo + row0;
       if (out_f32) {
@@ -1087,7 +1096,7 @@ __global__ void __launch_bounds__(16 * kWave)
     for (int r = 0; r < 4; ++r) {
       v[r] = acc[b][r];
       if (!GATED && bias && row0 + r < m) v[r] += bias[row0 + r];
-      if (!GATED) v[r] = plain_act(v[r], accumulate);
+      if (!GATED) v[r] = plain_act(v[r], accumulate, row0 + r);
     }
     if (ksplit > 1) {
       float* o = static_cast<float*>(out) + (static_cast<size_t>(blockIdx.y) * n + token) * ldo + row0;
@@ -1414,7 +1423,8 @@ extern "C" int shk_gemm_bf16_tiled_weight(const void* a, const void* wt, const f
               out_dtype);
   SHK_REQUIRE(n >= 0 && m > 0 && k > 0, "gemm_bf16: bad sizes n=%d m=%d k=%d", n, m, k);
   SHK_REQUIRE(lda >= k && ldo >= m, "gemm_bf16: row strides lda=%d ldo=%d too small", lda, ldo);
-  SHK_REQUIRE(accumulate >= 0 && accumulate <= kPlainReluSquared, "gemm_bf16: unknown epilogue %d", accumulate);
+  SHK_REQUIRE(accumulate >= 0 && (accumulate <= kPlainReluSquared || accumulate % kPlainSiluRows == 0),
+              "gemm_bf16: unknown epilogue %d", accumulate);
   SHK_REQUIRE(accumulate != 1 || out_dtype == kF32, "gemm_bf16: accumulate needs a float32 output");
   if (n == 0) return 0;
   if (gated) accumulate = gated;  // the gated kernels read the activation from this argument
@@ -1440,22 +1450,23 @@ extern "C" int shk_gemm_bf16_tiled_weight(const void* a, const void* wt, const f
       launch_big<4, 4, 4, 4, 1>(s, ap, lda, n, k, wp, kt, main_rows, bias, out, ldo, of, accumulate,
                                 vec, gated, main_blocks, 1);
       const uint4* rest_w = wp + static_cast<size_t>(main_blocks) * kt * kWave;
+      const int rest_act = gated ? accumulate : plain_act_from(accumulate, main_rows);
       // (a gated product's `bias` is its gate's two constants, the same for every row)
       const float* rest_bias = (bias && !gated) ? bias + main_rows : bias;
       void* rest_out = of ? static_cast<void*>(static_cast<float*>(out) + main_rows)
                           : static_cast<void*>(static_cast<bf16*>(out) + main_rows);
       if (rest_shape == 0)
         launch_big<4, 4, 4, 4, 1>(s, ap, lda, n, k, rest_w, kt, rest_rows, rest_bias, rest_out, ldo,
-                                  of, accumulate, vec, gated, rest_blocks, 1);
+                                  of, rest_act, vec, gated, rest_blocks, 1);
       else if (rest_shape == 1)
         launch_big<4, 4, 4, 2, 2>(s, ap, lda, n, k, rest_w, kt, rest_rows, rest_bias, rest_out, ldo,
-                                  of, accumulate, vec, gated, rest_blocks, 1);
+                                  of, rest_act, vec, gated, rest_blocks, 1);
       else if (static_cast<long long>((rest_blocks + 7) / 8) * ((n + 127) / 128) <= 256)
         launch_big<4, 2, 2, 4, 2>(s, ap, lda, n, k, rest_w, kt, rest_rows, rest_bias, rest_out, ldo,
-                                  of, accumulate, vec, gated, rest_blocks, 1);
+                                  of, rest_act, vec, gated, rest_blocks, 1);
       else
         launch_big<2, 2, 4, 4, 2>(s, ap, lda, n, k, rest_w, kt, rest_rows, rest_bias, rest_out, ldo,
-                                  of, accumulate, vec, gated, rest_blocks, 1);
+                                  of, rest_act, vec, gated, rest_blocks, 1);
       SHK_LAUNCH_CHECK("gemm_bf16");
       return 0;
     }

@@ -169,9 +169,9 @@ __global__ void __launch_bounds__(kScanWaves* kWave)
 // out[t, h, :] = o[t, h, :] / rms(o[t, h, :]) * weight[h, :] * sigmoid(gate[t, h, :]): the
 // per-head unit norm of a mixer's readout, its weight and its output gate in one pass.
 // One wavefront per (token, head).
-template <typename T>
+template <typename T, typename TG>
 __global__ void __launch_bounds__(256)
-    headnorm_gate_kernel(const float* __restrict__ o, const float* __restrict__ gate, int gate_ld,
+    headnorm_gate_kernel(const float* __restrict__ o, const TG* __restrict__ gate, int gate_ld,
                          const float* __restrict__ weight, float eps, T* __restrict__ out, int n, int heads,
                          int v_dim, int gate_act) {
   const int unit = blockIdx.x * (256 / kWave) + threadIdx.x / kWave;
@@ -182,50 +182,54 @@ __global__ void __launch_bounds__(256)
   float sq = 0.f;
   for (int d = lane; d < v_dim; d += kWave) sq = fmaf(x[d], x[d], sq);
   const float r = 1.f / sqrtf(wave_sum(sq) / static_cast<float>(v_dim) + eps);
-  const float* g = gate + static_cast<size_t>(t) * gate_ld + h * v_dim;
+  const TG* g = gate + static_cast<size_t>(t) * gate_ld + h * v_dim;
   T* y = out + (static_cast<size_t>(t) * heads + h) * v_dim;
   for (int d = lane; d < v_dim; d += kWave) {
-    const float s = (gate_act == 1 ? g[d] : 1.f) / (1.f + expf(-g[d]));
+    const float gv = to_float(g[d]);
+    const float s = (gate_act == 1 ? gv : 1.f) / (1.f + expf(-gv));
     y[d] = from_float<T>(x[d] * r * (weight ? weight[h * v_dim + d] : 1.f) * s);
   }
 }
 
-// The same for wide rows (many heads normed together): a workgroup per (token, head), the row held in
-// registers between its mean square and its write.
-constexpr int kWideRow = 512;   // wider rows take the workgroup
-constexpr int kWideHeld = 16;   // elements a thread holds (rows of up to 4096); beyond that they are read again
-template <typename T>
-__global__ void __launch_bounds__(256)
-    headnorm_gate_wide_kernel(const float* __restrict__ o, const float* __restrict__ gate, int gate_ld,
+// The same for wide rows (many heads normed together): a workgroup of THREADS per (token, head), the row held
+// in registers between its mean square and its write.  Few rows take wide workgroups, many rows narrow ones.
+constexpr int kWideRow = 512;    // wider rows take a workgroup
+constexpr int kWideHeld = 4096;  // elements a workgroup holds; beyond that they are read again
+template <typename T, typename TG, int THREADS>
+__global__ void __launch_bounds__(THREADS)
+    headnorm_gate_wide_kernel(const float* __restrict__ o, const TG* __restrict__ gate, int gate_ld,
                               const float* __restrict__ weight, float eps, T* __restrict__ out, int heads, int v_dim,
                               int gate_act) {
+  constexpr int kHeld = kWideHeld / THREADS;
   __shared__ float scratch[16];
   const int t = blockIdx.x / heads, h = blockIdx.x % heads;
   const float* x = o + (static_cast<size_t>(t) * heads + h) * v_dim;
-  const float* g = gate + static_cast<size_t>(t) * gate_ld + h * v_dim;
-  float held[kWideHeld], gates[kWideHeld];
+  const TG* g = gate + static_cast<size_t>(t) * gate_ld + h * v_dim;
+  const float* w = weight ? weight + h * v_dim : nullptr;
+  float held[kHeld], gates[kHeld], weights[kHeld];
   float sq = 0.f;
 #pragma unroll
-  for (int i = 0; i < kWideHeld; ++i) {
-    const int d = threadIdx.x + i * 256;
+  for (int i = 0; i < kHeld; ++i) {
+    const int d = threadIdx.x + i * THREADS;
     held[i] = d < v_dim ? x[d] : 0.f;
-    gates[i] = d < v_dim ? g[d] : 0.f;
+    gates[i] = d < v_dim ? to_float(g[d]) : 0.f;
+    weights[i] = d < v_dim && w ? w[d] : 1.f;
   }
 #pragma unroll
-  for (int i = 0; i < kWideHeld; ++i) sq = fmaf(held[i], held[i], sq);
-  for (int d = threadIdx.x + kWideHeld * 256; d < v_dim; d += 256) sq = fmaf(x[d], x[d], sq);
+  for (int i = 0; i < kHeld; ++i) sq = fmaf(held[i], held[i], sq);
+  for (int d = threadIdx.x + kWideHeld; d < v_dim; d += THREADS) sq = fmaf(x[d], x[d], sq);
   const float r = 1.f / sqrtf(block_sum(sq, scratch) / static_cast<float>(v_dim) + eps);
   T* y = out + (static_cast<size_t>(t) * heads + h) * v_dim;
-  auto put = [&](int d, float xv, float gv) {
+  auto put = [&](int d, float xv, float gv, float wv) {
     const float s = (gate_act == 1 ? gv : 1.f) / (1.f + expf(-gv));
-    y[d] = from_float<T>(xv * r * (weight ? weight[h * v_dim + d] : 1.f) * s);
+    y[d] = from_float<T>(xv * r * wv * s);
   };
 #pragma unroll
-  for (int i = 0; i < kWideHeld; ++i) {
-    const int d = threadIdx.x + i * 256;
-    if (d < v_dim) put(d, held[i], gates[i]);
+  for (int i = 0; i < kHeld; ++i) {
+    const int d = threadIdx.x + i * THREADS;
+    if (d < v_dim) put(d, held[i], gates[i], weights[i]);
   }
-  for (int d = threadIdx.x + kWideHeld * 256; d < v_dim; d += 256) put(d, x[d], g[d]);
+  for (int d = threadIdx.x + kWideHeld; d < v_dim; d += THREADS) put(d, x[d], to_float(g[d]), w ? w[d] : 1.f);
 }
 
 }  // namespace shk
@@ -272,9 +276,10 @@ extern "C" int shk_mlstm_scan(const float* proj, int ld, int q_off, int k_off, i
   return 0;
 }
 
-extern "C" int shk_headnorm_gate(const float* o, const float* gate, int gate_ld, const float* weight, float eps,
-                                 void* out, int dtype, int n, int heads, int v_dim, int gate_act, void* stream) {
+extern "C" int shk_headnorm_gate(const float* o, const void* gate, int gate_dtype, int gate_ld, const float* weight,
+                                 float eps, void* out, int dtype, int n, int heads, int v_dim, int gate_act, void* stream) {
   SHK_REQUIRE(dtype == kF32 || dtype == kBF16, "headnorm_gate: unknown dtype %d", dtype);
+  SHK_REQUIRE(gate_dtype == kF32 || (gate_dtype == kBF16 && dtype == kBF16), "headnorm_gate: unknown gate dtype %d", gate_dtype);
   SHK_REQUIRE(gate_act == 0 || gate_act == 1, "headnorm_gate: unknown gate %d (0: sigmoid, 1: SiLU)", gate_act);
   SHK_REQUIRE(n >= 0 && heads > 0 && v_dim > 0 && gate_ld >= heads * v_dim, "headnorm_gate: bad sizes n=%d heads=%d v_dim=%d gate_ld=%d",
               n, heads, v_dim, gate_ld);
@@ -282,22 +287,25 @@ extern "C" int shk_headnorm_gate(const float* o, const float* gate, int gate_ld,
   SHK_REQUIRE(o && gate && out, "headnorm_gate: null pointer");
   hipStream_t s = static_cast<hipStream_t>(stream);
   const long long units = static_cast<long long>(n) * heads;
-  if (v_dim > kWideRow) {
-    SHK_REQUIRE(units < (1LL << 31), "headnorm_gate: too many rows");
-    if (dtype == kF32)
-      headnorm_gate_wide_kernel<float><<<static_cast<unsigned>(units), 256, 0, s>>>(
-          o, gate, gate_ld, weight, eps, static_cast<float*>(out), heads, v_dim, gate_act);
-    else
-      headnorm_gate_wide_kernel<bf16><<<static_cast<unsigned>(units), 256, 0, s>>>(
-          o, gate, gate_ld, weight, eps, static_cast<bf16*>(out), heads, v_dim, gate_act);
-    SHK_LAUNCH_CHECK("headnorm_gate");
-    return 0;
-  }
-  const int grid = static_cast<int>((units + 3) / 4);
-  if (dtype == kF32)
-    headnorm_gate_kernel<float><<<grid, 256, 0, s>>>(o, gate, gate_ld, weight, eps, static_cast<float*>(out), n, heads, v_dim, gate_act);
-  else
-    headnorm_gate_kernel<bf16><<<grid, 256, 0, s>>>(o, gate, gate_ld, weight, eps, static_cast<bf16*>(out), n, heads, v_dim, gate_act);
+  SHK_REQUIRE(units < (1LL << 31), "headnorm_gate: too many rows");
+#define SHK_GO(T, TG)                                                                                              \
+  do {                                                                                                             \
+    const TG* gp = static_cast<const TG*>(gate);                                                                   \
+    T* op = static_cast<T*>(out);                                                                                  \
+    if (v_dim > kWideRow && units < 512)                                                                           \
+      headnorm_gate_wide_kernel<T, TG, 1024><<<static_cast<unsigned>(units), 1024, 0, s>>>(o, gp, gate_ld, weight, \
+                                                                                          eps, op, heads, v_dim, gate_act); \
+    else if (v_dim > kWideRow)                                                                                     \
+      headnorm_gate_wide_kernel<T, TG, 256><<<static_cast<unsigned>(units), 256, 0, s>>>(o, gp, gate_ld, weight,   \
+                                                                                        eps, op, heads, v_dim, gate_act); \
+    else                                                                                                           \
+      headnorm_gate_kernel<T, TG><<<static_cast<unsigned>((units + 3) / 4), 256, 0, s>>>(o, gp, gate_ld, weight, eps, op, n, \
+                                                                                        heads, v_dim, gate_act);   \
+  } while (0)
+  if (dtype == kF32) SHK_GO(float, float);
+  else if (gate_dtype == kF32) SHK_GO(bf16, float);
+  else SHK_GO(bf16, bf16);
+#undef SHK_GO
   SHK_LAUNCH_CHECK("headnorm_gate");
   return 0;
 }

@@ -257,9 +257,9 @@ inline int retention_heads_a_workgroup(int lanes, int heads, int v_dim) {
 
 // One sequence's tokens for one (head, value column); LANES lanes share the column's rows
 // of S (LANES * 8 >= dim).
-template <int LANES, int kRowsPerLane>
+template <typename T, int LANES, int kRowsPerLane>
 __global__ void __launch_bounds__(256)
-    retention_scan_kernel(const float* __restrict__ proj, int ld, int q_off, int k_off, int v_off,
+    retention_scan_kernel(const T* __restrict__ proj, int ld, int q_off, int k_off, int v_off,
                           const float* __restrict__ decay, int heads, int dim, int v_dim,
                           const int32_t* __restrict__ positions, const int32_t* __restrict__ cu_q,
                           const int32_t* __restrict__ slots, float* __restrict__ state, long long slot_stride,
@@ -296,14 +296,14 @@ __global__ void __launch_bounds__(256)
     for (int i = threadIdx.x; i < count * nh * 2 * dim; i += 256) {
       const int tt = i / (nh * 2 * dim), rest = i % (nh * 2 * dim);
       const int hh = rest / (2 * dim), j = rest % (2 * dim);
-      const float* row = proj + static_cast<size_t>(t0 + tt) * ld;
-      const float x = j < dim ? row[q_off + (h_lo + hh) * dim + j] : row[k_off + (h_lo + hh) * dim + j - dim];
+      const T* row = proj + static_cast<size_t>(t0 + tt) * ld;
+      const float x = to_float(j < dim ? row[q_off + (h_lo + hh) * dim + j] : row[k_off + (h_lo + hh) * dim + j - dim]);
       qks[i] = act ? silu_f(x) : x;
     }
     float vs[kRetBlock];
 #pragma unroll
     for (int k = 0; k < kRetBlock; ++k)
-      vs[k] = proj[static_cast<size_t>(t0 + (k < count ? k : 0)) * ld + v_off + h * v_dim + col];
+      vs[k] = to_float(proj[static_cast<size_t>(t0 + (k < count ? k : 0)) * ld + v_off + h * v_dim + col]);
     if (act) {
 #pragma unroll
       for (int k = 0; k < kRetBlock; ++k) vs[k] = silu_f(vs[k]);
@@ -461,10 +461,11 @@ extern "C" long long shk_retention_state_floats(int heads, int dim, int v_dim) {
   return static_cast<long long>(heads) * v_dim * dim;
 }
 
-extern "C" int shk_retention_scan(const float* proj, int ld, int q_off, int k_off, int v_off, const float* decay,
+extern "C" int shk_retention_scan(const void* proj, int dtype, int ld, int q_off, int k_off, int v_off, const float* decay,
                                   int num_seqs, int heads, int dim, int v_dim, const int32_t* positions,
                                   const int32_t* cu_q, const int32_t* slots, float* state, long long slot_stride,
                                   float* out, int act, void* stream) {
+  SHK_REQUIRE(dtype == kF32 || dtype == kBF16, "retention_scan: unknown dtype %d", dtype);
   SHK_REQUIRE(act == 0 || act == 1, "retention_scan: unknown activation %d (0: none, 1: SiLU)", act);
   SHK_REQUIRE(num_seqs >= 0 && heads > 0 && dim > 0 && dim <= 1024 && v_dim > 0,
               "retention_scan: bad sizes seqs=%d heads=%d dim=%d v_dim=%d", num_seqs, heads, dim, v_dim);
@@ -484,18 +485,27 @@ extern "C" int shk_retention_scan(const float* proj, int ld, int q_off, int k_of
               retention_heads_a_workgroup(lanes, heads, v_dim), dim);
   const int block = static_cast<int>(64000 / a_token) < kRetBlock ? static_cast<int>(64000 / a_token) : kRetBlock;
   const size_t lds = block * a_token;
-#define SHK_GO(L)                                                                                              \
-  retention_scan_kernel<L, (L == 64 ? 16 : kRowsPerLane)><<<dim3((units + 256 / L - 1) / (256 / L), num_seqs), 256, lds, s>>>(                \
-      proj, ld, q_off, k_off, v_off, decay, heads, dim, v_dim, positions, cu_q, slots, state, slot_stride, out, block, act)
-  switch (lanes) {
-    case 1: SHK_GO(1); break;
-    case 2: SHK_GO(2); break;
-    case 4: SHK_GO(4); break;
-    case 8: SHK_GO(8); break;
-    case 16: SHK_GO(16); break;
-    case 32: SHK_GO(32); break;
-    default: SHK_GO(64); break;
+#define SHK_GO(T, L)                                                                                             \
+  retention_scan_kernel<T, L, (L == 64 ? 16 : kRowsPerLane)>                                                    \
+      <<<dim3((units + 256 / L - 1) / (256 / L), num_seqs), 256, lds, s>>>(                                      \
+          static_cast<const T*>(proj), ld, q_off, k_off, v_off, decay, heads, dim, v_dim, positions, cu_q, slots, \
+          state, slot_stride, out, block, act)
+#define SHK_LANES(T)                                                                                             \
+  switch (lanes) {                                                                                               \
+    case 1: SHK_GO(T, 1); break;                                                                                 \
+    case 2: SHK_GO(T, 2); break;                                                                                 \
+    case 4: SHK_GO(T, 4); break;                                                                                 \
+    case 8: SHK_GO(T, 8); break;                                                                                 \
+    case 16: SHK_GO(T, 16); break;                                                                               \
+    case 32: SHK_GO(T, 32); break;                                                                               \
+    default: SHK_GO(T, 64); break;                                                                               \
   }
+  if (dtype == kF32) {
+    SHK_LANES(float)
+  } else {
+    SHK_LANES(bf16)
+  }
+#undef SHK_LANES
 #undef SHK_GO
   SHK_LAUNCH_CHECK("retention_scan");
   return 0;

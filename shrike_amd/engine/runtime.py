@@ -66,13 +66,16 @@ class Runtime:
         self.linear(x, w, gate_up)
         ops.act_mul(gate_up, out, activation, limit, up_shift)
 
-    def linear(self, x, w: LinearWeight, out, bias=None, accumulate=False, activation: str | None = None) -> None:
-        """out (+)= x @ w.T + bias; with `activation` ("relu_squared") out = act(x @ w.T + bias), in the
-        product's epilogue for bfloat16, by a kernel of its own for float32."""
+    def linear(self, x, w: LinearWeight, out, bias=None, accumulate=False, activation=None) -> None:
+        """out (+)= x @ w.T + bias; with `activation` "relu_squared" out = act(x @ w.T + bias), with
+        ("silu", r) the first r columns of out alone pass SiLU, in the product's epilogue for bfloat16, by a
+        kernel of its own for float32 ("relu_squared" only)."""
         if w.tiled is not None:
             ops.gemm_tiled_weight(x, w.tiled, w.rows, w.cols, out, bias=bias, accumulate=accumulate,
                                   activation=activation)
             return
+        if activation not in (None, "relu_squared"):
+            raise ValueError(f"activation {activation!r} is not built for float32 products")
         ops.gemm(x, w.dense, out, bias=bias, accumulate=accumulate)
         if activation is not None:
             ops.activate(out, out, activation)

@@ -58,7 +58,7 @@ _SIGNATURES = {
     "shk_latent_attention_bf16": [_P, _P, _I, _I, _I, _I, _P, _P, _P, _I, _P, _I, _I, _I, _I, _F, _P, _I, _I, _P],
     "shk_gemm_batched": [_P, _P, _P, _I, _I, _I, _I, _I, _I, c_longlong, c_longlong, c_longlong, _I, _P],
     "shk_mlstm_scan": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _F, _F, _I, _I, _I, _I, _P, _P, _P, _P, c_longlong, _P, _P],
-    "shk_headnorm_gate": [_P, _P, _I, _P, _F, _P, _I, _I, _I, _I, _I, _P],
+    "shk_headnorm_gate": [_P, _P, _I, _I, _P, _F, _P, _I, _I, _I, _I, _I, _P],
     "shk_add_layernorm": [_P, _P, _I, _P, _P, _F, _P, _P, _F, _P, _I, _I, _P, _I, _I, _I, _I, _P],
     "shk_mix_history": [_P, c_longlong, _P, _I, _P, _I, _I, _P, _I, _P, _P, _F, _I, _P],
     "shk_scale_softcap": [_P, c_longlong, _F, _F, _P],
@@ -71,7 +71,9 @@ _SIGNATURES = {
     "shk_selective_scan": [_P, _P, _P, _I, _I, _I, _P, _I, _P, _P, _I, _I, _I, _P, _I, _P, _P, _P, _P, c_longlong,
                            _P, _I, _I, _P],
     "shk_rotate_half_rows": [_P, _I, _I, _I, _I, _I, _P, _P, _F, _I, _P],
-    "shk_retention_scan": [_P, _I, _I, _I, _I, _P, _I, _I, _I, _I, _P, _P, _P, _P, c_longlong, _P, _I, _P],
+    "shk_retention_scan": [_P, _I, _I, _I, _I, _I, _P, _I, _I, _I, _I, _P, _P, _P, _P, c_longlong, _P, _I, _P],
+    "shk_retention_chunk_supports": [_I, _I],
+    "shk_retention_chunk_bf16": [_P, _I, _I, _I, _I, _P, _I, _I, _I, _I, _I, _P, _P, _P, _P, c_longlong, _P, _P],
     "shk_add_dynamic_tanh": [_P, _P, _I, _F, _F, _P, _P, _P, _I, _P, _I, _I, _I, _I, _P],
     "shk_conv_store": [_P, _I, _P, _I, _P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _P, _F, _I, _I, _I, _P, _P, _P, _P, _I, _P,
                        c_longlong, _P, _I, _I, _P, _P, _P, _P, _I, _I, _P],

@@ -395,7 +395,7 @@ def mfma_alone(operands: torch.Tensor, workgroups: int, iters: int) -> float:
 
 
 def gemm_tiled_weight(a, wt, m: int, k: int, out, bias=None, accumulate=False, gated=False,
-                      splits: int = 1, gate_args=None, activation: str | None = None) -> None:
+                      splits: int = 1, gate_args=None, activation=None) -> None:
     """out (+)= a @ w.T + bias with wt = retile_weight(w): up to 64 rows of a
     stream the weights once; more rows run the LDS-staged MFMA kernel (tiles of
     128 x 128 to 256 x 256, chosen by how many the product has).
@@ -403,11 +403,19 @@ def gemm_tiled_weight(a, wt, m: int, k: int, out, bias=None, accumulate=False, g
     gated: False, or the gate's activation (one of GATE_ACTIVATIONS; True is "silu") for
     an interleaved gate/up weight.  gate_args: float32 [2] on the device, (limit, up_shift) of
     such a gate: act(min(g, limit)) * (clamp(u, -limit, limit) + up_shift), limit 0: no bounds.
-    activation "relu_squared": max(v, 0)^2 of every result is stored (no gate, no accumulation,
-    no shares of k)."""
+    activation "relu_squared": max(v, 0)^2 of every result is stored, ("silu", r): SiLU of the first r
+    columns of out (no gate, no accumulation, no shares of k)."""
     _rows(a, "gemm a")
-    if activation is not None and (activation != "relu_squared" or gated or accumulate or splits > 1):
-        raise KernelError(f"gemm_tiled_weight: activation {activation!r} of a plain whole product must be 'relu_squared'")
+    epilogue = int(bool(accumulate))
+    if activation is not None:
+        if gated or accumulate or splits > 1:
+            raise KernelError("gemm_tiled_weight: only a plain whole product takes an activation")
+        if activation == "relu_squared":
+            epilogue = 2
+        elif isinstance(activation, tuple) and activation[0] == "silu" and 0 < activation[1] <= m:
+            epilogue = 4 * int(activation[1])
+        else:
+            raise KernelError(f"gemm_tiled_weight: unknown activation {activation!r}")
     n = a.shape[0]
     if a.shape[1] != k or a.dtype != torch.bfloat16:
         raise KernelError(f"gemm_tiled_weight: a must be bfloat16 [n, {k}], got {tuple(a.shape)}")
@@ -431,7 +439,7 @@ def gemm_tiled_weight(a, wt, m: int, k: int, out, bias=None, accumulate=False, g
             _dev(a, "a"), _dev(wt, "wt"),
             None if bias is None else _dev(bias, "bias", torch.float32),
             _dev(out, "out"), n, m, k, a.stride(0), out.stride(-2), dtype_code(out.dtype),
-            2 if activation else int(bool(accumulate)), activation_code(gated), int(splits), _stream(),
+            epilogue, activation_code(gated), int(splits), _stream(),
         )
     )
 
@@ -745,19 +753,20 @@ def mlstm_scan(proj, q_off, k_off, v_off, i_off, f_off, i_bias, f_bias, cap, q_s
 
 def headnorm_gate(o, gate, weight, eps, out, heads, v_dim, gate_act: str = "sigmoid") -> None:
     """out[t, h] = o[t, h] / rms(o[t, h]) * weight[h] * g(gate[t, h]); o float32 [n, heads * v_dim],
-    gate float32 rows (a view with a row stride is fine), out of the compute dtype.  weight
+    gate float32 rows or rows of out's dtype (a view with a row stride is fine), out of the compute dtype.  weight
     None: none; gate_act "sigmoid" or "silu"."""
     _rows(gate, "headnorm_gate gate")
     n = o.shape[0]
-    if o.dtype != torch.float32 or gate.dtype != torch.float32 or not o.is_contiguous() or not out.is_contiguous() \
+    if o.dtype != torch.float32 or gate.dtype not in (torch.float32, out.dtype) or not o.is_contiguous() or not out.is_contiguous() \
             or tuple(o.shape) != (n, heads * v_dim) or tuple(out.shape) != (n, heads * v_dim) \
             or gate.shape[0] != n or gate.shape[1] < heads * v_dim \
             or (weight is not None and weight.numel() != heads * v_dim):
-        raise KernelError("headnorm_gate: o, gate float32 [n, heads * v_dim], out alike in the compute dtype")
+        raise KernelError("headnorm_gate: o float32, gate float32 or of out's dtype, [n, heads * v_dim], out alike in "
+                          "the compute dtype")
     if gate_act not in ("sigmoid", "silu"):
         raise KernelError(f"headnorm_gate: unknown gate {gate_act!r}")
-    check(load().shk_headnorm_gate(_dev(o, "o"), _dev(gate, "gate"), gate.stride(0),
-                                   None if weight is None else _dev(weight, "weight", torch.float32), float(eps),
+    check(load().shk_headnorm_gate(_dev(o, "o"), _dev(gate, "gate"), dtype_code(gate.dtype),
+                                   gate.stride(0), None if weight is None else _dev(weight, "weight", torch.float32), float(eps),
                                    _dev(out, "out"), dtype_code(out.dtype), n, heads, v_dim,
                                    int(gate_act == "silu"), _stream()))
 
@@ -1017,24 +1026,49 @@ def retention_state_floats(heads: int, dim: int, v_dim: int) -> int:
 
 def retention_scan(proj, q_off, k_off, v_off, decay, num_seqs, heads, dim, v_dim, positions, cu_q, slots, state,
                    out, activation: str | None = None) -> None:
-    """S_t = decay S_(t-1) + k v^T, o = S^T q per head over the step's tokens; proj float32 rows,
-    out float32 [n, heads * v_dim]; activation "silu": of q, k and v."""
+    """S_t = decay S_(t-1) + k v^T, o = S^T q per head over the tokens of the step's first num_seqs
+    sequences; proj float32 or bfloat16 rows, out float32 [n, heads * v_dim]; activation "silu": of q, k
+    and v."""
     if activation not in (None, "silu"):
         raise KernelError(f"retention_scan: unknown activation {activation!r}")
     _rows(proj, "retention_scan proj")
     n = proj.shape[0]
-    if proj.dtype != torch.float32 or out.dtype != torch.float32 or tuple(out.shape) != (n, heads * v_dim) \
-            or not out.is_contiguous():
-        raise KernelError("retention_scan: proj and out must be float32, out contiguous [n, heads * v_dim]")
+    if out.dtype != torch.float32 or tuple(out.shape) != (n, heads * v_dim) or not out.is_contiguous():
+        raise KernelError("retention_scan: out must be contiguous float32 [n, heads * v_dim]")
     if decay.dtype != torch.float32 or decay.numel() != heads:
         raise KernelError("retention_scan: one float32 decay per head")
     _state2d(state, "retention_scan")
     if cu_q.shape[0] < num_seqs + 1 or slots.shape[0] < num_seqs:
         raise KernelError("retention_scan: cu_q / slots are shorter than the step's sequences")
     check(load().shk_retention_scan(
-        _dev(proj, "proj"), proj.stride(0), q_off, k_off, v_off, _dev(decay, "decay"), num_seqs, heads, dim, v_dim,
+        _dev(proj, "proj"), dtype_code(proj.dtype), proj.stride(0), q_off, k_off, v_off, _dev(decay, "decay"), num_seqs, heads,
+        dim, v_dim, _dev(positions, "positions", torch.int32), _dev(cu_q, "cu_q", torch.int32),
+        _dev(slots, "slots", torch.int32), _dev(state, "state"), state.stride(0), _dev(out, "out"),
+        int(activation == "silu"), _stream()))
+
+
+def retention_chunk_supports(dim: int, v_dim: int) -> bool:
+    return bool(load().shk_retention_chunk_supports(int(dim), int(v_dim)))
+
+
+def retention_chunk(proj, q_off, k_off, v_off, decay, first_seq, num_seqs, heads, dim, v_dim, positions, cu_q, slots,
+                    state, out) -> None:
+    """retention_scan for prompt portions over bfloat16 rows, in chunks on the matrix units: sequences
+    first_seq .. first_seq + num_seqs - 1 of the step."""
+    _rows(proj, "retention_chunk proj")
+    n = proj.shape[0]
+    if proj.dtype != torch.bfloat16 or out.dtype != torch.float32 or tuple(out.shape) != (n, heads * v_dim) \
+            or not out.is_contiguous():
+        raise KernelError("retention_chunk: proj bfloat16, out contiguous float32 [n, heads * v_dim]")
+    if decay.dtype != torch.float32 or decay.numel() != heads:
+        raise KernelError("retention_chunk: one float32 decay per head")
+    _state2d(state, "retention_chunk")
+    if cu_q.shape[0] < first_seq + num_seqs + 1 or slots.shape[0] < first_seq + num_seqs:
+        raise KernelError("retention_chunk: cu_q / slots are shorter than the step's sequences")
+    check(load().shk_retention_chunk_bf16(
+        _dev(proj, "proj"), proj.stride(0), q_off, k_off, v_off, _dev(decay, "decay"), first_seq, num_seqs, heads, dim, v_dim,
         _dev(positions, "positions", torch.int32), _dev(cu_q, "cu_q", torch.int32), _dev(slots, "slots", torch.int32),
-        _dev(state, "state"), state.stride(0), _dev(out, "out"), int(activation == "silu"), _stream()))
+        _dev(state, "state"), state.stride(0), _dev(out, "out"), _stream()))
 
 
 def moe_route(logits, correction, top: int, chosen, weights) -> None:

@@ -205,8 +205,9 @@ class DifferentialAttention(Mixer):
             return
         tiles = ops.diff_attention_tiles(h, hkv)
         small = ops.diff_attention_tiles(h, hkv, small=True)
-        # workgroups of half the size while all of them find room on the chip at once
-        if small and int((-(-portions // (QUERY_TILE * small))).sum()) * hkv <= 2 * compute_units():
+        # workgroups of half the size: for two maps wherever they hold the heads (their registers), for one
+        # while all of them find room on the chip at once
+        if small and (self.maps == 2 or int((-(-portions // (QUERY_TILE * small))).sum()) * hkv <= 2 * compute_units()):
             plan.small, tiles = True, small
         run = QUERY_TILE * tiles
         seqs, q0 = portion_runs(portions, shape.num_decode, run)

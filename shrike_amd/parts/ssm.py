@@ -93,8 +93,9 @@ register_mixer("selective_scan", SelectiveScan)
 
 
 class Retention(Mixer):
-    """One product yields queries, keys, values and the output gate of a token in float32; by the
-    spec SiLU is applied to the first three; queries and keys are rotated (the spec's position
+    """One product yields queries, keys, values and the output gate of a token, in float32 where
+    they enter the recurrence as projected, in the compute dtype where an activation comes
+    between (bfloat16: prompt portions then run in chunks on the matrix units); by the spec SiLU is applied to the first three; queries and keys are rotated (the spec's position
     encoding, applied to float32 rows) and the keys scaled; the scan carries S per head in the
     request's state slot (float32); the readout is brought to unit root mean square (per head, or
     the heads together), weighted, gated by SiLU or the sigmoid of the gate projection, and
@@ -154,6 +155,8 @@ class Retention(Mixer):
         qk, v = s.num_heads * s.head_dim, s.num_heads * s.value_dim
         self.offsets = {"q": 0, "k": qk, "v": 2 * qk, "g": 2 * qk + v}
         self.in_width = 2 * qk + 2 * v
+        self.chunked = bool(s.activation == "silu" and self.position is None and qk % 8 == 0 and v % 8 == 0
+                            and ops.retention_chunk_supports(s.head_dim, s.value_dim))
         self.decay = torch.tensor([float(d) for d in s.decay], dtype=torch.float32, device=runtime.device)
         self.w_o = runtime.weight(tensors[self._t("o")])
         self.norm_weight = tensors[self._t("norm")].contiguous() if s.norm_weight else None
@@ -166,8 +169,14 @@ class Retention(Mixer):
     def forward(self, ctx, x: torch.Tensor, cache):
         s, off = self.spec, self.offsets
         n = x.shape[0]
-        proj = ctx.buffer("retention_proj", (n, self.in_width), torch.float32)
-        self.linear(x, self.w_in, proj)
+        # (an activation stands between the projections and the recurrence: both have the compute dtype)
+        proj = ctx.buffer("retention_proj", (n, self.in_width), ctx.dtype if s.activation else torch.float32)
+        left = s.activation  # what the recurrence's kernels still have to apply
+        if s.activation and proj.dtype == torch.bfloat16:
+            self.linear(x, self.w_in, proj, activation=(s.activation, off["g"]))  # in the product's epilogue
+            left = None
+        else:
+            self.linear(x, self.w_in, proj)
         inv_freq, rot_dim = self.position.rotary_table() if self.position is not None else (None, 0)
         if rot_dim:
             ops.rotate_half_rows(proj, off["q"], s.num_heads, s.head_dim, rot_dim, inv_freq, ctx.positions, 1.0)
@@ -175,8 +184,16 @@ class Retention(Mixer):
             ops.rotate_half_rows(proj, off["k"], s.num_heads, s.head_dim, rot_dim, inv_freq, ctx.positions, self.key_scale)
         read = ctx.buffer("retention_read", (n, s.num_heads * s.value_dim), torch.float32)
         state = cache.state_padded if cache.state_padded is not None else cache.state
-        ops.retention_scan(proj, off["q"], off["k"], off["v"], self.decay, ctx.num_seqs, s.num_heads, s.head_dim,
-                           s.value_dim, ctx.positions, ctx.cu_q, ctx.state_slots, state, read, activation=s.activation)
+        sizes = (s.num_heads, s.head_dim, s.value_dim)
+        in_order = ctx.num_seqs  # sequences whose tokens are walked one by one
+        if self.chunked and proj.dtype == torch.bfloat16:
+            in_order = ctx.num_decode
+            if ctx.num_seqs > in_order:
+                ops.retention_chunk(proj, off["q"], off["k"], off["v"], self.decay, in_order, ctx.num_seqs - in_order, *sizes,
+                                    ctx.positions, ctx.cu_q, ctx.state_slots, state, read)
+        if in_order:
+            ops.retention_scan(proj, off["q"], off["k"], off["v"], self.decay, in_order, *sizes, ctx.positions, ctx.cu_q,
+                               ctx.state_slots, state, read, activation=left)
         gated = ctx.buffer("retention_gated", (n, s.num_heads * s.value_dim), ctx.dtype)
         heads, size = (s.num_heads, s.value_dim) if s.norm_heads else (1, s.num_heads * s.value_dim)
         ops.headnorm_gate(read, proj[:, off["g"]:], self.norm_weight, s.eps, gated, heads, size, gate_act=s.gate)
