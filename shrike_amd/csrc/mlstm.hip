@@ -192,7 +192,8 @@ __global__ void __launch_bounds__(256)
 }
 
 // The same for wide rows (many heads normed together): a workgroup of THREADS per (token, head), the row held
-// in registers between its mean square and its write.  Few rows take wide workgroups, many rows narrow ones.
+// in registers between its mean square and its write.  Few bfloat16 rows take wide workgroups; float32 rows
+// always the same ones (a row has one order of summation whatever the step holds).
 constexpr int kWideRow = 512;    // wider rows take a workgroup
 constexpr int kWideHeld = 4096;  // elements a workgroup holds; beyond that they are read again
 template <typename T, typename TG, int THREADS>
@@ -292,7 +293,7 @@ extern "C" int shk_headnorm_gate(const float* o, const void* gate, int gate_dtyp
   do {                                                                                                             \
     const TG* gp = static_cast<const TG*>(gate);                                                                   \
     T* op = static_cast<T*>(out);                                                                                  \
-    if (v_dim > kWideRow && units < 512)                                                                           \
+    if (v_dim > kWideRow && sizeof(T) == 2 && units < 512)                                                        \
       headnorm_gate_wide_kernel<T, TG, 1024><<<static_cast<unsigned>(units), 1024, 0, s>>>(o, gp, gate_ld, weight, \
                                                                                           eps, op, heads, v_dim, gate_act); \
     else if (v_dim > kWideRow)                                                                                     \
