@@ -81,7 +81,12 @@ PAGE_SIZES = {"A": 16, "B": 4, "C": 32}
 
 def make_model_dir(name: str, root=None, dtype: str = "float32", mode: str = "unit") -> Path:
     """Writes the tiny model `name` with seeded random weights (stored in `dtype`) into
-    `root` (or a fresh temporary folder) and returns the folder."""
+    `root` (or a fresh temporary folder) and returns the folder.  The last map's weight is drawn
+    around zero and the embedding is small beside what the layers add: else, the output matrix being
+    the embedding, every token's best successor would be itself, whatever the layers do."""
+    import torch
+    from safetensors.torch import load_file, save_file
+
     from shrike_amd.weights import write_model_folder
 
     if root is None:
@@ -89,4 +94,10 @@ def make_model_dir(name: str, root=None, dtype: str = "float32", mode: str = "un
     path = Path(root) / f"fozedra_{name}_{dtype}_{mode}"
     if not (path / "model.safetensors").is_file():
         write_model_folder(dict(CONFIGS[name]), path, seed=SEEDS[name], dtype=dtype, mode=mode)
+        tensors = load_file(str(path / "model.safetensors"))
+        last = tensors["final.norm"]
+        gen = torch.Generator().manual_seed(SEEDS[name])
+        tensors["final.norm"] = torch.randn(last.shape, generator=gen).to(last.dtype)
+        tensors["embed"] = tensors["embed"] * 0.25
+        save_file(tensors, str(path / "model.safetensors"))
     return path
