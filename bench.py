@@ -326,7 +326,7 @@ def kernel_breakdown(engine, steps: int = 3, before_step=None) -> dict:
              "attention_decode", "attention_prefill", "attention_prefill_shared", "argmax", "sample",
              "add_deltas", "add_normed_rmsnorm", "act_mul_rows", "add_rows", "embed_pairs", "qkv_store",
              "latent_prepare", "rotate_heads", "latent_attention", "latent_attention_mfma", "gemm_batched", "mlstm_scan", "headnorm_gate",
-             "xielu", "layernorm", "add_layernorm", "attention_talking", "attention_talking_mfma", "conv_silu", "dt_softplus", "selective_scan",
+             "xielu", "layernorm", "add_layernorm", "attention_talking", "attention_talking_mfma", "short_conv", "dt_softplus", "selective_scan",
              "rotate_half_rows", "retention_scan", "retention_chunk", "moe_route", "moe_experts", "mix_history", "scale_softcap",
              "postnorm", "cast_rows", "activate", "gate_mul", "add_dynamic_tanh", "conv_store", "diff_attention",
              "diff_attention_decode", "diff_attention_prefill"]

@@ -189,7 +189,8 @@ class LatentAttentionSpec:
     W_uv c (``value_dim``); score = (q_plain . k_plain + q_rot . k_rot) * scale.  The
     rotation turns neighbouring pairs (2i, 2i + 1) of the rotated part by position *
     rot_theta ** (-2i / rotated), for the first ``rotated`` elements of the part (None: all
-    of it; the rest pass unchanged).  Both norms are RMS norms with a weight and ``eps``.
+    of it; the rest pass unchanged); ``rot_scaling`` stretches the rates and multiplies cosine and
+    sine as RotarySpec.scaling does.  Both norms are RMS norms with a weight and ``eps``.
     ``window`` / ``chunk`` bound the keys as in AttentionSpec.  Only c and the rotated key
     part are cached.  ``output_gate``: the heads' outputs side by side are multiplied by
     sigmoid(W_g x) before the output matrix."""
@@ -209,6 +210,7 @@ class LatentAttentionSpec:
     names: Names = ()
     rotated: int | None = None
     output_gate: bool = False
+    rot_scaling: tuple | None = None
 
 
 @dataclass(frozen=True)
@@ -275,6 +277,42 @@ class RetentionSpec:
 
 
 @dataclass(frozen=True)
+class GatedLinearAttentionSpec:
+    """Linear attention with a decay per token, head and key channel.  q = W_q x * head_dim ** -0.5, k = W_k x
+    ([heads, head_dim]), v = W_v x ([heads, value_dim]); alpha = sigmoid(W_a2 (W_a1 x) + b) ** (1 / tau)
+    ([heads, head_dim]); S_t = diag(alpha_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t.  Each head's o is divided by
+    its root mean square (``eps``) and multiplied by a weight of value_dim that the heads share, the heads side
+    by side by SiLU of W_g x, then W_o.  Per request: S (float32).  ``decay_rank``: rows of W_a1 (None: as many
+    as the file's tensor has)."""
+
+    kind: ClassVar[str] = "gated_linear_attention"
+    num_heads: int
+    head_dim: int
+    value_dim: int
+    tau: float
+    eps: float
+    decay_rank: int | None = None
+    names: Names = ()
+
+
+@dataclass(frozen=True)
+class GatedRecurrenceSpec:
+    """Griffin's recurrent block with a real-gated linear recurrent unit.  y = gelu(W_y x + b) (tanh form), u =
+    a causal convolution per channel (``conv`` taps, the last meets the current token, with a bias, no
+    activation) of W_x x + b, both ``recurrent_width`` wide.  u in ``blocks`` equal parts: r and i are the sigmoids of two
+    square matrices per part (with biases) applied to it.  log a = -power * r * softplus(lam); S_t = a S_(t-1) +
+    sqrt(1 - a^2) i u; out = W_o (S * y).  Per request: S (float32) and the convolution's last conv - 1
+    inputs."""
+
+    kind: ClassVar[str] = "gated_recurrence"
+    recurrent_width: int
+    blocks: int
+    conv: int
+    power: float = 8.0
+    names: Names = ()
+
+
+@dataclass(frozen=True)
 class ParallelMixerSpec:
     """Several mixers side by side on the same input: ``branches`` = ((sub-name, mixer spec),
     ...).  Each output is brought to unit root mean square over the model width (``eps``) and
@@ -299,7 +337,12 @@ class MoESpec:
     added (None: none).  ``gated`` False: experts (the shared one too) are down(act(up x)) and
     have no gate matrix; their activation is then "relu_squared".  ``router_bias``: a learned
     number per expert is added to the logits (a tensor).  ``shared_gate``: the shared expert's
-    output is multiplied by sigmoid(w . x), one number per token (a tensor [1, width])."""
+    output is multiplied by sigmoid(w . x), one number per token (a tensor [1, width]).  ``limit`` /
+    ``up_shift``: the experts' two products are bounded and the second shifted as in SwiGLUSpec;
+    ``shared_limit`` bounds the shared expert's.  ``identity``: so many router outputs behind the experts'
+    are experts without matrices whose output is their input.  ``groups`` = (count, keep): the router's
+    outputs form `count` equal groups of neighbours, and only those of the `keep` groups with the largest
+    best choice score (score + correction) can be chosen.  ``router_scale`` multiplies the weights."""
 
     kind: ClassVar[str] = "moe"
     experts: int
@@ -312,6 +355,12 @@ class MoESpec:
     gated: bool = True
     router_bias: bool = False
     shared_gate: bool = False
+    limit: float | None = None
+    shared_limit: float | None = None
+    up_shift: float = 0.0
+    identity: int = 0
+    groups: tuple | None = None
+    router_scale: float = 1.0
 
 
 @dataclass(frozen=True)
@@ -422,6 +471,29 @@ class PostNormBlockSpec:
     mixer_norm: object
     ffn_norm: object = None
     alpha: float = 1.0
+    layer_scale: bool = False
+    mixer_name: str = "mix"
+    ffn_name: str = "mlp"
+    mixer_norm_name: str = "norm1"
+    ffn_norm_name: str = "norm2"
+    mixer_scale_name: str = "ls1"
+    ffn_scale_name: str = "ls2"
+
+
+@dataclass(frozen=True)
+class OutputNormBlockSpec:
+    """The norm stands on the sublayer's output alone: x += s1 * mixer_norm(mixer(x)); x += s2 *
+    ffn_norm(ffn(x)), the sublayers reading x as it stands.  ``layer_scale``: s1 and s2 are learned vectors of
+    the model's width (tensors ``mixer_scale_name`` / ``ffn_scale_name`` below the block's name); else ones.
+    ``ffn`` may be None: the layer then adds nothing there (a second norm and scale in the weight file are
+    allowed and without effect)."""
+
+    kind: ClassVar[str] = "output_norm_residual"
+    name: str
+    mixer: object
+    ffn: object
+    mixer_norm: object
+    ffn_norm: object
     layer_scale: bool = False
     mixer_name: str = "mix"
     ffn_name: str = "mlp"

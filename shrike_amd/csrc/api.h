@@ -47,7 +47,7 @@ int shk_add_deltas(float* resid, const void* d1, int splits1, const void* d2, in
 // A product's output that is normed by itself before it joins the stream:
 // x = resid[row] + delta[row] * rsqrt(mean(delta[row]^2) + deps) * dweight, stored back
 // with write_resid; with out != null, out[r] = x * rsqrt(mean(x^2) + eps) * weight as
-// well (the norm that follows).  delta / delta_splits / rows / resid_rows as in
+// well (the norm that follows; weight null: x itself).  delta / delta_splits / rows / resid_rows as in
 // shk_add_rmsnorm, except that delta has `dtype` or is float32 partial sums.
 int shk_add_normed_rmsnorm(float* resid, const void* delta, int delta_splits, const float* dweight,
                            float deps, const float* weight, float eps, void* out, int dtype,
@@ -251,18 +251,19 @@ int shk_attention_prefill_shared_bf16(const void* q, int q_stride, void* out, in
 // down[:, :q_rank] * rsqrt(mean^2 + eps) * q_weight; the token's row of `pool`
 // ([num_pages, page_size, kv_rank + rot_dim], page through tables as elsewhere) receives
 // the next kv_rank columns normed likewise with kv_weight, then the last rot_dim columns
-// with neighbouring pairs (2i, 2i + 1) turned by position * inv_freq[i].
+// with neighbouring pairs (2i, 2i + 1) turned by position * inv_freq[i], cosine and sine
+// multiplied by magnitude.
 int shk_latent_prepare(const void* down, int dtype, int n, int q_rank, int kv_rank, int rot_dim,
                        const float* q_weight, const float* kv_weight, float eps, const float* inv_freq,
-                       const int32_t* positions, const int32_t* token_seq, const int32_t* tables,
+                       float magnitude, const int32_t* positions, const int32_t* token_seq, const int32_t* tables,
                        int table_stride, void* q_latent, void* pool, int page_size, int num_pages,
                        int write_kv, void* stream);
 // dst[t, h * dst_head + dst_off + e] = the rotation of src[t, h * src_head + src_off + e],
-// e < rot_dim, pairs (2i, 2i + 1) turned by positions[t] * inv_freq[i]; rows src_row /
-// dst_row elements apart.
+// e < rot_dim, pairs (2i, 2i + 1) turned by positions[t] * inv_freq[i] (cosine and sine times
+// magnitude); rows src_row / dst_row elements apart.
 int shk_rotate_heads(const void* src, int src_row, int src_head, int src_off, void* dst, int dst_row,
                      int dst_head, int dst_off, int dtype, int n, int heads, int rot_dim,
-                     const float* inv_freq, const int32_t* positions, void* stream);
+                     const float* inv_freq, float magnitude, const int32_t* positions, void* stream);
 // q [n, heads, key_dim], out [n, heads, v_dim]: every head attends over the rows of the
 // token's sequence in `pool` ([num_pages, page_size, key_dim]); score = q . row * scale, the
 // values are the rows' first v_dim elements.  window / chunk as in shk_attention.
@@ -285,10 +286,11 @@ int shk_latent_attention_bf16(const void* q, void* out, int n, int heads, int ke
 
 // A batch of products of one shape: out_b[n, m] = a_b[n, k] @ w_b[m, k]^T for b < batch, with
 // a_b = a + b * a_batch (rows lda apart), w_b = w + b * w_batch (contiguous), out_b = out + b *
-// out_batch (rows ldo apart); all of `dtype`, float32 accumulation in ascending k.
+// out_batch (rows ldo apart); operands of `dtype`, out of out_dtype (the same or float32), float32
+// accumulation in ascending k.
 int shk_gemm_batched(const void* a, const void* w, void* out, int n, int m, int k, int lda, int ldo,
                      int batch, long long a_batch, long long w_batch, long long out_batch, int dtype,
-                     void* stream);
+                     int out_dtype, void* stream);
 
 // The mLSTM recurrence (mlstm.hip) for the tokens of a step.  proj [n, ld] float32 holds each
 // token's projections: queries at column q_off ([heads, dim]), keys at k_off, values at v_off
@@ -361,37 +363,51 @@ int shk_attention_talking_bf16(const void* q, int q_stride, void* out, int n, in
 
 // The selective scan of Mamba and its causal convolution (ssm.hip).  A request's slot holds S
 // [inner, states] float32 and then the convolution's last taps - 1 inputs [(taps - 1), inner].
-// shk_conv_silu: y[t, c] = silu(bias[c] + sum_k taps[c, num_taps - 1 - k] * x[t - k, c]) over the
-// sequence's earlier inputs (rows of this step, else the slot's kept ones, zero before position 0).
-// shk_dt_softplus: dt[t, c] = softplus(b[c] + sum_r w[r, c] * low[t, r]), float32; w [rank, inner].
+// shk_short_conv: y[t, c] = act(bias[c] + sum_k taps[c, num_taps - 1 - k] * x[t - k, c]), act SiLU with
+// `silu`, else nothing, over the sequence's earlier inputs (rows of this step, else the slot's kept ones,
+// zero before position 0).
+// shk_dt_softplus: dt[t, c] = mult * softplus(sign * (b[c] + sum_r w[r, c] * low[t, r])), float32; w [rank,
+// inner].
 // shk_selective_scan: S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n, y_c = sum_n S[c, n] C_n +
 // dskip_c x_c, out = y * silu(z); A = -exp(a_log); B and C are columns b_off, c_off of bc (float32);
 // `raw` are the convolution's inputs of the step, of which the slot keeps the last taps - 1.
 long long shk_selective_scan_state_floats(int inner, int states, int taps);
-int shk_conv_silu(const void* x, int ldx, const float* taps, const float* bias, int num_taps, int inner,
-                  const int32_t* positions, const int32_t* token_seq, const int32_t* cu_q,
-                  const int32_t* slots, const float* state, long long slot_stride, int states, void* y,
-                  int dtype, int n, void* stream);
+int shk_short_conv(const void* x, int ldx, const float* taps, const float* bias, int num_taps, int inner,
+                   const int32_t* positions, const int32_t* token_seq, const int32_t* cu_q,
+                   const int32_t* slots, const float* state, long long slot_stride, int states, int silu, void* y,
+                   int dtype, int n, void* stream);
 int shk_dt_softplus(const float* low, int ld, const float* w, const float* b, int rank, int inner,
-                    float* dt, int n, void* stream);
+                    float sign, float mult, float* dt, int n, void* stream);
 int shk_selective_scan(const float* dt, const void* x, const float* bc, int ld_bc, int b_off, int c_off,
                        const void* z, int ldz, const float* a_log, const float* dskip, int inner,
                        int states, int num_taps, const void* raw, int ld_raw, const int32_t* positions,
                        const int32_t* cu_q, const int32_t* slots, float* state, long long slot_stride,
                        void* out, int dtype, int num_seqs, void* stream);
 
-// Retention (ssm.hip): per head S_t = decay[h] S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, over
+// The real-gated linear recurrent unit (rglru.hip): S_t = a_t S_(t-1) + sqrt(1 - a_t^2) i_t u_t per channel, log
+// a = -rate r, out = S gelu(y), over the step's sequences, of which the first num_single have one token.  gates
+// (float32 [n, 2 * width]): the products before bias_r / bias_i and the sigmoid, block by block [r | i] of width
+// / blocks channels each.  u [n, width], y and raw rows ldy / ld_raw apart, all of `dtype`; a slot holds S
+// [width] and the last taps - 1 rows of raw (the convolution's inputs).
+long long shk_rglru_state_floats(int width, int taps);
+int shk_rglru(const float* gates, int blocks, const float* bias_r, const float* bias_i, const float* rate,
+              const void* u, const void* y, int ldy, const void* raw, int ld_raw, int width, int taps,
+              const int32_t* positions, const int32_t* cu_q, const int32_t* slots, float* state,
+              long long slot_stride, void* out, int dtype, int num_single, int num_seqs, void* stream);
+
+// Retention (ssm.hip): per head S_t = decay[h] S_(t-1) + k_t v_t^T, o_t = q_scale S_t^T q_t, over
 // projections (of `dtype`) at columns q_off, k_off ([heads, dim]) and v_off ([heads, v_dim]) of proj (act 1: SiLU
-// of each of them, 0: as they are); a slot
+// of each of them, 0: as they are); with log_decay (float32 [n, heads * dim]) in the place of decay, S_t =
+// diag(exp(log_decay_t)) S_(t-1) + k_t v_t^T (gated linear attention); a slot
 // holds S as [heads, v_dim, dim].  shk_rotate_half_rows turns the pairs (i, i + rot_dim / 2) of
 // every head of float32 rows in place by positions[t] * inv_freq[i] and multiplies the head by mult.
 long long shk_retention_state_floats(int heads, int dim, int v_dim);
 int shk_rotate_half_rows(float* x, int ld, int off, int heads, int dim, int rot_dim, const float* inv_freq,
                          const int32_t* positions, float mult, int n, void* stream);
 int shk_retention_scan(const void* proj, int dtype, int ld, int q_off, int k_off, int v_off, const float* decay,
-                       int num_seqs, int heads, int dim, int v_dim, const int32_t* positions,
-                       const int32_t* cu_q, const int32_t* slots, float* state, long long slot_stride,
-                       float* out, int act, void* stream);
+                       const float* log_decay, float q_scale, int num_seqs, int heads, int dim, int v_dim,
+                       const int32_t* positions, const int32_t* cu_q, const int32_t* slots, float* state,
+                       long long slot_stride, float* out, int act, void* stream);
 // The same for prompt portions over bfloat16 projections as they are, in chunks on the matrix units
 // (retention_chunk.hip), for sequences first_seq .. first_seq + num_seqs - 1; dim 32, 64, 96, 128, 192 or
 // 256, v_dim in multiples of 32, columns in runs of 8.  A float32 operand of a product enters as the sum
@@ -462,25 +478,31 @@ int shk_diff_attention_prefill_bf16(const void* q, void* out, int num_wgs, int h
 
 // A routed mixture of gated experts (moe.hip).  shk_moe_route: softmax over the experts' logits
 // (float32 [n, ld]); the `top` largest of score + correction (null: none) are chosen [n, top],
-// their weights [n, top] are their scores over the chosen ones' sum (+ 1e-20).
+// their weights [n, top] are their scores over the chosen ones' sum (+ 1e-20), times scale.  groups > 1:
+// experts form that many groups of neighbours, and only those of the `keep` groups with the largest best
+// choice score can be chosen.
 // shk_moe_experts: out[t] = add[t] (null: nothing) + sum_k weights[t, k] * W_down_e (act(W_gate_e
-// x_t) * (W_up_e x_t)), e = chosen[t, k]; matrices stacked row-major [experts, ff, width] and
-// [experts, width, ff]; act_buf [n * top, ff]; all of `dtype`; act 1 SiLU, 2 GELU (tanh form), 3 ReLU
+// x_t) * (W_up_e x_t + shift)), e = chosen[t, k]; limit > 0: the gate's product is bounded from above and the
+// other one from both sides first; e >= experts (up to experts + identity): x_t itself; matrices stacked row-major [experts, ff, width] and
+// [experts, width, ff]; act_buf [n * top, ff]; all of `dtype`; act 1 SiLU, 2 GELU (tanh form), 3 ReLU,
+// 4 g sigmoid(1.702 g)
 // (experts without a gate whose activation is the square of ReLU pass their one matrix as both).
 // add_gate (float32, one number per token, gate_ld apart; null: none): add[t] is multiplied by
 // sigmoid(add_gate[t * gate_ld]).
 int shk_moe_route(const float* logits, int ld, const float* correction, int experts, int top,
-                  int32_t* chosen, float* weights, int n, void* stream);
+                  int groups, int keep, float scale, int32_t* chosen, float* weights, int n, void* stream);
 int shk_moe_experts(const void* x, const int32_t* chosen, const float* weights, const void* w_gate,
                     const void* w_up, const void* w_down, const void* add, const float* add_gate, int gate_ld,
-                    void* act_buf, void* out, int dtype, int n, int width, int ff, int experts, int top, int act, void* stream);
+                    void* act_buf, void* out, int dtype, int n, int width, int ff, int experts, int top,
+                    int identity, int act, float limit, float shift, void* stream);
 // The same for bfloat16 on the matrix units, expert by expert over the lists of the (token,
 // expert) pairs that chose it (built on the device).  width and ff in multiples of 8; scratch:
 // shk_moe_grouped_scratch_bytes(...) bytes, 16-byte aligned.
 long long shk_moe_grouped_scratch_bytes(int n, int width, int experts, int top);
 int shk_moe_experts_grouped(const void* x, const int32_t* chosen, const float* weights, const void* w_gate,
                             const void* w_up, const void* w_down, const void* add, const float* add_gate,
-                            int gate_ld, void* act_buf, void* out, void* scratch, int n, int width, int ff, int experts, int top, int act, void* stream);
+                            int gate_ld, void* act_buf, void* out, void* scratch, int n, int width, int ff, int experts, int top,
+                            int identity, int act, float limit, float shift, void* stream);
 
 // out = a_pos z^2 + z / 2 where z > 0, a_neg (exp(z) - 1 - z) + z / 2 elsewhere; elementwise.
 int shk_xielu(const void* x, void* out, int dtype, long long numel, float a_pos, float a_neg, void* stream);

@@ -85,10 +85,11 @@ const Launcher kLaunchers[] = {
     SHK_LAUNCHER(shk_scale_softcap),
     SHK_LAUNCHER(shk_attention_talking),
     SHK_LAUNCHER(shk_attention_talking_bf16),
-    SHK_LAUNCHER(shk_conv_silu),
+    SHK_LAUNCHER(shk_short_conv),
     SHK_LAUNCHER(shk_dt_softplus),
     SHK_LAUNCHER(shk_selective_scan),
     SHK_LAUNCHER(shk_rotate_half_rows),
+    SHK_LAUNCHER(shk_rglru),
     SHK_LAUNCHER(shk_retention_scan),
     SHK_LAUNCHER(shk_retention_chunk_bf16),
     SHK_LAUNCHER(shk_add_dynamic_tanh),

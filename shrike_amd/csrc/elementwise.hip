@@ -297,7 +297,8 @@ __global__ void __launch_bounds__(THREADS)
 // x = resid[row] + delta[row] * rsqrt(mean(delta[row]^2) + deps) * dweight: a product's
 // output that is normed by itself before it joins the stream.  With write_resid the sum
 // is stored back; with `out`, out[r] = x * rsqrt(mean(x^2) + eps) * weight follows in the
-// same pass (the next layer's norm).  rows: as in add_rmsnorm.
+// same pass (the next layer's norm), or x itself where `weight` is absent (a layer that reads
+// the stream as it stands).  rows: as in add_rmsnorm.
 template <typename T, int V, int THREADS, int S>
 __global__ void __launch_bounds__(THREADS)
     add_normed_rmsnorm_kernel(float* __restrict__ resid, const void* __restrict__ delta, int splits,
@@ -318,7 +319,7 @@ __global__ void __launch_bounds__(THREADS)
     if (c < nvec) {
       x[i] = row_load<V>(resid + row * hidden + c * V);
       dw[i] = row_load<V>(dweight + c * V);
-      if (out) w[i] = row_load<V>(weight + c * V);
+      if (weight) w[i] = row_load<V>(weight + c * V);
     }
   }
   row_gather<V, THREADS, S, T>(delta, splits, split_stride, row, hidden, d);
@@ -340,8 +341,9 @@ __global__ void __launch_bounds__(THREADS)
       xx += x[i].v[e] * x[i].v[e];
     }
     if (write_resid) row_store<V>(resid + row * hidden + c * V, x[i]);
+    if (out && !weight) row_store<V>(out + static_cast<size_t>(r) * hidden + c * V, x[i]);
   }
-  if (!out) return;
+  if (!out || !weight) return;
   xx = block_sum(xx, scratch);
   const float inv = rsqrtf(xx / static_cast<float>(hidden) + eps);
 #pragma unroll
@@ -606,9 +608,9 @@ extern "C" int shk_add_normed_rmsnorm(float* resid, const void* delta, int delta
   SHK_REQUIRE(dtype == kF32 || dtype == kBF16, "add_normed_rmsnorm: unknown dtype %d", dtype);
   SHK_REQUIRE(n >= 0 && hidden > 0 && delta_splits >= 0 && resid_rows >= 0,
               "add_normed_rmsnorm: bad sizes n=%d hidden=%d", n, hidden);
-  SHK_REQUIRE(deps > 0.f && (!out || eps > 0.f), "add_normed_rmsnorm: eps must be > 0");
+  SHK_REQUIRE(deps > 0.f && (!weight || eps > 0.f), "add_normed_rmsnorm: eps must be > 0");
   if (n == 0) return 0;
-  SHK_REQUIRE(resid && delta && dweight && (!out || weight), "add_normed_rmsnorm: null pointer");
+  SHK_REQUIRE(resid && delta && dweight && (out || !weight), "add_normed_rmsnorm: null pointer");
   SHK_REQUIRE(out || write_resid, "add_normed_rmsnorm: nothing to write");
   const int form = row_form(hidden, aligned16(resid) && aligned16(delta) && aligned16(dweight) &&
                                         aligned16(weight) && aligned16(out));

@@ -78,9 +78,9 @@ __global__ void __launch_bounds__(256)
 // kernel's few workgroups would each walk a long k alone.
 constexpr int kSkinnyRows = 16;
 
-template <typename T>
+template <typename T, typename TO>
 __global__ void __launch_bounds__(256)
-    gemm_batched_skinny_kernel(const T* __restrict__ a, const T* __restrict__ w, T* __restrict__ out, int n,
+    gemm_batched_skinny_kernel(const T* __restrict__ a, const T* __restrict__ w, TO* __restrict__ out, int n,
                                int m, int k, int lda, int ldo, long long a_batch, long long w_batch,
                                long long out_batch) {
   const int lane = threadIdx.x % kWave;
@@ -102,7 +102,7 @@ __global__ void __launch_bounds__(256)
 #pragma unroll
     for (int r = 0; r < kSkinnyRows; ++r) {
       const float total = wave_sum(acc[r]);
-      if (lane == 0 && n0 + r < n) out[b * out_batch + static_cast<size_t>(n0 + r) * ldo + row] = from_float<T>(total);
+      if (lane == 0 && n0 + r < n) out[b * out_batch + static_cast<size_t>(n0 + r) * ldo + row] = from_float<TO>(total);
     }
   }
 }
@@ -156,8 +156,9 @@ extern "C" int shk_gemm(const void* a, const void* w, const float* bias, void* o
 typedef __bf16 gbf16x8 __attribute__((ext_vector_type(8)));
 typedef float gf32x4 __attribute__((ext_vector_type(4)));
 
+template <typename TO>
 __global__ void __launch_bounds__(256)
-    gemm_batched_mfma_kernel(const bf16* __restrict__ a, const bf16* __restrict__ w, bf16* __restrict__ out, int n,
+    gemm_batched_mfma_kernel(const bf16* __restrict__ a, const bf16* __restrict__ w, TO* __restrict__ out, int n,
                              int m, int k, int lda, int ldo, long long a_batch, long long w_batch,
                              long long out_batch) {
   const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
@@ -192,13 +193,13 @@ __global__ void __launch_bounds__(256)
   // the products were formed transposed (features as rows): this lane holds features 4 kg + r of tile t for row i
   const int orow = (blockIdx.y * 4 + wave) * 16 + i;
   if (orow >= n) return;
-  bf16* dst = out + b * out_batch + static_cast<size_t>(orow) * ldo;
+  TO* dst = out + b * out_batch + static_cast<size_t>(orow) * ldo;
 #pragma unroll
   for (int t = 0; t < 4; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int c = col0 + t * 16 + 4 * kg + r;
-      if (c < m) dst[c] = from_float<bf16>(acc[t][r]);
+      if (c < m) dst[c] = from_float<TO>(acc[t][r]);
     }
 }
 
@@ -206,8 +207,9 @@ __global__ void __launch_bounds__(256)
 // (rows lda apart), w + b * w_batch ([m, k] contiguous) and writes out + b * out_batch.
 extern "C" int shk_gemm_batched(const void* a, const void* w, void* out, int n, int m, int k, int lda,
                                 int ldo, int batch, long long a_batch, long long w_batch,
-                                long long out_batch, int dtype, void* stream) {
+                                long long out_batch, int dtype, int out_dtype, void* stream) {
   SHK_REQUIRE(dtype == kF32 || dtype == kBF16, "gemm_batched: unknown dtype %d", dtype);
+  SHK_REQUIRE(out_dtype == dtype || out_dtype == kF32, "gemm_batched: outputs are of the operands' dtype or float32");
   SHK_REQUIRE(n >= 0 && m > 0 && k > 0 && batch > 0 && batch <= 65535, "gemm_batched: bad sizes n=%d m=%d k=%d batch=%d",
               n, m, k, batch);
   SHK_REQUIRE(lda >= k && ldo >= m, "gemm_batched: row strides lda=%d ldo=%d too small for k=%d m=%d", lda, ldo, k, m);
@@ -219,21 +221,29 @@ extern "C" int shk_gemm_batched(const void* a, const void* w, void* out, int n, 
   if (dtype == kBF16 && k % 8 == 0 && lda % 8 == 0 && a_batch % 8 == 0 && reinterpret_cast<uintptr_t>(a) % 16 == 0 &&
       reinterpret_cast<uintptr_t>(w) % 16 == 0 && (n + 63) / 64 <= 65535) {
     dim3 grid((m + 63) / 64, (n + 63) / 64, batch);
-    gemm_batched_mfma_kernel<<<grid, 256, 0, s>>>(static_cast<const bf16*>(a), static_cast<const bf16*>(w),
-                                                  static_cast<bf16*>(out), n, m, k, lda, ldo, a_batch, w_batch, out_batch);
+    if (out_dtype == kF32)
+      gemm_batched_mfma_kernel<float><<<grid, 256, 0, s>>>(static_cast<const bf16*>(a), static_cast<const bf16*>(w),
+                                                           static_cast<float*>(out), n, m, k, lda, ldo, a_batch, w_batch,
+                                                           out_batch);
+    else
+      gemm_batched_mfma_kernel<bf16><<<grid, 256, 0, s>>>(static_cast<const bf16*>(a), static_cast<const bf16*>(w),
+                                                          static_cast<bf16*>(out), n, m, k, lda, ldo, a_batch, w_batch,
+                                                          out_batch);
   } else if (n <= 2 * kSkinnyRows && dtype == kBF16) {
     // (float32 keeps one order of summation whatever the number of rows: the tiled kernel's ascending k)
     dim3 grid((m + 3) / 4, batch);
-    if (dtype == kF32)
-      gemm_batched_skinny_kernel<float><<<grid, 256, 0, s>>>(static_cast<const float*>(a), static_cast<const float*>(w),
-                                                             static_cast<float*>(out), n, m, k, lda, ldo, a_batch,
-                                                             w_batch, out_batch);
+    if (out_dtype == kF32)
+      gemm_batched_skinny_kernel<bf16, float><<<grid, 256, 0, s>>>(static_cast<const bf16*>(a), static_cast<const bf16*>(w),
+                                                                   static_cast<float*>(out), n, m, k, lda, ldo, a_batch,
+                                                                   w_batch, out_batch);
     else
-      gemm_batched_skinny_kernel<bf16><<<grid, 256, 0, s>>>(static_cast<const bf16*>(a), static_cast<const bf16*>(w),
-                                                            static_cast<bf16*>(out), n, m, k, lda, ldo, a_batch,
-                                                            w_batch, out_batch);
+      gemm_batched_skinny_kernel<bf16, bf16><<<grid, 256, 0, s>>>(static_cast<const bf16*>(a), static_cast<const bf16*>(w),
+                                                                  static_cast<bf16*>(out), n, m, k, lda, ldo, a_batch,
+                                                                  w_batch, out_batch);
   } else if (dtype == kF32)
     launch_tiled<float, float>(a, w, nullptr, out, n, m, k, lda, ldo, 0, s, batch, a_batch, w_batch, out_batch);
+  else if (out_dtype == kF32)
+    launch_tiled<bf16, float>(a, w, nullptr, out, n, m, k, lda, ldo, 0, s, batch, a_batch, w_batch, out_batch);
   else
     launch_tiled<bf16, bf16>(a, w, nullptr, out, n, m, k, lda, ldo, 0, s, batch, a_batch, w_batch, out_batch);
   SHK_LAUNCH_CHECK("gemm_batched");

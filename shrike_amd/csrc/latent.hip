@@ -7,7 +7,8 @@
 //
 // latent_prepare_kernel: from the joint down-projection of a token, [q latent |
 // key/value latent | rotated key part]: RMS norm of the two latents (float32, each
-// with its weight), rotation of the key part (neighbouring pairs, float32 angles),
+// with its weight), rotation of the key part (neighbouring pairs, float32 angles, cosine
+// and sine times `magnitude`),
 // the query latent to a buffer and the key row to its page slot.
 // rotate_heads_kernel: rotation of a slice of every head of a row, from one buffer
 // into another (the queries' rotated parts, into the folded queries' rows).
@@ -23,19 +24,20 @@ constexpr int kLatThreads = 256;
 constexpr int kMaxKeyDim = 1024;   // latent + rotated part
 constexpr int kMaxPerThread = 4;   // value elements per thread: latents up to 1024
 
-__device__ __forceinline__ void turn(float angle, float* c, float* s) {
+__device__ __forceinline__ void turn(float angle, float magnitude, float* c, float* s) {
   // angles reach thousands of radians: into [-pi, pi] in float64 before the float32 sine and cosine
   const double a = static_cast<double>(angle);
   const double turns = rint(a * 0.15915494309189535);
   const float reduced = static_cast<float>(fma(turns, -6.283185307179586, a));
   sincosf(reduced, s, c);
+  *s *= magnitude, *c *= magnitude;
 }
 
 template <typename T>
 __global__ void __launch_bounds__(kLatThreads)
     latent_prepare_kernel(const T* __restrict__ down, int q_rank, int kv_rank, int rot_dim,
                           const float* __restrict__ q_weight, const float* __restrict__ kv_weight, float eps,
-                          const float* __restrict__ inv_freq, const int32_t* __restrict__ positions,
+                          const float* __restrict__ inv_freq, float magnitude, const int32_t* __restrict__ positions,
                           const int32_t* __restrict__ token_seq, const int32_t* __restrict__ tables,
                           int table_stride, T* __restrict__ q_latent, T* __restrict__ pool, int page_size,
                           int num_pages, int write_kv) {
@@ -64,7 +66,7 @@ __global__ void __launch_bounds__(kLatThreads)
     dst[i] = from_float<T>(to_float(row[q_rank + i]) * rkv * kv_weight[i]);
   for (int i = threadIdx.x; i < rot_dim / 2; i += kLatThreads) {
     float c, s;
-    turn(static_cast<float>(pos) * inv_freq[i], &c, &s);
+    turn(static_cast<float>(pos) * inv_freq[i], magnitude, &c, &s);
     const float u = to_float(row[q_rank + kv_rank + 2 * i]), v = to_float(row[q_rank + kv_rank + 2 * i + 1]);
     dst[kv_rank + 2 * i] = from_float<T>(u * c - v * s);
     dst[kv_rank + 2 * i + 1] = from_float<T>(v * c + u * s);
@@ -75,7 +77,7 @@ __global__ void __launch_bounds__(kLatThreads)
 template <typename T>
 __global__ void rotate_heads_kernel(const T* __restrict__ src, int src_row, int src_head, int src_off,
                                     T* __restrict__ dst, int dst_row, int dst_head, int dst_off, int heads,
-                                    int rot_dim, const float* __restrict__ inv_freq,
+                                    int rot_dim, const float* __restrict__ inv_freq, float magnitude,
                                     const int32_t* __restrict__ positions) {
   const int t = blockIdx.x;
   const float pos = static_cast<float>(positions[t]);
@@ -83,7 +85,7 @@ __global__ void rotate_heads_kernel(const T* __restrict__ src, int src_row, int 
   for (int item = threadIdx.x; item < heads * half; item += blockDim.x) {
     const int h = item / half, i = item % half;
     float c, s;
-    turn(pos * inv_freq[i], &c, &s);
+    turn(pos * inv_freq[i], magnitude, &c, &s);
     const T* a = src + static_cast<size_t>(t) * src_row + h * src_head + src_off + 2 * i;
     T* b = dst + static_cast<size_t>(t) * dst_row + h * dst_head + dst_off + 2 * i;
     const float u = to_float(a[0]), v = to_float(a[1]);
@@ -187,7 +189,7 @@ using namespace shk;
 
 extern "C" int shk_latent_prepare(const void* down, int dtype, int n, int q_rank, int kv_rank, int rot_dim,
                                   const float* q_weight, const float* kv_weight, float eps, const float* inv_freq,
-                                  const int32_t* positions, const int32_t* token_seq, const int32_t* tables,
+                                  float magnitude, const int32_t* positions, const int32_t* token_seq, const int32_t* tables,
                                   int table_stride, void* q_latent, void* pool, int page_size, int num_pages,
                                   int write_kv, void* stream) {
   SHK_REQUIRE(dtype == kF32 || dtype == kBF16, "latent_prepare: unknown dtype %d", dtype);
@@ -206,12 +208,12 @@ extern "C" int shk_latent_prepare(const void* down, int dtype, int n, int q_rank
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (dtype == kF32)
     latent_prepare_kernel<float><<<n, kLatThreads, 0, s>>>(
-        static_cast<const float*>(down), q_rank, kv_rank, rot_dim, q_weight, kv_weight, eps, inv_freq, positions,
+        static_cast<const float*>(down), q_rank, kv_rank, rot_dim, q_weight, kv_weight, eps, inv_freq, magnitude, positions,
         token_seq, tables, table_stride, static_cast<float*>(q_latent), static_cast<float*>(pool), page_size,
         num_pages, write_kv);
   else
     latent_prepare_kernel<bf16><<<n, kLatThreads, 0, s>>>(
-        static_cast<const bf16*>(down), q_rank, kv_rank, rot_dim, q_weight, kv_weight, eps, inv_freq, positions,
+        static_cast<const bf16*>(down), q_rank, kv_rank, rot_dim, q_weight, kv_weight, eps, inv_freq, magnitude, positions,
         token_seq, tables, table_stride, static_cast<bf16*>(q_latent), static_cast<bf16*>(pool), page_size,
         num_pages, write_kv);
   SHK_LAUNCH_CHECK("latent_prepare");
@@ -220,7 +222,7 @@ extern "C" int shk_latent_prepare(const void* down, int dtype, int n, int q_rank
 
 extern "C" int shk_rotate_heads(const void* src, int src_row, int src_head, int src_off, void* dst, int dst_row,
                                 int dst_head, int dst_off, int dtype, int n, int heads, int rot_dim,
-                                const float* inv_freq, const int32_t* positions, void* stream) {
+                                const float* inv_freq, float magnitude, const int32_t* positions, void* stream) {
   SHK_REQUIRE(dtype == kF32 || dtype == kBF16, "rotate_heads: unknown dtype %d", dtype);
   SHK_REQUIRE(n >= 0 && heads > 0 && rot_dim >= 0 && rot_dim % 2 == 0, "rotate_heads: bad sizes n=%d heads=%d rot_dim=%d",
               n, heads, rot_dim);
@@ -235,11 +237,11 @@ extern "C" int shk_rotate_heads(const void* src, int src_row, int src_head, int 
   if (dtype == kF32)
     rotate_heads_kernel<float><<<n, threads, 0, s>>>(static_cast<const float*>(src), src_row, src_head, src_off,
                                                      static_cast<float*>(dst), dst_row, dst_head, dst_off, heads,
-                                                     rot_dim, inv_freq, positions);
+                                                     rot_dim, inv_freq, magnitude, positions);
   else
     rotate_heads_kernel<bf16><<<n, threads, 0, s>>>(static_cast<const bf16*>(src), src_row, src_head, src_off,
                                                     static_cast<bf16*>(dst), dst_row, dst_head, dst_off, heads,
-                                                    rot_dim, inv_freq, positions);
+                                                    rot_dim, inv_freq, magnitude, positions);
   SHK_LAUNCH_CHECK("rotate_heads");
   return 0;
 }

@@ -1,10 +1,14 @@
 // A routed mixture of gated feed-forward experts.
 //
 //   scores s = softmax(router logits) over all experts (float32);
-//   the `top` experts with the largest s + correction are chosen (the lowest index wins a tie);
-//   their weights are their s divided by the chosen experts' sum (+ 1e-20);
-//   out = sum over the chosen of weight * W_down_e (act(W_gate_e x) * (W_up_e x))  (+ what a
-//   shared expert gave, times sigmoid of a number per token where the design gates it).
+//   the `top` experts with the largest s + correction are chosen (the lowest index wins a tie),
+//   where the experts form groups only from those of the `keep` groups (of neighbours, of equal
+//   size) whose largest s + correction is largest;
+//   their weights are their s divided by the chosen experts' sum (+ 1e-20), times `scale`;
+//   out = sum over the chosen of weight * W_down_e (act(W_gate_e x) * (W_up_e x + shift))  (+ what a
+//   shared expert gave, times sigmoid of a number per token where the design gates it); with a
+//   limit the gate's product is bounded from above and the other one from both sides first.
+//   Router outputs from `experts` on are identity experts: they have no matrices, their output is x.
 //   Experts without a gate whose activation is the square of ReLU are the same with ReLU as act and
 //   their one matrix in both places: relu(u) * u; the kernels then form that product once.
 //
@@ -31,7 +35,8 @@ constexpr int kMaxExpertsPerLane = 8;  // experts <= 512
 
 __global__ void __launch_bounds__(256)
     moe_route_kernel(const float* __restrict__ logits, int ld, const float* __restrict__ correction, int experts,
-                     int top, int32_t* __restrict__ chosen, float* __restrict__ weights, int n) {
+                     int top, int groups, int keep, float scale, int32_t* __restrict__ chosen,
+                     float* __restrict__ weights, int n) {
   const int t = blockIdx.x * (256 / kWave) + threadIdx.x / kWave;
   const int lane = threadIdx.x % kWave;
   if (t >= n) return;
@@ -57,6 +62,34 @@ __global__ void __launch_bounds__(256)
     const int e = lane + i * kWave;
     s[i] /= sum;
     c[i] = e < experts ? s[i] + (correction ? correction[e] : 0.f) : -INFINITY;
+  }
+  if (keep < groups) {
+    // lane g keeps the best choice score of group g; the `keep` best groups stay, of equal ones the lowest
+    const int size = experts / groups;
+    float group_best = -INFINITY;
+    for (int g = 0; g < groups; ++g) {
+      float b = -INFINITY;
+#pragma unroll
+      for (int i = 0; i < kMaxExpertsPerLane; ++i) {
+        const int e = lane + i * kWave;
+        if (e >= g * size && e < (g + 1) * size) b = fmaxf(b, c[i]);
+      }
+      b = wave_max(b);
+      if (lane == g) group_best = b;
+    }
+    unsigned long long kept = 0;
+    for (int k = 0; k < keep; ++k) {
+      const bool open = lane < groups && !((kept >> lane) & 1ull);
+      const float best = wave_max(open ? group_best : -INFINITY);
+      unsigned long long at = __ballot(open && group_best == best);
+      if (at == 0) at = __ballot(open);  // (scores that are not numbers: the lowest group left)
+      kept |= at & (~at + 1ull);
+    }
+#pragma unroll
+    for (int i = 0; i < kMaxExpertsPerLane; ++i) {
+      const int e = lane + i * kWave;
+      if (e < experts && !((kept >> (e / size)) & 1ull)) c[i] = -INFINITY;
+    }
   }
   float picked_sum = 0.f, my_score = 0.f;
   int my_expert = 0;
@@ -114,14 +147,30 @@ __global__ void __launch_bounds__(256)
   }
   if (lane < top) {
     chosen[static_cast<size_t>(t) * top + lane] = my_expert;
-    weights[static_cast<size_t>(t) * top + lane] = my_score / (picked_sum + 1e-20f);
+    weights[static_cast<size_t>(t) * top + lane] = my_score / (picked_sum + 1e-20f) * scale;
   }
 }
 
+// What joins an expert's two products: the gate's activation, the bound (0: none), what is added to the
+// other factor.
+struct GateForm {
+  int act;
+  float limit, shift;
+};
+
 __device__ __forceinline__ float gate_act(float g, int act) {
   if (act == 3) return fmaxf(g, 0.f);  // ReLU; with the gate's matrix also the other factor's, the square of ReLU
+  if (act == 4) return g / (1.f + expf(-1.702f * g));
   const float x = act == 2 ? 2.f * 0.7978845608028654f * (g + 0.044715f * g * g * g) : g;
   return g / (1.f + expf(-x));
+}
+
+__device__ __forceinline__ float gate_times_up(float g, float u, GateForm form) {
+  if (form.limit > 0.f) {
+    g = fminf(g, form.limit);
+    u = fminf(fmaxf(u, -form.limit), form.limit);
+  }
+  return gate_act(g, form.act) * (u + form.shift);
 }
 
 // What multiplies the shared expert's output for token t: sigmoid(add_gate[t * gate_ld]), one number
@@ -135,11 +184,12 @@ constexpr int kMoeFeatures = 32;  // features (or columns) a workgroup
 template <typename T>
 __global__ void __launch_bounds__(256)
     moe_gate_up_kernel(const T* __restrict__ x, const int32_t* __restrict__ chosen, const T* __restrict__ wg,
-                       const T* __restrict__ wu, T* __restrict__ act_out, int width, int ff, int top, int act,
+                       const T* __restrict__ wu, T* __restrict__ act_out, int width, int ff, int top, GateForm form,
                        int experts) {
   extern __shared__ float xs[];
   const int pair = blockIdx.y, t = pair / top;
-  const int e = min(max(chosen[pair], 0), experts - 1);  // an index from memory never leaves the stack of experts
+  const int e = max(chosen[pair], 0);
+  if (e >= experts) return;  // an identity expert (an index from memory never leaves the stack of experts)
   for (int k = threadIdx.x; k < width; k += 256) xs[k] = to_float(x[static_cast<size_t>(t) * width + k]);
   __syncthreads();
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
@@ -160,13 +210,13 @@ __global__ void __launch_bounds__(256)
       g = wave_sum(g);
       u = wave_sum(u);
     }
-    if (lane == 0) act_out[static_cast<size_t>(pair) * ff + f] = from_float<T>(gate_act(g, act) * u);
+    if (lane == 0) act_out[static_cast<size_t>(pair) * ff + f] = from_float<T>(gate_times_up(g, u, form));
   }
 }
 
 template <typename T>
 __global__ void __launch_bounds__(256)
-    moe_down_kernel(const T* __restrict__ act_in, const int32_t* __restrict__ chosen,
+    moe_down_kernel(const T* __restrict__ x, const T* __restrict__ act_in, const int32_t* __restrict__ chosen,
                     const float* __restrict__ weights, const T* __restrict__ wd, const T* __restrict__ add,
                     const float* __restrict__ add_gate, int gate_ld, T* __restrict__ out, int width, int ff, int top,
                     int experts) {
@@ -180,7 +230,11 @@ __global__ void __launch_bounds__(256)
     if (c >= width) break;
     float total = 0.f;
     for (int k = 0; k < top; ++k) {
-      const int e = min(max(chosen[static_cast<size_t>(t) * top + k], 0), experts - 1);
+      const int e = max(chosen[static_cast<size_t>(t) * top + k], 0);
+      if (e >= experts) {  // an identity expert
+        total = fmaf(weights[static_cast<size_t>(t) * top + k], to_float(x[static_cast<size_t>(t) * width + c]), total);
+        continue;
+      }
       const T* dr = wd + (static_cast<size_t>(e) * width + c) * ff;
       float d = 0.f;
       for (int f = lane; f < ff; f += kWave) d = fmaf(to_float(dr[f]), as[k * ff + f], d);
@@ -233,7 +287,7 @@ __global__ void __launch_bounds__(256)
     moe_gate_up_mfma_kernel(const bf16* __restrict__ x, const int32_t* __restrict__ order,
                             const int32_t* __restrict__ counts, const bf16* __restrict__ wg,
                             const bf16* __restrict__ wu, bf16* __restrict__ act_out, int n, int width, int ff, int top,
-                            int act) {
+                            GateForm form) {
   const int e = blockIdx.z;
   const int count = min(counts[e], n);
   const int row0 = blockIdx.y * 32;
@@ -325,7 +379,7 @@ __global__ void __launch_bounds__(256)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int f = f0 + b * 16 + 4 * kg + r;
-        if (f < ff) dst[f] = from_float<bf16>(gate_act(accg[a][b][r], act) * (single ? accg[a][b][r] : accu[a][b][r]));
+        if (f < ff) dst[f] = from_float<bf16>(gate_times_up(accg[a][b][r], single ? accg[a][b][r] : accu[a][b][r], form));
       }
   }
 }
@@ -425,7 +479,7 @@ template <bool GATED, bool SINGLE = false>
 __global__ void __launch_bounds__(256)
     moe_tiled_mfma_kernel(const bf16* __restrict__ a, const int32_t* __restrict__ order,
                           const int32_t* __restrict__ counts, const bf16* __restrict__ w0, const bf16* __restrict__ w1,
-                          bf16* __restrict__ act_out, float* __restrict__ pair_out, int n, int k, int m, int top, int act) {
+                          bf16* __restrict__ act_out, float* __restrict__ pair_out, int n, int k, int m, int top, GateForm form) {
   __shared__ __attribute__((aligned(16))) uint16_t sa[2][kTileRows * kTileLd];
   __shared__ __attribute__((aligned(16))) uint16_t sb[2][kTileRows * kTileLd];
   const int e = blockIdx.z;
@@ -514,7 +568,7 @@ __global__ void __launch_bounds__(256)
         const int f = blockIdx.x * 128 + wn * 64 + bn * 16 + 4 * kg;
 #pragma unroll
         for (int q = 0; q < 4; ++q)
-          if (f + q < m) dst[f + q] = from_float<bf16>(gate_act(acc[am][bn][q], act) * acc[am][bn][q]);
+          if (f + q < m) dst[f + q] = from_float<bf16>(gate_times_up(acc[am][bn][q], acc[am][bn][q], form));
       }
     } else if (GATED) {
       bf16* dst = act_out + static_cast<size_t>(pair) * m;
@@ -523,7 +577,7 @@ __global__ void __launch_bounds__(256)
         const int f = blockIdx.x * 64 + wn * 32 + bn * 16 + 4 * kg;
 #pragma unroll
         for (int q = 0; q < 4; ++q)
-          if (f + q < m) dst[f + q] = from_float<bf16>(gate_act(acc[am][bn][q], act) * acc[am][bn + 2][q]);
+          if (f + q < m) dst[f + q] = from_float<bf16>(gate_times_up(acc[am][bn][q], acc[am][bn + 2][q], form));
       }
     } else {
       float* dst = pair_out + static_cast<size_t>(pair) * m;
@@ -542,16 +596,21 @@ __global__ void __launch_bounds__(256)
   }
 }
 
-// out[t, c] = add[t, c] + sum_k weights[t, k] * pair_out[t * top + k, c], k in the order chosen
+// out[t, c] = add[t, c] + sum_k weights[t, k] * pair_out[t * top + k, c], k in the order chosen; an identity
+// expert's output is x[t, c]
 __global__ void __launch_bounds__(256)
-    moe_join_kernel(const float* __restrict__ pair_out, const float* __restrict__ weights, const bf16* __restrict__ add,
-                    const float* __restrict__ add_gate, int gate_ld, bf16* __restrict__ out, int width, int top) {
+    moe_join_kernel(const float* __restrict__ pair_out, const int32_t* __restrict__ chosen, const bf16* __restrict__ x,
+                    const float* __restrict__ weights, const bf16* __restrict__ add, const float* __restrict__ add_gate,
+                    int gate_ld, bf16* __restrict__ out, int width, int top, int experts) {
   const int t = blockIdx.y;
   const int c = blockIdx.x * blockDim.x + threadIdx.x;
   if (c >= width) return;
   float total = 0.f;
-  for (int k = 0; k < top; ++k)
-    total = fmaf(weights[static_cast<size_t>(t) * top + k], pair_out[(static_cast<size_t>(t) * top + k) * width + c], total);
+  for (int k = 0; k < top; ++k) {
+    const size_t pair = static_cast<size_t>(t) * top + k;
+    const float y = chosen[pair] < experts ? pair_out[pair * width + c] : to_float(x[static_cast<size_t>(t) * width + c]);
+    total = fmaf(weights[pair], y, total);
+  }
   if (add) total += shared_share(add_gate, gate_ld, t) * to_float(add[static_cast<size_t>(t) * width + c]);
   out[static_cast<size_t>(t) * width + c] = from_float<bf16>(total);
 }
@@ -561,25 +620,29 @@ __global__ void __launch_bounds__(256)
 using namespace shk;
 
 extern "C" int shk_moe_route(const float* logits, int ld, const float* correction, int experts, int top,
-                             int32_t* chosen, float* weights, int n, void* stream) {
+                             int groups, int keep, float scale, int32_t* chosen, float* weights, int n, void* stream) {
   SHK_REQUIRE(n >= 0 && experts > 0 && experts <= kMaxExpertsPerLane * kWave && top >= 1 && top <= experts &&
                   top <= kWave && ld >= experts,
               "moe_route: bad sizes n=%d experts=%d top=%d", n, experts, top);
+  SHK_REQUIRE(groups >= 1 && groups <= kWave && experts % groups == 0 && keep >= 1 && keep <= groups &&
+                  top <= keep * (experts / groups),
+              "moe_route: %d of %d experts cannot be chosen from %d of %d groups", top, experts, keep, groups);
   if (n == 0) return 0;
   SHK_REQUIRE(logits && chosen && weights, "moe_route: null pointer");
   moe_route_kernel<<<(n + 3) / 4, 256, 0, static_cast<hipStream_t>(stream)>>>(logits, ld, correction, experts, top,
-                                                                              chosen, weights, n);
+                                                                              groups, keep, scale, chosen, weights, n);
   SHK_LAUNCH_CHECK("moe_route");
   return 0;
 }
 
 extern "C" int shk_moe_experts(const void* x, const int32_t* chosen, const float* weights, const void* w_gate,
                                const void* w_up, const void* w_down, const void* add, const float* add_gate,
-                               int gate_ld, void* act_buf, void* out, int dtype, int n, int width, int ff, int experts, int top, int act, void* stream) {
+                               int gate_ld, void* act_buf, void* out, int dtype, int n, int width, int ff, int experts, int top,
+                               int identity, int act, float limit, float shift, void* stream) {
   SHK_REQUIRE(dtype == kF32 || dtype == kBF16, "moe_experts: unknown dtype %d", dtype);
-  SHK_REQUIRE(n >= 0 && width > 0 && ff > 0 && experts > 0 && top >= 1 && top <= experts,
+  SHK_REQUIRE(n >= 0 && width > 0 && ff > 0 && experts > 0 && identity >= 0 && top >= 1 && top <= experts + identity,
               "moe_experts: bad sizes n=%d width=%d ff=%d experts=%d top=%d", n, width, ff, experts, top);
-  SHK_REQUIRE(act >= 1 && act <= 3, "moe_experts: unknown activation %d", act);
+  SHK_REQUIRE(act >= 1 && act <= 4, "moe_experts: unknown activation %d", act);
   SHK_REQUIRE(!add_gate || (add && gate_ld >= 1), "moe_experts: a gate of the added rows needs those rows and a stride");
   SHK_REQUIRE(width <= 15000 && static_cast<long long>(top) * ff <= 15000,
               "moe_experts: rows of %d, or %d chosen experts of %d features, do not fit a workgroup's LDS", width, top,
@@ -588,14 +651,16 @@ extern "C" int shk_moe_experts(const void* x, const int32_t* chosen, const float
   SHK_REQUIRE(static_cast<long long>(n) * top <= 65535, "moe_experts: at most 65535 (token, expert) pairs a call");
   SHK_REQUIRE(x && chosen && weights && w_gate && w_up && w_down && act_buf && out, "moe_experts: null pointer");
   hipStream_t s = static_cast<hipStream_t>(stream);
+  const GateForm form{act, limit, shift};
   const dim3 g1((ff + kMoeFeatures - 1) / kMoeFeatures, n * top), g2((width + kMoeFeatures - 1) / kMoeFeatures, n);
 #define SHK_GO(T)                                                                                                     \
   moe_gate_up_kernel<T><<<g1, 256, width * sizeof(float), s>>>(static_cast<const T*>(x), chosen,                      \
                                                                static_cast<const T*>(w_gate),                         \
                                                                static_cast<const T*>(w_up), static_cast<T*>(act_buf), \
-                                                               width, ff, top, act, experts);                         \
+                                                               width, ff, top, form, experts);                        \
   moe_down_kernel<T><<<g2, 256, static_cast<size_t>(top) * ff * sizeof(float), s>>>(                                  \
-      static_cast<const T*>(act_buf), chosen, weights, static_cast<const T*>(w_down), static_cast<const T*>(add),     \
+      static_cast<const T*>(x), static_cast<const T*>(act_buf), chosen, weights, static_cast<const T*>(w_down),       \
+      static_cast<const T*>(add),                                                                                     \
       add_gate, gate_ld, static_cast<T*>(out), width, ff, top, experts)
   if (dtype == kF32) {
     SHK_GO(float);
@@ -615,11 +680,11 @@ extern "C" long long shk_moe_grouped_scratch_bytes(int n, int width, int experts
 
 extern "C" int shk_moe_experts_grouped(const void* x, const int32_t* chosen, const float* weights, const void* w_gate,
                                        const void* w_up, const void* w_down, const void* add, const float* add_gate,
-                                       int gate_ld, void* act_buf, void* out, void* scratch, int n, int width, int ff, int experts, int top, int act,
-                                       void* stream) {
-  SHK_REQUIRE(n >= 0 && width > 0 && ff > 0 && experts > 0 && experts <= 65535 && top >= 1 && top <= experts,
+                                       int gate_ld, void* act_buf, void* out, void* scratch, int n, int width, int ff, int experts, int top,
+                                       int identity, int act, float limit, float shift, void* stream) {
+  SHK_REQUIRE(n >= 0 && width > 0 && ff > 0 && experts > 0 && experts <= 65535 && identity >= 0 && top >= 1 && top <= experts + identity,
               "moe_experts_grouped: bad sizes n=%d width=%d ff=%d experts=%d top=%d", n, width, ff, experts, top);
-  SHK_REQUIRE(act >= 1 && act <= 3, "moe_experts_grouped: unknown activation %d", act);
+  SHK_REQUIRE(act >= 1 && act <= 4, "moe_experts_grouped: unknown activation %d", act);
   SHK_REQUIRE(!add_gate || (add && gate_ld >= 1),
               "moe_experts_grouped: a gate of the added rows needs those rows and a stride");
   SHK_REQUIRE(width % 8 == 0 && ff % 8 == 0, "moe_experts_grouped: width %d and ff %d must be multiples of 8", width, ff);
@@ -631,6 +696,7 @@ extern "C" int shk_moe_experts_grouped(const void* x, const int32_t* chosen, con
   for (const void* p : {x, w_gate, w_up, w_down, static_cast<const void*>(act_buf), static_cast<const void*>(scratch)})
     SHK_REQUIRE(reinterpret_cast<uintptr_t>(p) % 16 == 0, "moe_experts_grouped: operands must be 16-byte aligned");
   hipStream_t s = static_cast<hipStream_t>(stream);
+  const GateForm form{act, limit, shift};
   int32_t* order = static_cast<int32_t*>(scratch);
   int32_t* counts = order + static_cast<size_t>(experts) * n;
   const long long ints = static_cast<long long>(experts) * n + experts;
@@ -642,24 +708,25 @@ extern "C" int shk_moe_experts_grouped(const void* x, const int32_t* chosen, con
     if (w_gate == w_up)
       moe_tiled_mfma_kernel<true, true><<<dim3((ff + 127) / 128, row_tiles, experts), 256, 0, s>>>(
           static_cast<const bf16*>(x), order, counts, static_cast<const bf16*>(w_gate), static_cast<const bf16*>(w_up),
-          static_cast<bf16*>(act_buf), nullptr, n, width, ff, top, act);
+          static_cast<bf16*>(act_buf), nullptr, n, width, ff, top, form);
     else
       moe_tiled_mfma_kernel<true><<<dim3((ff + 63) / 64, row_tiles, experts), 256, 0, s>>>(
           static_cast<const bf16*>(x), order, counts, static_cast<const bf16*>(w_gate), static_cast<const bf16*>(w_up),
-          static_cast<bf16*>(act_buf), nullptr, n, width, ff, top, act);
+          static_cast<bf16*>(act_buf), nullptr, n, width, ff, top, form);
     moe_tiled_mfma_kernel<false><<<dim3((width + 127) / 128, row_tiles, experts), 256, 0, s>>>(
         static_cast<const bf16*>(act_buf), order, counts, static_cast<const bf16*>(w_down), nullptr, nullptr, pair_out, n,
-        ff, width, top, act);
+        ff, width, top, form);
   } else {
     const int row_tiles = (n + 31) / 32;
     moe_gate_up_mfma_kernel<<<dim3((ff + 127) / 128, row_tiles, experts), 256, 0, s>>>(
         static_cast<const bf16*>(x), order, counts, static_cast<const bf16*>(w_gate), static_cast<const bf16*>(w_up),
-        static_cast<bf16*>(act_buf), n, width, ff, top, act);
+        static_cast<bf16*>(act_buf), n, width, ff, top, form);
     moe_down_mfma_kernel<<<dim3((width + 255) / 256, row_tiles, experts), 256, 0, s>>>(
         static_cast<const bf16*>(act_buf), order, counts, static_cast<const bf16*>(w_down), pair_out, n, width, ff, top);
   }
-  moe_join_kernel<<<dim3((width + 255) / 256, n), 256, 0, s>>>(pair_out, weights, static_cast<const bf16*>(add), add_gate,
-                                                               gate_ld, static_cast<bf16*>(out), width, top);
+  moe_join_kernel<<<dim3((width + 255) / 256, n), 256, 0, s>>>(pair_out, chosen, static_cast<const bf16*>(x), weights,
+                                                               static_cast<const bf16*>(add), add_gate, gate_ld,
+                                                               static_cast<bf16*>(out), width, top, experts);
   SHK_LAUNCH_CHECK("moe_experts_grouped");
   return 0;
 }

@@ -1,6 +1,6 @@
 // Recurrent mixers whose state is a fixed-size tensor per request: the selective
 // scan of Mamba (with its short causal convolution) and retention (linear
-// attention with a fixed decay per head).  A sequence's tokens of the step are
+// attention with a fixed decay per head, or one per token and key channel).  A sequence's tokens of the step are
 // walked in order, whether they are a prompt's portion or one decoded token, so
 // a position's result does not depend on how the prompt was cut.  All state and
 // everything in the recurrences is float32.  A state is taken as zero where the
@@ -14,7 +14,8 @@
 // inputs [(taps - 1), inner], oldest first.
 //
 // Retention, per head:  S_t = decay S_(t-1) + k_t v_t^T;  o_t = S_t^T q_t, q, k and v as projected or
-// with SiLU applied to each.
+// with SiLU applied to each; gated linear attention is the same with a decay per token and key channel,
+// S_t = diag(exp(g_t)) S_(t-1) + k_t v_t^T.
 // A request's slot holds S as [heads, v_dim, dim].
 #include "api.h"
 #include "common.h"
@@ -43,16 +44,16 @@ __device__ __forceinline__ float group_sum(float v) {
 }
 __device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
-// y[t, c] = silu(bias[c] + sum_k taps[c, K - 1 - k] * x(t - k, c)): x(t - k) is a row of this
+// y[t, c] = act(bias[c] + sum_k taps[c, K - 1 - k] * x(t - k, c)), act SiLU or nothing: x(t - k) is a row of this
 // step where the sequence's portion reaches that far back, else the slot's kept input of
 // that position, else (before the sequence's start) zero.
 template <typename T>
 __global__ void __launch_bounds__(256)
-    conv_silu_kernel(const T* __restrict__ x, int ldx, const float* __restrict__ taps, const float* __restrict__ bias,
+    short_conv_kernel(const T* __restrict__ x, int ldx, const float* __restrict__ taps, const float* __restrict__ bias,
                      int K, int inner, const int32_t* __restrict__ positions, const int32_t* __restrict__ token_seq,
                      const int32_t* __restrict__ cu_q, const int32_t* __restrict__ slots,
                      const float* __restrict__ state, long long slot_stride, long long tail_off,
-                     T* __restrict__ y) {
+                     T* __restrict__ y, int silu) {
   const int t = blockIdx.y;
   const int c = blockIdx.x * blockDim.x + threadIdx.x;
   if (c >= inner) return;
@@ -76,18 +77,19 @@ __global__ void __launch_bounds__(256)
     }
     acc = fmaf(taps[c * K + (K - 1 - k)], v, acc);
   }
-  y[static_cast<size_t>(t) * inner + c] = from_float<T>(silu_f(acc));
+  y[static_cast<size_t>(t) * inner + c] = from_float<T>(silu ? silu_f(acc) : acc);
 }
 
 constexpr int kDtTokens = 8;  // tokens a workgroup where a step has many: the matrix is read once for all of them
 
-// dt[t, c] = softplus(b[c] + sum_r W[r, c] * low[t, r]) in float32; W is given transposed, [rank, inner], so
+// dt[t, c] = mult * softplus(sign * (b[c] + sum_r W[r, c] * low[t, r])) in float32 (sign and mult -1: the logarithm
+// of a sigmoid); W is given transposed, [rank, inner], so
 // that neighbouring channels' weights are neighbours in memory.  A token's sum runs over r in ascending
 // order whatever else is in the step.
 template <int kDtTokens>
 __global__ void __launch_bounds__(256)
     dt_softplus_kernel(const float* __restrict__ low, int ld, const float* __restrict__ wt, const float* __restrict__ b,
-                       int rank, int inner, float* __restrict__ dt, int n) {
+                       int rank, int inner, float sign, float mult, float* __restrict__ dt, int n) {
   extern __shared__ float lows[];  // [kDtTokens, rank]
   const int t0 = blockIdx.y * kDtTokens;
   const int count = min(kDtTokens, n - t0);
@@ -113,7 +115,7 @@ __global__ void __launch_bounds__(256)
   }
 #pragma unroll
   for (int k = 0; k < kDtTokens; ++k)
-    if (k < count) dt[static_cast<size_t>(t0 + k) * inner + c] = softplus_f(acc[k]);
+    if (k < count) dt[static_cast<size_t>(t0 + k) * inner + c] = mult * softplus_f(sign * acc[k]);
 }
 
 constexpr int kStatesPerLane = 4;  // (8 where a channel has more than 256 states)
@@ -256,18 +258,19 @@ inline int retention_heads_a_workgroup(int lanes, int heads, int v_dim) {
 }
 
 // One sequence's tokens for one (head, value column); LANES lanes share the column's rows
-// of S (LANES * 8 >= dim).
-template <typename T, int LANES, int kRowsPerLane>
+// of S (LANES * 8 >= dim).  GATED: log_decay [n, heads * dim] holds the decays' logarithms, token by token.
+template <typename T, int LANES, int kRowsPerLane, bool GATED>
 __global__ void __launch_bounds__(256)
     retention_scan_kernel(const T* __restrict__ proj, int ld, int q_off, int k_off, int v_off,
-                          const float* __restrict__ decay, int heads, int dim, int v_dim,
-                          const int32_t* __restrict__ positions, const int32_t* __restrict__ cu_q,
+                          const float* __restrict__ decay, const float* __restrict__ log_decay, float q_scale,
+                          int heads, int dim, int v_dim, const int32_t* __restrict__ positions, const int32_t* __restrict__ cu_q,
                           const int32_t* __restrict__ slots, float* __restrict__ state, long long slot_stride,
                           float* __restrict__ out, int block, int act) {
   // Tokens go by in blocks of `block` (at most kRetBlock): the queries and keys of the heads that this workgroup's columns
-  // belong to are staged in LDS by the workgroup ([token][head][q | k]), a lane fetches its column's
+  // belong to are staged in LDS by the workgroup ([token][head][q | k], GATED [q | k | decay]), a lane fetches its column's
   // values of the block at once: the walk waits for memory once a block.
   extern __shared__ float qks[];
+  constexpr int kParts = GATED ? 3 : 2;
   const int seq = blockIdx.y;
   const int per_wg = 256 / LANES;
   const int unit_raw = blockIdx.x * per_wg + threadIdx.x / LANES;  // (head, column)
@@ -289,16 +292,21 @@ __global__ void __launch_bounds__(256)
     const int d = part * kRowsPerLane + i;
     S[i] = (d < dim && !fresh) ? srow[d] : 0.f;
   }
-  const float a = decay[h];
+  const float a = GATED ? 0.f : decay[h];
   for (int t0 = first; t0 < last; t0 += block) {
     const int count = min(block, last - t0);
     __syncthreads();
-    for (int i = threadIdx.x; i < count * nh * 2 * dim; i += 256) {
-      const int tt = i / (nh * 2 * dim), rest = i % (nh * 2 * dim);
-      const int hh = rest / (2 * dim), j = rest % (2 * dim);
+    for (int i = threadIdx.x; i < count * nh * kParts * dim; i += 256) {
+      const int tt = i / (nh * kParts * dim), rest = i % (nh * kParts * dim);
+      const int hh = rest / (kParts * dim), j = rest % (kParts * dim);
+      if (GATED && j >= 2 * dim) {
+        const float g = log_decay[(static_cast<size_t>(t0 + tt) * heads + h_lo + hh) * dim + j - 2 * dim];
+        qks[i] = sizeof(T) == 2 ? __expf(g) : expf(g);
+        continue;
+      }
       const T* row = proj + static_cast<size_t>(t0 + tt) * ld;
       const float x = to_float(j < dim ? row[q_off + (h_lo + hh) * dim + j] : row[k_off + (h_lo + hh) * dim + j - dim]);
-      qks[i] = act ? silu_f(x) : x;
+      qks[i] = (act ? silu_f(x) : x) * (j < dim ? q_scale : 1.f);
     }
     float vs[kRetBlock];
 #pragma unroll
@@ -312,7 +320,7 @@ __global__ void __launch_bounds__(256)
 #pragma unroll
     for (int k = 0; k < kRetBlock; ++k) {
       if (k >= count) break;
-      const float* qt = qks + (static_cast<size_t>(k) * nh + (h - h_lo)) * 2 * dim;
+      const float* qt = qks + (static_cast<size_t>(k) * nh + (h - h_lo)) * kParts * dim;
       const float* kt = qt + dim;
       const float vv = vs[k];
       float o = 0.f;
@@ -320,7 +328,7 @@ __global__ void __launch_bounds__(256)
       for (int i = 0; i < kRowsPerLane; ++i) {
         const int d = part * kRowsPerLane + i;
         if (d < dim) {
-          S[i] = fmaf(a, S[i], kt[d] * vv);
+          S[i] = fmaf(GATED ? kt[dim + d] : a, S[i], kt[d] * vv);
           o = fmaf(S[i], qt[d], o);
         }
       }
@@ -350,35 +358,35 @@ extern "C" long long shk_selective_scan_state_floats(int inner, int states, int 
   return static_cast<long long>(inner) * states + static_cast<long long>(taps > 1 ? taps - 1 : 0) * inner;
 }
 
-extern "C" int shk_conv_silu(const void* x, int ldx, const float* taps, const float* bias, int num_taps, int inner,
+extern "C" int shk_short_conv(const void* x, int ldx, const float* taps, const float* bias, int num_taps, int inner,
                              const int32_t* positions, const int32_t* token_seq, const int32_t* cu_q,
-                             const int32_t* slots, const float* state, long long slot_stride, int states, void* y,
-                             int dtype, int n, void* stream) {
-  SHK_REQUIRE(dtype == kF32 || dtype == kBF16, "conv_silu: unknown dtype %d", dtype);
+                             const int32_t* slots, const float* state, long long slot_stride, int states, int silu,
+                              void* y, int dtype, int n, void* stream) {
+  SHK_REQUIRE(dtype == kF32 || dtype == kBF16, "short_conv: unknown dtype %d", dtype);
   SHK_REQUIRE(n >= 0 && inner > 0 && num_taps >= 1 && num_taps <= 64 && ldx >= inner && states > 0,
-              "conv_silu: bad sizes n=%d inner=%d taps=%d", n, inner, num_taps);
+              "short_conv: bad sizes n=%d inner=%d taps=%d", n, inner, num_taps);
   SHK_REQUIRE(slot_stride >= shk_selective_scan_state_floats(inner, states, num_taps),
-              "conv_silu: a slot of %lld floats does not hold the state", slot_stride);
+              "short_conv: a slot of %lld floats does not hold the state", slot_stride);
   if (n == 0) return 0;
-  SHK_REQUIRE(n <= 65535, "conv_silu: at most 65535 tokens a call, got %d", n);
-  SHK_REQUIRE(x && taps && bias && positions && token_seq && cu_q && slots && state && y, "conv_silu: null pointer");
+  SHK_REQUIRE(n <= 65535, "short_conv: at most 65535 tokens a call, got %d", n);
+  SHK_REQUIRE(x && taps && bias && positions && token_seq && cu_q && slots && state && y, "short_conv: null pointer");
   hipStream_t s = static_cast<hipStream_t>(stream);
   dim3 grid((inner + 255) / 256, n);
   const long long tail_off = static_cast<long long>(inner) * states;
   if (dtype == kF32)
-    conv_silu_kernel<float><<<grid, 256, 0, s>>>(static_cast<const float*>(x), ldx, taps, bias, num_taps, inner,
+    short_conv_kernel<float><<<grid, 256, 0, s>>>(static_cast<const float*>(x), ldx, taps, bias, num_taps, inner,
                                                  positions, token_seq, cu_q, slots, state, slot_stride, tail_off,
-                                                 static_cast<float*>(y));
+                                                 static_cast<float*>(y), silu);
   else
-    conv_silu_kernel<bf16><<<grid, 256, 0, s>>>(static_cast<const bf16*>(x), ldx, taps, bias, num_taps, inner,
+    short_conv_kernel<bf16><<<grid, 256, 0, s>>>(static_cast<const bf16*>(x), ldx, taps, bias, num_taps, inner,
                                                 positions, token_seq, cu_q, slots, state, slot_stride, tail_off,
-                                                static_cast<bf16*>(y));
-  SHK_LAUNCH_CHECK("conv_silu");
+                                                static_cast<bf16*>(y), silu);
+  SHK_LAUNCH_CHECK("short_conv");
   return 0;
 }
 
 extern "C" int shk_dt_softplus(const float* low, int ld, const float* w, const float* b, int rank, int inner,
-                               float* dt, int n, void* stream) {
+                               float sign, float mult, float* dt, int n, void* stream) {
   SHK_REQUIRE(n >= 0 && inner > 0 && rank > 0 && rank <= 1024 && ld >= rank, "dt_softplus: bad sizes n=%d inner=%d rank=%d",
               n, inner, rank);
   if (n == 0) return 0;
@@ -387,11 +395,11 @@ extern "C" int shk_dt_softplus(const float* low, int ld, const float* w, const f
     // few tokens: a wavefront per (64 channels, token), so that the launch has workgroups enough
     SHK_REQUIRE(n <= 65535, "dt_softplus: bad n");
     dt_softplus_kernel<1><<<dim3((inner + 63) / 64, n), 64, rank * sizeof(float), static_cast<hipStream_t>(stream)>>>(
-        low, ld, w, b, rank, inner, dt, n);
+        low, ld, w, b, rank, inner, sign, mult, dt, n);
   } else {
     dim3 grid((inner + 255) / 256, (n + kDtTokens - 1) / kDtTokens);
     dt_softplus_kernel<kDtTokens><<<grid, 256, kDtTokens * rank * sizeof(float), static_cast<hipStream_t>(stream)>>>(
-        low, ld, w, b, rank, inner, dt, n);
+        low, ld, w, b, rank, inner, sign, mult, dt, n);
   }
   SHK_LAUNCH_CHECK("dt_softplus");
   return 0;
@@ -462,9 +470,9 @@ extern "C" long long shk_retention_state_floats(int heads, int dim, int v_dim) {
 }
 
 extern "C" int shk_retention_scan(const void* proj, int dtype, int ld, int q_off, int k_off, int v_off, const float* decay,
-                                  int num_seqs, int heads, int dim, int v_dim, const int32_t* positions,
-                                  const int32_t* cu_q, const int32_t* slots, float* state, long long slot_stride,
-                                  float* out, int act, void* stream) {
+                                  const float* log_decay, float q_scale, int num_seqs, int heads, int dim, int v_dim,
+                                  const int32_t* positions, const int32_t* cu_q, const int32_t* slots, float* state,
+                                  long long slot_stride, float* out, int act, void* stream) {
   SHK_REQUIRE(dtype == kF32 || dtype == kBF16, "retention_scan: unknown dtype %d", dtype);
   SHK_REQUIRE(act == 0 || act == 1, "retention_scan: unknown activation %d (0: none, 1: SiLU)", act);
   SHK_REQUIRE(num_seqs >= 0 && heads > 0 && dim > 0 && dim <= 1024 && v_dim > 0,
@@ -476,19 +484,23 @@ extern "C" int shk_retention_scan(const void* proj, int dtype, int ld, int q_off
               "retention_scan: a slot of %lld floats does not hold the state", slot_stride);
   if (num_seqs == 0) return 0;
   SHK_REQUIRE(num_seqs <= 65535, "retention_scan: at most 65535 sequences a call");
-  SHK_REQUIRE(proj && decay && positions && cu_q && slots && state && out, "retention_scan: null pointer");
+  SHK_REQUIRE(proj && (decay || log_decay) && positions && cu_q && slots && state && out, "retention_scan: null pointer");
+  SHK_REQUIRE(!(decay && log_decay), "retention_scan: a decay per head or one per token and key channel, not both");
   hipStream_t s = static_cast<hipStream_t>(stream);
   const int lanes = dim > 64 * kRowsPerLane ? 64 : lanes_for(dim, kRowsPerLane);
   const int units = heads * v_dim;
-  const size_t a_token = static_cast<size_t>(retention_heads_a_workgroup(lanes, heads, v_dim)) * 2 * dim * sizeof(float);
+  const size_t a_token =
+      static_cast<size_t>(retention_heads_a_workgroup(lanes, heads, v_dim)) * (log_decay ? 3 : 2) * dim * sizeof(float);
   SHK_REQUIRE(a_token <= 64000, "retention_scan: %d heads of %d elements a workgroup do not fit its LDS",
               retention_heads_a_workgroup(lanes, heads, v_dim), dim);
   const int block = static_cast<int>(64000 / a_token) < kRetBlock ? static_cast<int>(64000 / a_token) : kRetBlock;
   const size_t lds = block * a_token;
 #define SHK_GO(T, L)                                                                                             \
-  retention_scan_kernel<T, L, (L == 64 ? 16 : kRowsPerLane)>                                                    \
+  if (log_decay) SHK_GO2(T, L, true); else SHK_GO2(T, L, false)
+#define SHK_GO2(T, L, G)                                                                                         \
+  retention_scan_kernel<T, L, (L == 64 ? 16 : kRowsPerLane), G>                                                 \
       <<<dim3((units + 256 / L - 1) / (256 / L), num_seqs), 256, lds, s>>>(                                      \
-          static_cast<const T*>(proj), ld, q_off, k_off, v_off, decay, heads, dim, v_dim, positions, cu_q, slots, \
+          static_cast<const T*>(proj), ld, q_off, k_off, v_off, decay, log_decay, q_scale, heads, dim, v_dim, positions, cu_q, slots, \
           state, slot_stride, out, block, act)
 #define SHK_LANES(T)                                                                                             \
   switch (lanes) {                                                                                               \
@@ -507,6 +519,7 @@ extern "C" int shk_retention_scan(const void* proj, int dtype, int ld, int q_off
   }
 #undef SHK_LANES
 #undef SHK_GO
+#undef SHK_GO2
   SHK_LAUNCH_CHECK("retention_scan");
   return 0;
 }

@@ -51,12 +51,12 @@ _SIGNATURES = {
     "shk_attention": [_P, _I, _P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _I, _F, _P, _P,
                       _I, _P],
     "shk_qkv_store": [_P, _I, _I, _I, _I, _I, _I, _F, _I, _F, _F, _P, _P, _I, _P, _P, _P, _I, _P, _P, _I, _I, _I, _P],
-    "shk_latent_prepare": [_P, _I, _I, _I, _I, _I, _P, _P, _F, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _P],
-    "shk_rotate_heads": [_P, _I, _I, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P, _P, _P],
+    "shk_latent_prepare": [_P, _I, _I, _I, _I, _I, _P, _P, _F, _P, _F, _P, _P, _P, _I, _P, _P, _I, _I, _I, _P],
+    "shk_rotate_heads": [_P, _I, _I, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P, _F, _P, _P],
     "shk_latent_attention": [_P, _P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _P, _I, _I, _I, _I, _F, _P],
     "shk_latent_attention_supports_mfma": [_I, _I, _I],
     "shk_latent_attention_bf16": [_P, _P, _I, _I, _I, _I, _P, _P, _P, _I, _P, _I, _I, _I, _I, _F, _P, _I, _I, _P],
-    "shk_gemm_batched": [_P, _P, _P, _I, _I, _I, _I, _I, _I, c_longlong, c_longlong, c_longlong, _I, _P],
+    "shk_gemm_batched": [_P, _P, _P, _I, _I, _I, _I, _I, _I, c_longlong, c_longlong, c_longlong, _I, _I, _P],
     "shk_mlstm_scan": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _F, _F, _I, _I, _I, _I, _P, _P, _P, _P, c_longlong, _P, _P],
     "shk_headnorm_gate": [_P, _P, _I, _I, _P, _F, _P, _I, _I, _I, _I, _I, _P],
     "shk_add_layernorm": [_P, _P, _I, _P, _P, _F, _P, _P, _F, _P, _I, _I, _P, _I, _I, _I, _I, _P],
@@ -66,12 +66,13 @@ _SIGNATURES = {
                               _P, _I, _F, _P, _I, _P],
     "shk_attention_talking_bf16": [_P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I,
                                    _I, _F, _P, _P, _P, _I, _F, _P, _I, _P],
-    "shk_conv_silu": [_P, _I, _P, _P, _I, _I, _P, _P, _P, _P, _P, c_longlong, _I, _P, _I, _I, _P],
-    "shk_dt_softplus": [_P, _I, _P, _P, _I, _I, _P, _I, _P],
+    "shk_short_conv": [_P, _I, _P, _P, _I, _I, _P, _P, _P, _P, _P, c_longlong, _I, _I, _P, _I, _I, _P],
+    "shk_dt_softplus": [_P, _I, _P, _P, _I, _I, _F, _F, _P, _I, _P],
     "shk_selective_scan": [_P, _P, _P, _I, _I, _I, _P, _I, _P, _P, _I, _I, _I, _P, _I, _P, _P, _P, _P, c_longlong,
                            _P, _I, _I, _P],
     "shk_rotate_half_rows": [_P, _I, _I, _I, _I, _I, _P, _P, _F, _I, _P],
-    "shk_retention_scan": [_P, _I, _I, _I, _I, _I, _P, _I, _I, _I, _I, _P, _P, _P, _P, c_longlong, _P, _I, _P],
+    "shk_rglru": [_P, _I, _P, _P, _P, _P, _P, _I, _P, _I, _I, _I, _P, _P, _P, _P, c_longlong, _P, _I, _I, _I, _P],
+    "shk_retention_scan": [_P, _I, _I, _I, _I, _I, _P, _P, _F, _I, _I, _I, _I, _P, _P, _P, _P, c_longlong, _P, _I, _P],
     "shk_retention_chunk_supports": [_I, _I],
     "shk_retention_chunk_bf16": [_P, _I, _I, _I, _I, _P, _I, _I, _I, _I, _I, _P, _P, _P, _P, c_longlong, _P, _P],
     "shk_add_dynamic_tanh": [_P, _P, _I, _F, _F, _P, _P, _P, _I, _P, _I, _I, _I, _I, _P],
@@ -86,9 +87,9 @@ _SIGNATURES = {
                                        _P, _I, _I, _P],
     "shk_diff_attention_prefill_bf16": [_P, _P, _I, _I, _I, _I, _I, _I, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _F, _F, _F,
                                         _F, _P, _I, _P, _I, _I, _I, _P],
-    "shk_moe_route": [_P, _I, _P, _I, _I, _P, _P, _I, _P],
-    "shk_moe_experts": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
-    "shk_moe_experts_grouped": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
+    "shk_moe_route": [_P, _I, _P, _I, _I, _I, _I, _F, _P, _P, _I, _P],
+    "shk_moe_experts": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _F, _P],
+    "shk_moe_experts_grouped": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _P],
     "shk_xielu": [_P, _P, _I, c_longlong, _F, _F, _P],
     "shk_embed_pairs": [_P, _P, _I, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
     "shk_attention_supports_mfma": [_I, _I, _I, _I, _I],
@@ -158,6 +159,7 @@ def load():
         for name, argtypes in (("shk_attention_talking_scratch_floats", [_I, _I, _I, _I]),
                                ("shk_selective_scan_state_floats", [_I, _I, _I]),
                                ("shk_retention_state_floats", [_I, _I, _I]),
+                               ("shk_rglru_state_floats", [_I, _I]),
                                ("shk_conv_store_state_floats", [_I, _I]),
                                ("shk_moe_grouped_scratch_bytes", [_I, _I, _I, _I]),
                                ("shk_attention_talking_mfma_scratch_floats", [_I, _I, _I, _I, _I, _I])):

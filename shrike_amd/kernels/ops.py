@@ -165,7 +165,7 @@ def add_deltas(resid, d1, d2=None, cast=None, dtype=None) -> None:
 def add_normed_rmsnorm(resid, delta, dweight, deps: float, weight=None, eps: float = 0.0, out=None,
                        rows=None, write_resid=True, dtype=None) -> None:
     """x = resid + delta * rsqrt(mean(delta^2) + deps) * dweight (per row; stored back with
-    write_resid); with `out`, out = x * rsqrt(mean(x^2) + eps) * weight too.  With `rows`
+    write_resid); with `out`, out = x * rsqrt(mean(x^2) + eps) * weight too, or x itself without `weight`.  With `rows`
     (int32 [n]) only those rows, into out[0..n)."""
     hidden = resid.shape[1]
     dtype = out.dtype if out is not None else dtype
@@ -601,11 +601,11 @@ def qkv_store(qkv, heads, kv_heads, head_dim, v_dim, positions, token_seq, table
 
 
 def latent_prepare(down, q_rank, kv_rank, rot_dim, q_weight, kv_weight, eps, inv_freq, positions, token_seq,
-                   tables, q_latent, pool, page_size, write_kv=True) -> None:
+                   tables, q_latent, pool, page_size, write_kv=True, magnitude: float = 1.0) -> None:
     """From a token's joint down-projection [q latent | key/value latent | rotated key part]:
     the normed query latent into q_latent [n, q_rank]; the normed key/value latent and the
-    rotated key part (neighbouring pairs) into the token's row of pool [pages, page_size,
-    kv_rank + rot_dim]."""
+    rotated key part (neighbouring pairs; cosine and sine times magnitude) into the token's row of
+    pool [pages, page_size, kv_rank + rot_dim]."""
     n = down.shape[0]
     if not down.is_contiguous() or down.shape[1] != q_rank + kv_rank + rot_dim:
         raise KernelError("latent_prepare: down must be contiguous [n, q_rank + kv_rank + rot_dim]")
@@ -627,7 +627,7 @@ def latent_prepare(down, q_rank, kv_rank, rot_dim, q_weight, kv_weight, eps, inv
     check(load().shk_latent_prepare(
         _dev(down, "down"), dtype_code(down.dtype), n, q_rank, kv_rank, rot_dim,
         _dev(q_weight, "q_weight", torch.float32), _dev(kv_weight, "kv_weight", torch.float32), float(eps),
-        None if inv_freq is None else _dev(inv_freq, "inv_freq", torch.float32),
+        None if inv_freq is None else _dev(inv_freq, "inv_freq", torch.float32), float(magnitude),
         _dev(positions, "positions", torch.int32),
         _dev(token_seq, "token_seq", torch.int32) if write_kv else None,
         _dev(tables, "tables", torch.int32) if write_kv else None, tables.shape[1] if write_kv else 0,
@@ -635,9 +635,10 @@ def latent_prepare(down, q_rank, kv_rank, rot_dim, q_weight, kv_weight, eps, inv
         int(bool(write_kv)), _stream()))
 
 
-def rotate_heads(src, src_head, src_off, dst, dst_head, dst_off, heads, rot_dim, inv_freq, positions) -> None:
+def rotate_heads(src, src_head, src_off, dst, dst_head, dst_off, heads, rot_dim, inv_freq, positions,
+                 magnitude: float = 1.0) -> None:
     """dst[t, h*dst_head + dst_off + e] = rotation of src[t, h*src_head + src_off + e] for e < rot_dim:
-    neighbouring pairs (2i, 2i + 1) turned by positions[t] * inv_freq[i]."""
+    neighbouring pairs (2i, 2i + 1) turned by positions[t] * inv_freq[i], cosine and sine times magnitude."""
     _rows(src, "rotate_heads src")
     _rows(dst, "rotate_heads dst")
     n = src.shape[0]
@@ -650,7 +651,7 @@ def rotate_heads(src, src_head, src_off, dst, dst_head, dst_off, heads, rot_dim,
     check(load().shk_rotate_heads(
         _dev(src, "src"), src.stride(0), src_head, src_off, _dev(dst, "dst"), dst.stride(0), dst_head, dst_off,
         dtype_code(src.dtype), n, heads, rot_dim,
-        None if inv_freq is None else _dev(inv_freq, "inv_freq", torch.float32),
+        None if inv_freq is None else _dev(inv_freq, "inv_freq", torch.float32), float(magnitude),
         _dev(positions, "positions", torch.int32), _stream()))
 
 
@@ -709,18 +710,19 @@ def latent_attention_mfma(q, out, heads, key_dim, v_dim, positions, token_seq, t
 
 def gemm_batched(a, w, out, batch: int, a_step: int, out_step: int) -> None:
     """out[:, b*out_step : b*out_step + m] = a[:, b*a_step : b*a_step + k] @ w[b].T for b < batch;
-    w [batch, m, k] contiguous; a and out 2-d with unit inner stride; all of one dtype."""
+    w [batch, m, k] contiguous; a and out 2-d with unit inner stride; all of one dtype, or out float32."""
     _rows(a, "gemm_batched a")
     _rows(out, "gemm_batched out")
     n = a.shape[0]
-    if w.dim() != 3 or w.shape[0] != batch or not w.is_contiguous() or w.dtype != a.dtype or out.dtype != a.dtype:
-        raise KernelError("gemm_batched: w must be contiguous [batch, m, k] of a's dtype, as out is")
+    if w.dim() != 3 or w.shape[0] != batch or not w.is_contiguous() or w.dtype != a.dtype \
+            or out.dtype not in (a.dtype, torch.float32):
+        raise KernelError("gemm_batched: w must be contiguous [batch, m, k] of a's dtype, out of that dtype or float32")
     m, k = w.shape[1], w.shape[2]
     if out.shape[0] != n or (batch - 1) * a_step + k > a.shape[1] or (batch - 1) * out_step + m > out.shape[1] \
             or out_step < m or a_step < 0:
         raise KernelError("gemm_batched: the batch's slices do not fit a or out")
     check(load().shk_gemm_batched(_dev(a, "a"), _dev(w, "w"), _dev(out, "out"), n, m, k, a.stride(0), out.stride(0),
-                                  batch, a_step, m * k, out_step, dtype_code(a.dtype), _stream()))
+                                  batch, a_step, m * k, out_step, dtype_code(a.dtype), dtype_code(out.dtype), _stream()))
 
 
 def mlstm_state_floats(heads: int, dim: int, v_dim: int) -> int:
@@ -950,27 +952,31 @@ def _state2d(state, who):
         raise KernelError(f"{who}: state must be float32 [slots, floats]")
 
 
-def conv_silu(x, taps, bias, positions, token_seq, cu_q, slots, state, states: int, y) -> None:
-    """y = silu(causal convolution of x's channels over each sequence's inputs): x rows [n, >= inner]
+def short_conv(x, taps, bias, positions, token_seq, cu_q, slots, state, states: int, y,
+               activation: str | None = None) -> None:
+    """y = act(causal convolution of x's channels over each sequence's inputs), act "silu" or nothing: x rows [n, >= inner]
     (a view is fine), taps float32 [inner, K] whose last column meets the current token, the
-    slot's kept inputs for the positions before the step."""
-    _rows(x, "conv_silu x")
+    slot's kept inputs (behind `states` numbers per channel) for the positions before the step."""
+    if activation not in (None, "silu"):
+        raise KernelError(f"short_conv: unknown activation {activation!r}")
+    _rows(x, "short_conv x")
     n, inner = y.shape
     if y.dtype != x.dtype or not y.is_contiguous() or x.shape[0] != n or x.shape[1] < inner:
-        raise KernelError("conv_silu: y must be contiguous [n, inner] of x's dtype")
+        raise KernelError("short_conv: y must be contiguous [n, inner] of x's dtype")
     if taps.dtype != torch.float32 or taps.dim() != 2 or taps.shape[0] != inner or not taps.is_contiguous() \
             or bias.dtype != torch.float32 or bias.numel() != inner:
-        raise KernelError("conv_silu: taps float32 [inner, K], bias float32 [inner]")
-    _state2d(state, "conv_silu")
-    check(load().shk_conv_silu(_dev(x, "x"), x.stride(0), _dev(taps, "taps"), _dev(bias, "bias"), taps.shape[1], inner,
+        raise KernelError("short_conv: taps float32 [inner, K], bias float32 [inner]")
+    _state2d(state, "short_conv")
+    check(load().shk_short_conv(_dev(x, "x"), x.stride(0), _dev(taps, "taps"), _dev(bias, "bias"), taps.shape[1], inner,
                                _dev(positions, "positions", torch.int32), _dev(token_seq, "token_seq", torch.int32),
                                _dev(cu_q, "cu_q", torch.int32), _dev(slots, "slots", torch.int32), _dev(state, "state"),
-                               state.stride(0), states, _dev(y, "y"), dtype_code(y.dtype), n, _stream()))
+                               state.stride(0), states, int(activation == "silu"), _dev(y, "y"), dtype_code(y.dtype), n,
+                                _stream()))
 
 
-def dt_softplus(low, w, b, dt) -> None:
-    """dt = softplus(low[:, :rank] @ w + b) in float32, w [rank, inner] (the stored matrix transposed);
-    low rows may be a view."""
+def dt_softplus(low, w, b, dt, sign: float = 1.0, mult: float = 1.0) -> None:
+    """dt = mult * softplus(sign * (low[:, :rank] @ w + b)) in float32, w [rank, inner] (the stored matrix
+    transposed); low rows may be a view.  (sign and mult -1: the logarithm of a sigmoid.)"""
     _rows(low, "dt_softplus low")
     n, inner = dt.shape
     rank = w.shape[0]
@@ -979,7 +985,7 @@ def dt_softplus(low, w, b, dt) -> None:
             or low.shape[0] != n or low.shape[1] < rank:
         raise KernelError("dt_softplus: float32 low [n, >= rank], w [rank, inner], b [inner], dt [n, inner]")
     check(load().shk_dt_softplus(_dev(low, "low"), low.stride(0), _dev(w, "w"), _dev(b, "b"), rank, inner,
-                                 _dev(dt, "dt"), n, _stream()))
+                                 float(sign), float(mult), _dev(dt, "dt"), n, _stream()))
 
 
 def selective_scan(dt, x, bc, b_off, c_off, z, a_log, dskip, states, taps, raw, positions, cu_q, slots, state,
@@ -1020,29 +1026,65 @@ def rotate_half_rows(x, off, heads, dim, rot_dim, inv_freq, positions, mult: flo
                                       _dev(positions, "positions", torch.int32), float(mult), x.shape[0], _stream()))
 
 
+def rglru_state_floats(width: int, taps: int) -> int:
+    return int(load().shk_rglru_state_floats(width, taps))
+
+
+def rglru(gates, blocks: int, bias_r, bias_i, rate, u, y, raw, taps: int, positions, cu_q, slots, state, out,
+          num_single: int, num_seqs: int) -> None:
+    """S_t = a S_(t-1) + sqrt(1 - a^2) i u, out = S * gelu(y): gates float32 [n, 2 * width] (block by block [r | i],
+    before biases and sigmoid), log a = -rate * r; u [n, width], y and raw rows of out's dtype (views are fine);
+    raw: the convolution's inputs, of which the slot keeps the last taps - 1.  The first num_single of the
+    num_seqs sequences have one token."""
+    n, width = out.shape
+    for name, t in (("y", y), ("raw", raw)):
+        _rows(t, f"rglru {name}")
+    if tuple(gates.shape) != (n, 2 * width) or gates.dtype != torch.float32 or not gates.is_contiguous() \
+            or tuple(u.shape) != (n, width) or not u.is_contiguous() or not out.is_contiguous() \
+            or any(t.dtype != out.dtype for t in (u, y, raw)) or y.shape[0] != n or raw.shape[0] != n \
+            or y.shape[1] < width or raw.shape[1] < width:
+        raise KernelError("rglru: gates float32 [n, 2 * width]; u, y, raw and out rows of one dtype")
+    _state2d(state, "rglru")
+    if cu_q.shape[0] < num_seqs + 1 or slots.shape[0] < num_seqs:
+        raise KernelError("rglru: cu_q / slots are shorter than the step's sequences")
+    check(load().shk_rglru(
+        _dev(gates, "gates"), int(blocks), _f32vec(bias_r, width, "bias_r"), _f32vec(bias_i, width, "bias_i"),
+        _f32vec(rate, width, "rate"), _dev(u, "u"), _dev(y, "y"), y.stride(0), _dev(raw, "raw"), raw.stride(0), width,
+        int(taps), _dev(positions, "positions", torch.int32), _dev(cu_q, "cu_q", torch.int32),
+        _dev(slots, "slots", torch.int32), _dev(state, "state"), state.stride(0), _dev(out, "out"),
+        dtype_code(out.dtype), int(num_single), int(num_seqs), _stream()))
+
+
 def retention_state_floats(heads: int, dim: int, v_dim: int) -> int:
     return int(load().shk_retention_state_floats(heads, dim, v_dim))
 
 
 def retention_scan(proj, q_off, k_off, v_off, decay, num_seqs, heads, dim, v_dim, positions, cu_q, slots, state,
-                   out, activation: str | None = None) -> None:
-    """S_t = decay S_(t-1) + k v^T, o = S^T q per head over the tokens of the step's first num_seqs
+                   out, activation: str | None = None, log_decay=None, q_scale: float = 1.0) -> None:
+    """S_t = decay S_(t-1) + k v^T, o = q_scale S^T q per head over the tokens of the step's first num_seqs
     sequences; proj float32 or bfloat16 rows, out float32 [n, heads * v_dim]; activation "silu": of q, k
-    and v."""
+    and v.  log_decay (float32 [n, heads * dim], with decay None): a decay per token and key channel,
+    S_t = diag(exp(log_decay_t)) S_(t-1) + k v^T."""
     if activation not in (None, "silu"):
         raise KernelError(f"retention_scan: unknown activation {activation!r}")
     _rows(proj, "retention_scan proj")
     n = proj.shape[0]
     if out.dtype != torch.float32 or tuple(out.shape) != (n, heads * v_dim) or not out.is_contiguous():
         raise KernelError("retention_scan: out must be contiguous float32 [n, heads * v_dim]")
-    if decay.dtype != torch.float32 or decay.numel() != heads:
+    if (decay is None) == (log_decay is None):
+        raise KernelError("retention_scan: either one decay per head or log_decay")
+    if decay is not None and (decay.dtype != torch.float32 or decay.numel() != heads):
         raise KernelError("retention_scan: one float32 decay per head")
+    if log_decay is not None and (log_decay.dtype != torch.float32 or tuple(log_decay.shape) != (n, heads * dim)
+                                  or not log_decay.is_contiguous()):
+        raise KernelError("retention_scan: log_decay must be contiguous float32 [n, heads * dim]")
     _state2d(state, "retention_scan")
     if cu_q.shape[0] < num_seqs + 1 or slots.shape[0] < num_seqs:
         raise KernelError("retention_scan: cu_q / slots are shorter than the step's sequences")
     check(load().shk_retention_scan(
-        _dev(proj, "proj"), dtype_code(proj.dtype), proj.stride(0), q_off, k_off, v_off, _dev(decay, "decay"), num_seqs, heads,
-        dim, v_dim, _dev(positions, "positions", torch.int32), _dev(cu_q, "cu_q", torch.int32),
+        _dev(proj, "proj"), dtype_code(proj.dtype), proj.stride(0), q_off, k_off, v_off,
+        None if decay is None else _dev(decay, "decay"), None if log_decay is None else _dev(log_decay, "log_decay"),
+        float(q_scale), num_seqs, heads, dim, v_dim, _dev(positions, "positions", torch.int32), _dev(cu_q, "cu_q", torch.int32),
         _dev(slots, "slots", torch.int32), _dev(state, "state"), state.stride(0), _dev(out, "out"),
         int(activation == "silu"), _stream()))
 
@@ -1071,9 +1113,12 @@ def retention_chunk(proj, q_off, k_off, v_off, decay, first_seq, num_seqs, heads
         _dev(state, "state"), state.stride(0), _dev(out, "out"), _stream()))
 
 
-def moe_route(logits, correction, top: int, chosen, weights) -> None:
+def moe_route(logits, correction, top: int, chosen, weights, groups: tuple | None = None, scale: float = 1.0) -> None:
     """softmax over float32 logits [n, experts]; the `top` largest of score + correction chosen
-    (int32 [n, top]), weights their scores over the chosen ones' sum (float32 [n, top])."""
+    (int32 [n, top]), weights their scores over the chosen ones' sum, times scale (float32 [n, top]).
+    groups = (count, keep): only experts of the `keep` groups (of `count` equal ones of neighbours) whose
+    largest score + correction is largest can be chosen."""
+    count, keep = (1, 1) if groups is None else (int(groups[0]), int(groups[1]))
     _rows(logits, "moe_route logits")
     n, experts = logits.shape
     if logits.dtype != torch.float32 or chosen.dtype != torch.int32 or weights.dtype != torch.float32 \
@@ -1083,8 +1128,8 @@ def moe_route(logits, correction, top: int, chosen, weights) -> None:
     if correction is not None and (correction.dtype != torch.float32 or correction.numel() != experts):
         raise KernelError("moe_route: one float32 correction per expert")
     check(load().shk_moe_route(_dev(logits, "logits"), logits.stride(0),
-                               None if correction is None else _dev(correction, "correction"), experts, top,
-                               _dev(chosen, "chosen"), _dev(weights, "weights"), n, _stream()))
+                               None if correction is None else _dev(correction, "correction"), experts, top, count, keep,
+                               float(scale), _dev(chosen, "chosen"), _dev(weights, "weights"), n, _stream()))
 
 
 MOE_GROUPED_FROM = 1  # tokens of a step from which the experts' products run per expert on the matrix units
@@ -1101,8 +1146,10 @@ def moe_grouped_scratch_bytes(n: int, width: int, experts: int, top: int) -> int
 
 
 def moe_experts(x, chosen, weights, w_gate, w_up, w_down, act_buf, out, activation: str = "silu", add=None,
-                scratch=None, add_gate=None) -> None:
-    """out = add + sum_k weights[:, k] * down_e(act(gate_e x) * up_e x), e = chosen[:, k]; matrices
+                scratch=None, add_gate=None, identity: int = 0, limit: float | None = None, up_shift: float = 0.0) -> None:
+    """out = add + sum_k weights[:, k] * down_e(act(gate_e x) * (up_e x + up_shift)), e = chosen[:, k]; with `limit`
+    the gate's product is bounded from above and the other one from both sides first; the `identity` indices
+    behind the stacked experts stand for x itself; matrices
     stacked [experts, ff, width] / [experts, width, ff] row-major in x's dtype.  scratch (uint8,
     moe_grouped_scratch_bytes): the products run per expert on the matrix units (see moe_grouped).
     add_gate: a float32 column (a view [n] with any stride): add[t] is multiplied by
@@ -1111,6 +1158,7 @@ def moe_experts(x, chosen, weights, w_gate, w_up, w_down, act_buf, out, activati
     n, width = x.shape
     experts, ff, _ = w_gate.shape
     top = chosen.shape[1]
+    form = (int(identity), activation_code(activation), float(limit or 0.0), float(up_shift))
     tensors = (x, w_gate, w_up, w_down, act_buf, out) + (() if add is None else (add,))
     if any(t.dtype != x.dtype or not t.is_contiguous() for t in tensors):
         raise KernelError("moe_experts: tensors must be contiguous and of one dtype")
@@ -1132,13 +1180,13 @@ def moe_experts(x, chosen, weights, w_gate, w_up, w_down, act_buf, out, activati
         check(load().shk_moe_experts_grouped(
             _dev(x, "x"), _dev(chosen, "chosen"), _dev(weights, "weights"), _dev(w_gate, "w_gate"), _dev(w_up, "w_up"),
             _dev(w_down, "w_down"), None if add is None else _dev(add, "add"), gate_ptr, gate_ld,
-            _dev(act_buf, "act_buf"), _dev(out, "out"), _dev(scratch, "scratch"), n, width, ff, experts, top, activation_code(activation),
+            _dev(act_buf, "act_buf"), _dev(out, "out"), _dev(scratch, "scratch"), n, width, ff, experts, top, *form,
             _stream()))
         return
     check(load().shk_moe_experts(_dev(x, "x"), _dev(chosen, "chosen"), _dev(weights, "weights"), _dev(w_gate, "w_gate"),
                                  _dev(w_up, "w_up"), _dev(w_down, "w_down"), None if add is None else _dev(add, "add"),
                                  gate_ptr, gate_ld, _dev(act_buf, "act_buf"), _dev(out, "out"), dtype_code(x.dtype), n, width, ff, experts,
-                                 top, activation_code(activation), _stream()))
+                                 top, *form, _stream()))
 
 
 def xielu(x, out, a_pos: float, a_neg: float) -> None:

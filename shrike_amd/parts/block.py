@@ -263,3 +263,110 @@ class PostNormResidualBlock(Block):
 
 
 register_block("postnorm_residual", PostNormResidualBlock)
+
+
+class OutputNormResidualBlock(Block):
+    """x += s1 * norm1(mixer(x)); x += s2 * norm2(ffn(x)): the sublayers read the stream itself, and what
+    they give is normed on its way into it.  A sublayer's output stays pending together with its norm
+    (whose weight has the layer scale multiplied in); one kernel then adds up a split product's parts,
+    norms them, adds them to the float32 stream and leaves the stream in the compute dtype for the next
+    sublayer's products.  After a layer that is the next block's first step, or the final norm's, which
+    does it in its own pass."""
+
+    def __init__(self, spec, width, name):
+        super().__init__(spec, width, name)
+        self.mixer = build_part("mixer", spec.mixer, width, f"{name}.{spec.mixer_name}")
+        self.mixer_norm = build_part("norm", spec.mixer_norm, width, f"{name}.{spec.mixer_norm_name}")
+        self.ffn = build_part("ffn", spec.ffn, width, f"{name}.{spec.ffn_name}") if spec.ffn is not None else None
+        self.ffn_norm = build_part("norm", spec.ffn_norm, width, f"{name}.{spec.ffn_norm_name}")
+        self.parts = tuple(p for p in (self.mixer, self.mixer_norm, self.ffn, self.ffn_norm) if p is not None)
+        self.parts += tuple(getattr(self.mixer, "parts", ()))
+
+    def _own(self):
+        return tuple(p for p in (self.mixer, self.mixer_norm, self.ffn, self.ffn_norm) if p is not None)
+
+    def _scale_name(self, which: str) -> str:
+        return f"{self.name}.{which}"
+
+    def params(self):
+        from dataclasses import replace
+
+        from .base import ParamSpec
+
+        s, out = self.spec, []
+        for part in self._own():
+            loose = part is self.ffn_norm and self.ffn is None
+            out += [replace(p, optional=True) if loose else p for p in part.params()]
+        if s.layer_scale:
+            out.append(ParamSpec(self._scale_name(s.mixer_scale_name), (self.width,), init="norm", keep_float32=True))
+            out.append(ParamSpec(self._scale_name(s.ffn_scale_name), (self.width,), init="norm", keep_float32=True,
+                                 optional=self.ffn is None))
+        return out
+
+    def check(self, runtime):
+        for part in (self.mixer_norm, self.ffn_norm):
+            if getattr(part.spec, "kind", None) != "rmsnorm":
+                raise ValueError(f"{self.name}: the norm of a sublayer's output must be an RMS norm (rmsnorm)")
+        for part in self._own():
+            part.check(runtime)
+
+    @property
+    def graph_safe(self):
+        return all(part.graph_safe for part in self.parts)
+
+    @property
+    def launches_follow_shape(self):
+        return all(part.launches_follow_shape for part in self.parts)
+
+    def load(self, tensors, runtime):
+        for part in self._own():
+            if part is self.ffn_norm and self.ffn is None:
+                continue
+            part.load(tensors, runtime)
+        s = self.spec
+
+        def pending(norm, scale_name):
+            weight = norm.weight
+            if s.layer_scale:
+                weight = weight * tensors[self._scale_name(scale_name)]
+            return (weight.contiguous(), norm.eps)
+
+        self.mixer_pending = pending(self.mixer_norm, s.mixer_scale_name)
+        self.ffn_pending = None if self.ffn is None else pending(self.ffn_norm, s.ffn_scale_name)
+
+    def _stream(self, ctx, hidden: HiddenState):
+        """The stream as it stands, in the compute dtype (nothing pending afterwards)."""
+        import torch
+
+        from ..kernels import ops
+
+        if ctx.dtype == torch.float32:
+            hidden.settle(ctx)
+            return hidden.resid
+        normed = hidden.pending is not None and hidden.pending_norm is not None and len(hidden.pending_norm) == 2
+        if not normed:
+            hidden.settle(ctx)
+        if hidden.pending is None and hidden.cast is not None:
+            return hidden.cast
+        out = ctx.buffer("stream_cast", hidden.resid.shape, ctx.dtype)
+        if normed:
+            weight, eps = hidden.pending_norm
+            ops.add_normed_rmsnorm(hidden.resid, hidden.pending, weight, eps, out=out)
+            hidden.pending = hidden.pending_norm = None
+        else:
+            ops.cast_rows(hidden.resid, out)
+        hidden.cast = out
+        return out
+
+    def forward(self, ctx, hidden: HiddenState, cache) -> None:
+        x = self._stream(ctx, hidden)
+        hidden.pending = self.mixer.forward(ctx, x, cache)
+        hidden.pending_norm = self.mixer_pending
+        if self.ffn is None:
+            return
+        x = self._stream(ctx, hidden)
+        hidden.pending = self.ffn.forward(ctx, x)
+        hidden.pending_norm = self.ffn_pending
+
+
+register_block("output_norm_residual", OutputNormResidualBlock)

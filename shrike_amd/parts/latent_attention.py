@@ -7,6 +7,7 @@ import torch
 from ..kernels import ops
 from .attention import compute_units
 from .base import PAGE, Mixer, PagedSpec, PageTensor, ParamSpec, register_mixer
+from .rotary import yarn_rates
 
 
 def latent_cache_spec(kv_rank: int, rot_dim: int, window: int | None = None, chunk: int | None = None) -> PagedSpec:
@@ -115,13 +116,19 @@ class LatentAttention(Mixer):
         self.w_o = runtime.weight(tensors[self._t("o")])
         self.w_gate = runtime.weight(tensors[self._t("g")]) if getattr(s, "output_gate", False) else None
         d = int(s.rot_dim)
-        self.inv_freq = None
+        self.inv_freq, self.magnitude = None, 1.0
         if d:
             # one rate per pair of the rotated part; pairs beyond the first `rotated` elements
             # get the rate 0: they turn by nothing and pass unchanged
             turned = d if s.rotated is None else int(s.rotated)
             rates = torch.zeros(d // 2, dtype=torch.float64)
-            rates[: turned // 2] = float(s.rot_theta) ** (-torch.arange(0, turned, 2, dtype=torch.float64) / turned)
+            if s.rot_scaling is not None:
+                if turned < d:
+                    raise ValueError(f"{self.name}: stretched rates need a part that is rotated whole")
+                stretched, self.magnitude = yarn_rates(float(s.rot_theta), turned, *s.rot_scaling)
+                rates[: turned // 2] = torch.tensor(stretched, dtype=torch.float64)
+            else:
+                rates[: turned // 2] = float(s.rot_theta) ** (-torch.arange(0, turned, 2, dtype=torch.float64) / turned)
             self.inv_freq = rates.to(torch.float32).to(runtime.device)
         self.linear = runtime.linear
         self.linear_deferred = runtime.linear_deferred
@@ -137,13 +144,13 @@ class LatentAttention(Mixer):
         c_q = ctx.buffer("latent_cq", (n, s.q_rank), ctx.dtype)
         ops.latent_prepare(down, s.q_rank, s.kv_rank, s.rot_dim, self.q_norm, self.kv_norm, s.eps, self.inv_freq,
                            ctx.positions, ctx.token_seq, tables, c_q, cache.pools["latent"], cache.page_size,
-                           write_kv=cache.owned)
+                           write_kv=cache.owned, magnitude=self.magnitude)
         q = ctx.buffer("latent_q", (n, H * q_head), ctx.dtype)
         self.linear(c_q, self.w_uq, q)
         folded = ctx.buffer("latent_q_folded", (n, H * key_dim), ctx.dtype)
         ops.gemm_batched(q, self.w_uk_t, folded, H, q_head, key_dim)
         ops.rotate_heads(q, q_head, s.head_dim, folded, key_dim, s.kv_rank, H, s.rot_dim, self.inv_freq,
-                         ctx.positions)
+                         ctx.positions, magnitude=self.magnitude)
         mixed = ctx.buffer("latent_mixed", (n, H * s.kv_rank), ctx.dtype)
         if self.mfma:
             nsplit, group = ctx.notes[("latent_attention", H, s.kv_rank, s.rot_dim, s.window, s.chunk)]

@@ -10,7 +10,7 @@ from .base import FeedForward, ParamSpec, register_ffn
 
 class MixtureOfExperts(FeedForward):
     """Router logits come from one product with float32 output; a kernel forms the softmax, adds
-    the correction for the choice only, picks the `top` experts and their weights; the experts'
+    the correction for the choice only, picks the `top` experts (of the best groups) and their weights; the experts'
     matrices are stacked [experts, ...] when the weights are loaded and every (token, chosen
     expert) pair is multiplied by its own expert's rows on the device, chosen there: nothing of
     the routing is read on the host, so steps are recorded into graphs.  The shared expert is
@@ -30,6 +30,11 @@ class MixtureOfExperts(FeedForward):
     def gated(self) -> bool:
         return bool(getattr(self.spec, "gated", True))
 
+    @property
+    def choices(self) -> int:
+        """The router's outputs: the experts, then the identity experts."""
+        return self.spec.experts + self.spec.identity
+
     def params(self):
         s, h = self.spec, self.width
         out = []
@@ -38,11 +43,11 @@ class MixtureOfExperts(FeedForward):
                 out.append(ParamSpec(self._expert(e, "gate"), (s.expert_size, h)))
             out += [ParamSpec(self._expert(e, "up"), (s.expert_size, h)),
                     ParamSpec(self._expert(e, "down"), (h, s.expert_size))]
-        out.append(ParamSpec(self._t("router"), (s.experts, h)))
+        out.append(ParamSpec(self._t("router"), (self.choices, h)))
         if getattr(s, "router_bias", False):
-            out.append(ParamSpec(self._t("router.b"), (s.experts,), init="bias", keep_float32=True))
+            out.append(ParamSpec(self._t("router.b"), (self.choices,), init="bias", keep_float32=True))
         if s.correction:
-            out.append(ParamSpec(self._t("correction"), (s.experts,), init="bias", keep_float32=True))
+            out.append(ParamSpec(self._t("correction"), (self.choices,), init="bias", keep_float32=True))
         if s.shared_size is not None:
             if self.gated:
                 out.append(ParamSpec(f"{self.name}.shared.gate", (s.shared_size, h)))
@@ -61,10 +66,20 @@ class MixtureOfExperts(FeedForward):
                              f"got {s.activation!r}")
         if getattr(s, "shared_gate", False) and s.shared_size is None:
             raise ValueError(f"{self.name}: a gate of the shared expert needs a shared expert")
-        if not 1 <= s.top <= s.experts:
-            raise ValueError(f"{self.name}: top {s.top} is outside 1..{s.experts} experts")
-        if s.experts > 512 or s.top > 64:
-            raise ValueError(f"{self.name}: at most 512 experts and 64 chosen ones, got {s.experts} and {s.top}")
+        if s.identity < 0 or s.experts < 1 or not 1 <= s.top <= self.choices:
+            raise ValueError(f"{self.name}: top {s.top} is outside 1..{self.choices} experts")
+        if self.choices > 512 or s.top > 64:
+            raise ValueError(f"{self.name}: at most 512 experts and 64 chosen ones, got {self.choices} and {s.top}")
+        if s.groups is not None:
+            count, keep = s.groups
+            if not 1 <= count <= 64 or self.choices % count or not 1 <= keep <= count or s.top > keep * (self.choices // count):
+                raise ValueError(f"{self.name}: {s.top} of {self.choices} experts cannot be chosen from {keep} of {count} equal "
+                                 "groups (at most 64)")
+        for limit in (s.limit, s.shared_limit):
+            if limit is not None and not (limit > 0 and self.gated):
+                raise ValueError(f"{self.name}: a limit is a positive number and for gated experts, got {limit}")
+        if s.up_shift and not self.gated:
+            raise ValueError(f"{self.name}: only gated experts have a factor that can be shifted")
         if s.expert_size < 1 or (s.shared_size is not None and s.shared_size < 1):
             raise ValueError(f"{self.name}: expert sizes must be positive")
 
@@ -89,7 +104,8 @@ class MixtureOfExperts(FeedForward):
         self.correction = tensors[self._t("correction")].contiguous() if s.correction else None
         self.shared = None
         if s.shared_size is not None and self.gated:
-            self.shared = (runtime.gated_weight(tensors[f"{self.name}.shared.gate"], tensors[f"{self.name}.shared.up"]),
+            self.shared = (runtime.gated_weight(tensors[f"{self.name}.shared.gate"], tensors[f"{self.name}.shared.up"],
+                                                s.activation, s.shared_limit, s.up_shift),
                            runtime.weight(tensors[f"{self.name}.shared.down"]))
         elif s.shared_size is not None:
             self.shared = (runtime.weight(tensors[f"{self.name}.shared.up"]),
@@ -100,16 +116,17 @@ class MixtureOfExperts(FeedForward):
     def forward(self, ctx, x: torch.Tensor):
         s = self.spec
         n = x.shape[0]
-        logits = ctx.buffer("moe_logits", (n, s.experts + int(self.shared_gate)), torch.float32)
+        logits = ctx.buffer("moe_logits", (n, self.choices + int(self.shared_gate)), torch.float32)
         self.linear(x, self.w_router, logits, bias=self.router_bias)
         chosen = ctx.buffer("moe_chosen", (n, s.top), torch.int32)
         weights = ctx.buffer("moe_weights", (n, s.top), torch.float32)
-        ops.moe_route(logits[:, : s.experts], self.correction, s.top, chosen, weights)
+        ops.moe_route(logits[:, : self.choices], self.correction, s.top, chosen, weights, groups=s.groups,
+                      scale=s.router_scale)
         shared_out = None
         if self.shared is not None:
             act = ctx.buffer("moe_shared_act", (n, s.shared_size), ctx.dtype)
             if self.gated:
-                self.gated_linear(ctx, x, self.shared[0], act, s.activation)
+                self.gated_linear(ctx, x, self.shared[0], act, s.activation, s.shared_limit, s.up_shift)
             else:
                 up = ctx.buffer("moe_shared_up", (n, s.shared_size), ctx.dtype)
                 self.linear(x, self.shared[0], up)
@@ -124,7 +141,8 @@ class MixtureOfExperts(FeedForward):
                                  torch.uint8)
         ops.moe_experts(x, chosen, weights, self.w_gate, self.w_up, self.w_down, act_buf, out, self.activation,
                         add=shared_out, scratch=scratch,
-                        add_gate=logits[:, s.experts] if self.shared_gate else None)
+                        add_gate=logits[:, self.choices] if self.shared_gate else None, identity=s.identity,
+                        limit=s.limit, up_shift=s.up_shift)
         return out
 
 

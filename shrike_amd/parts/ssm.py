@@ -1,5 +1,6 @@
-"""Mixers whose cache is a state of fixed size per request: the selective scan of Mamba and
-retention (linear attention with a fixed decay per head)."""
+"""Mixers whose cache is a state of fixed size per request: the selective scan of Mamba,
+retention (linear attention with a fixed decay per head), gated linear attention (a decay per token
+and key channel) and the real-gated linear recurrent unit of Griffin."""
 
 from __future__ import annotations
 
@@ -77,8 +78,8 @@ class SelectiveScan(Mixer):
         uz = ctx.buffer("scan_in", (n, 2 * s.inner), ctx.dtype)
         self.linear(x, self.w_in, uz)
         u = ctx.buffer("scan_u", (n, s.inner), ctx.dtype)
-        ops.conv_silu(uz, self.taps, self.conv_bias, ctx.positions, ctx.token_seq, ctx.cu_q, ctx.state_slots,
-                      state, s.state, u)
+        ops.short_conv(uz, self.taps, self.conv_bias, ctx.positions, ctx.token_seq, ctx.cu_q, ctx.state_slots,
+                       state, s.state, u, activation="silu")
         low = ctx.buffer("scan_low", (n, s.dt_rank + 2 * s.state), torch.float32)
         self.linear(u, self.w_x, low)
         dt = ctx.buffer("scan_dt", (n, s.inner), torch.float32)
@@ -201,3 +202,164 @@ class Retention(Mixer):
 
 
 register_mixer("retention", Retention)
+
+
+class GatedLinearAttention(Mixer):
+    """One product yields queries, keys, values and the output gate; the decays come through a low-rank
+    pair of matrices of their own, whose results are never rounded (float32): log alpha = -softplus(-(W_a2 (W_a1
+    x) + b)) / tau.  The scan carries S per head in the request's state slot (float32); each head's readout is
+    brought to unit root mean square, weighted, gated by SiLU and projected."""
+
+    launches_follow_shape = True
+    state_graph_safe = True
+
+    def _t(self, role: str) -> str:
+        return self.tensor_name(role)
+
+    def params(self):
+        s, h = self.spec, self.width
+        qk, v = s.num_heads * s.head_dim, s.num_heads * s.value_dim
+        free = s.decay_rank or 16
+        return [
+            ParamSpec(self._t("q"), (qk, h)), ParamSpec(self._t("k"), (qk, h)), ParamSpec(self._t("v"), (v, h)),
+            ParamSpec(self._t("g"), (v, h)), ParamSpec(self._t("o"), (h, v)),
+            ParamSpec(self._t("norm"), (s.value_dim,), init="norm", keep_float32=True),
+            ParamSpec(self._t("a1"), (s.decay_rank, h), free_size=free),
+            ParamSpec(self._t("a2"), (qk, s.decay_rank), keep_float32=True, free_size=free),
+            ParamSpec(self._t("a2.b"), (qk,), init="bias", keep_float32=True),
+        ]
+
+    def state_floats(self) -> int:
+        s = self.spec
+        return s.num_heads * s.value_dim * s.head_dim
+
+    def cache_spec(self):
+        return StateSpec((self.state_floats(),), "float32")
+
+    def check(self, runtime):
+        s = self.spec
+        if min(s.num_heads, s.head_dim, s.value_dim) < 1 or not s.tau > 0:
+            raise ValueError(f"{self.name}: heads, head_dim, value_dim and tau must be positive")
+        if s.head_dim > 1024:
+            raise ValueError(f"{self.name}: head_dim {s.head_dim} is more than the 1024 the scan kernel holds")
+        if ops.retention_state_floats(s.num_heads, s.head_dim, s.value_dim) != self.state_floats():
+            raise RuntimeError(f"{self.name}: the kernel's state layout and the cache's size disagree")
+
+    def load(self, tensors, runtime):
+        s = self.spec
+        qk, v = s.num_heads * s.head_dim, s.num_heads * s.value_dim
+        a1, a2 = tensors[self._t("a1")], tensors[self._t("a2")]
+        self.rank = a1.shape[0]
+        if a2.shape[1] != self.rank or not 1 <= self.rank <= 1024:
+            raise ValueError(f"{self.name}: the decays' two matrices have ranks {self.rank} and {a2.shape[1]} (1 to 1024)")
+        self.w_in = runtime.weight(torch.cat([tensors[self._t(r)] for r in ("q", "k", "v", "g")], dim=0))
+        self.offsets = {"q": 0, "k": qk, "v": 2 * qk, "g": 2 * qk + v}
+        self.in_width = 2 * qk + 2 * v
+        self.w_a1 = runtime.weight(a1)
+        self.w_a2 = a2.t().contiguous()  # [rank, heads * head_dim]: channels are neighbours in memory
+        self.a2_bias = tensors[self._t("a2.b")].contiguous()
+        self.norm_weight = tensors[self._t("norm")].repeat(s.num_heads).contiguous()
+        self.w_o = runtime.weight(tensors[self._t("o")])
+        self.q_scale = float(s.head_dim) ** -0.5
+        self.linear = runtime.linear
+        self.linear_deferred = runtime.linear_deferred
+
+    def forward(self, ctx, x: torch.Tensor, cache):
+        s, off = self.spec, self.offsets
+        n = x.shape[0]
+        proj = ctx.buffer("gla_proj", (n, self.in_width), torch.float32)
+        self.linear(x, self.w_in, proj)
+        low = ctx.buffer("gla_low", (n, self.rank), torch.float32)
+        self.linear(x, self.w_a1, low)
+        log_decay = ctx.buffer("gla_log_decay", (n, s.num_heads * s.head_dim), torch.float32)
+        ops.dt_softplus(low, self.w_a2, self.a2_bias, log_decay, sign=-1.0, mult=-1.0 / s.tau)
+        read = ctx.buffer("gla_read", (n, s.num_heads * s.value_dim), torch.float32)
+        state = cache.state_padded if cache.state_padded is not None else cache.state
+        ops.retention_scan(proj, off["q"], off["k"], off["v"], None, ctx.num_seqs, s.num_heads, s.head_dim, s.value_dim,
+                           ctx.positions, ctx.cu_q, ctx.state_slots, state, read, log_decay=log_decay,
+                           q_scale=self.q_scale)
+        gated = ctx.buffer("gla_gated", (n, s.num_heads * s.value_dim), ctx.dtype)
+        ops.headnorm_gate(read, proj[:, off["g"]:], self.norm_weight, s.eps, gated, s.num_heads, s.value_dim, gate_act="silu")
+        return self.linear_deferred(ctx, "gla_out", gated, self.w_o)
+
+
+register_mixer("gated_linear_attention", GatedLinearAttention)
+
+
+class GatedRecurrence(Mixer):
+    """One product yields both branches; the recurrent one passes a short causal convolution, a
+    block-diagonal product gives both gates' pre-activations in float32, and one kernel forms the gates, the
+    decays and the recurrence (float32) and multiplies its state by GELU of the other branch; out-projection.
+
+    A request's state slot holds S [recurrent_width] and the convolution's last taps - 1 inputs."""
+
+    launches_follow_shape = True
+    state_graph_safe = True
+
+    def _t(self, role: str) -> str:
+        return self.tensor_name(role)
+
+    def params(self):
+        s, h = self.spec, self.width
+        w, part = s.recurrent_width, s.recurrent_width // max(1, s.blocks)
+        out = []
+        for role in ("y", "x"):
+            out += [ParamSpec(self._t(role), (w, h)), ParamSpec(self._t(role + ".b"), (w,), init="bias", keep_float32=True)]
+        out += [ParamSpec(self._t("conv"), (w, s.conv), init="taps", keep_float32=True),
+                ParamSpec(self._t("conv.b"), (w,), init="bias", keep_float32=True)]
+        for role in ("ra", "ri"):
+            out += [ParamSpec(self._t(role), (s.blocks, part, part)),
+                    ParamSpec(self._t(role + ".b"), (s.blocks, part), init="bias", keep_float32=True)]
+        return out + [ParamSpec(self._t("lam"), (w,), init="slow_rate", keep_float32=True), ParamSpec(self._t("o"), (h, w))]
+
+    def state_floats(self) -> int:
+        return self.spec.recurrent_width * max(1, self.spec.conv)
+
+    def cache_spec(self):
+        return StateSpec((self.state_floats(),), "float32")
+
+    def check(self, runtime):
+        s = self.spec
+        if min(s.recurrent_width, s.blocks, s.conv) < 1 or s.recurrent_width % s.blocks or not s.power > 0:
+            raise ValueError(f"{self.name}: recurrent_width {s.recurrent_width} must be a positive multiple of blocks {s.blocks}, "
+                             f"conv ({s.conv}) and power ({s.power}) positive")
+        if s.conv > 64:
+            raise ValueError(f"{self.name}: at most 64 taps, got {s.conv}")
+        if ops.rglru_state_floats(s.recurrent_width, s.conv) != self.state_floats():
+            raise RuntimeError(f"{self.name}: the kernel's state layout and the cache's size disagree")
+
+    def load(self, tensors, runtime):
+        s = self.spec
+        self.w_in = runtime.weight(torch.cat([tensors[self._t("y")], tensors[self._t("x")]], dim=0))
+        self.b_in = torch.cat([tensors[self._t("y.b")], tensors[self._t("x.b")]]).contiguous()
+        self.taps = tensors[self._t("conv")].contiguous()
+        self.conv_bias = tensors[self._t("conv.b")].contiguous()
+        # per block [r rows; i rows]: one batched product gives both gates
+        self.w_gates = torch.cat([tensors[self._t("ra")], tensors[self._t("ri")]], dim=1).contiguous()
+        self.r_bias = tensors[self._t("ra.b")].reshape(-1).contiguous()
+        self.i_bias = tensors[self._t("ri.b")].reshape(-1).contiguous()
+        lam = tensors[self._t("lam")].to(torch.float64)
+        self.rate = (float(s.power) * torch.nn.functional.softplus(lam)).to(torch.float32).contiguous()
+        self.w_o = runtime.weight(tensors[self._t("o")])
+        self.linear = runtime.linear
+        self.linear_deferred = runtime.linear_deferred
+
+    def forward(self, ctx, x: torch.Tensor, cache):
+        s = self.spec
+        n, w = x.shape[0], s.recurrent_width
+        part = w // s.blocks
+        state = cache.state_padded if cache.state_padded is not None else cache.state
+        yx = ctx.buffer("rglru_in", (n, 2 * w), ctx.dtype)
+        self.linear(x, self.w_in, yx, bias=self.b_in)
+        raw = yx[:, w:]
+        u = ctx.buffer("rglru_u", (n, w), ctx.dtype)
+        ops.short_conv(raw, self.taps, self.conv_bias, ctx.positions, ctx.token_seq, ctx.cu_q, ctx.state_slots, state, 1, u)
+        gates = ctx.buffer("rglru_gates", (n, 2 * w), torch.float32)
+        ops.gemm_batched(u, self.w_gates, gates, s.blocks, part, 2 * part)
+        read = ctx.buffer("rglru_read", (n, w), ctx.dtype)
+        ops.rglru(gates, s.blocks, self.r_bias, self.i_bias, self.rate, u, yx, raw, s.conv, ctx.positions, ctx.cu_q,
+                  ctx.state_slots, state, read, ctx.num_decode, ctx.num_seqs)
+        return self.linear_deferred(ctx, "rglru_out", read, self.w_o)
+
+
+register_mixer("gated_recurrence", GatedRecurrence)

@@ -28,7 +28,9 @@ _STD = {"matrix": 0.02, "embedding": 0.02, "bias": 0.02, "norm": 0.1, "norm_zero
         # a table of numbers that are added to attention scores: N(0, 1) in both modes
         "score_bias": 1.0,
         # the taps of a short convolution: N(0, 0.3), and 1 added to the last (the current token's)
-        "taps": 0.3}
+        "taps": 0.3,
+        # the argument of a softplus that a recurrence's rate is proportional to: -5 + N(0, 1.5)
+        "slow_rate": 1.5}
 
 #: "reference": the distributions above.  "unit": matrices N(0, 1/fan_in) (the
 #: embedding table N(0, 1)), biases N(0, 0.1): every part's output is as large
@@ -70,6 +72,8 @@ def random_tensor(p: ParamSpec, seed: int, dtype: torch.dtype, device="cpu",
         t += torch.eye(shape[0], shape[1], device=device)
     elif p.init == "average":
         t += 1.0 / shape[0]
+    elif p.init == "slow_rate":
+        t -= 5.0
     elif p.init == "taps":
         t[:, -1] += 1.0
     return t.to(dtype)

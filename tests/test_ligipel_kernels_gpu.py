@@ -316,7 +316,7 @@ def run_scan_chain(ops, uz, low_of, w, inner, states, rank, taps, dtype, state, 
         rows = dev(torch.cat([uz[s][st:st + c] for s, _, st, c in step]), dtype)
         n = rows.shape[0]
         x = torch.empty(n, inner, dtype=dtype, device="cuda")
-        ops.conv_silu(rows, wd["conv"], wd["conv.b"], positions, token_seq, cu, slots, state, states, x)
+        ops.short_conv(rows, wd["conv"], wd["conv.b"], positions, token_seq, cu, slots, state, states, x, activation="silu")
         low = dev(low_of(x.double().cpu()), torch.float32)
         dt = torch.empty(n, inner, device="cuda")
         ops.dt_softplus(low, wd["dt"], wd["dt.b"], dt)
