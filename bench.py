@@ -329,7 +329,7 @@ def kernel_breakdown(engine, steps: int = 3, before_step=None) -> dict:
              "xielu", "layernorm", "add_layernorm", "attention_talking", "attention_talking_mfma", "short_conv", "dt_softplus", "selective_scan",
              "rotate_half_rows", "retention_scan", "retention_chunk", "moe_route", "moe_experts", "mix_history", "scale_softcap",
              "postnorm", "cast_rows", "activate", "gate_mul", "add_dynamic_tanh", "conv_store", "diff_attention",
-             "diff_attention_decode", "diff_attention_prefill"]
+             "diff_attention_decode", "diff_attention_prefill", "rglru", "gla_chunk"]
     names = [n for n in names if hasattr(ops, n)]
     spans: list[tuple[str, object, object]] = []
     saved = {n: getattr(ops, n) for n in names}
@@ -637,6 +637,64 @@ def fozedra_like(qcfg, window: int, pattern: str):
     return fcfg, sizes
 
 
+def bevovik_like(qcfg, pattern: str, experts: int, top: int):
+    """A Bevovik configuration with the layer sizes of a Qwen2 one (same width, vocabulary and number of
+    layers).  `pattern` says which mixer each layer has, letter by letter, repeated: r, Griffin's recurrent
+    block as wide as the model, its gates' matrices in blocks of 128 or 256, 4 taps; l, latent attention as
+    Poresun's (no output gate, stretched rates); g, gated linear attention with width / 256 heads of 128
+    query/key and 256 value elements (as Ligipel's retention) and decays through a product of rank 16.
+    Every layer has `experts` routed experts in two groups of which one is kept, two of the router's outputs
+    identity experts, `top` of them a token's (together half of Qwen2's feed-forward), and a shared expert
+    of the other half.  With it an object that names the sizes as the formulas of this program expect them
+    (see ligipel_like)."""
+    from types import SimpleNamespace
+
+    from shrike_amd.models.bevovik import (BevovikConfig, BevovikLayer, GroupedMixture, KeyDecayAttention, Recurrence,
+                                           StretchedLatentAttention)
+
+    h, d, H, KV = qcfg.hidden_size, qcfg.head_dim, qcfg.num_attention_heads, qcfg.num_key_value_heads
+    inter, gheads = qcfg.intermediate_size, max(1, qcfg.hidden_size // 256)
+    up64 = lambda x: max(64, -(-int(x) // 64) * 64)  # noqa: E731
+    ff, shared = max(64, inter // (2 * top) // 64 * 64), up64(inter / 2)
+    identity = 2 if experts % 2 == 0 else 1
+    part = 256 if h % 256 == 0 else 128
+    latent = StretchedLatentAttention(heads=H, dim=d, rot_dim=d // 2, vdim=d, q_rank=up64(3 * h / 8),
+                                      kv_rank=min(up64(h / 8), 512), scale=(1.5 * d) ** -0.5, rot_base=10000.0,
+                                      rot_dims=d // 2, rot_scaling=(4.0, 4096.0, 32.0, 1.0))
+    mixers = {"r": ("rglru", Recurrence(width=h, blocks=h // part, conv=4)), "l": ("latent_attention", latent),
+              "g": ("gla", KeyDecayAttention(heads=gheads, dim=128, vdim=256, tau=16.0, decay_rank=16))}
+    if set(pattern) - set(mixers):
+        raise SystemExit(f"--pattern: unknown letters {pattern!r} for --bevovik (g, l, r)")
+    mlp = GroupedMixture(experts=experts, top=top, ff=ff, limit=7.0, identity=identity, groups=(2, 1), scale=2.0,
+                         shared=(shared, 7.0))
+    letters = [pattern[i % len(pattern)] for i in range(qcfg.num_hidden_layers)]
+    bcfg = BevovikConfig(vocab=qcfg.vocab_size, width=h, norm_eps=qcfg.rms_norm_eps,
+                         layers=tuple(BevovikLayer(*mixers[c], mlp) for c in letters))
+    n = len(letters)
+    elements = {
+        "r": 3 * h * h + 2 * h * part, "g": (2 * 128 + 3 * 256) * gheads * h + 16 * (h + 128 * gheads),
+        "l": (latent.q_rank + latent.kv_rank + latent.rot_dim) * h + H * (d + latent.rot_dim) * latent.q_rank
+        + 2 * H * d * latent.kv_rank + H * d * h,
+    }
+    states = {"r": 4 * h, "g": gheads * 128 * 256, "l": 0}
+    sizes = SimpleNamespace(
+        hidden_size=h, head_dim=d, num_attention_heads=H, num_key_value_heads=KV, intermediate_size=inter,
+        num_hidden_layers=n, vocab_size=qcfg.vocab_size, attention_layers=letters.count("l"),
+        kv_elements_per_token=letters.count("l") * (latent.kv_rank + latent.rot_dim),
+        state_bytes_per_seq=2 * 4 * sum(states[c] for c in letters))
+    picked = top * experts / (experts + identity)  # of a token's choices, on average, those with matrices
+
+    def layer_elements(per_experts: float) -> int:
+        return int(sum(elements[c] for c in letters) // n + (experts + identity) * h + 3 * h * shared + per_experts * 3 * h * ff)
+
+    def at_batch(b: int) -> None:
+        sizes.layer_elements = layer_elements(experts * (1.0 - (1.0 - picked / experts) ** b))
+
+    sizes.at_batch = at_batch
+    sizes.layer_elements = layer_elements(picked)  # a prompt: every token's own experts are work
+    return bcfg, sizes
+
+
 def run_designs(args, qcfg) -> dict:
     """Another design beside Qwen2 at equal layer sizes, random weights: a prompt of 2,048
     tokens in one step, decode steps at batch 1, 8 and 64 from that context, and what each
@@ -646,9 +704,12 @@ def run_designs(args, qcfg) -> dict:
     import torch
 
     from shrike_amd import SamplingParams
-    from shrike_amd.models import fozedra, ligipel, minilorn, mofarax, poresun, qwen2
+    from shrike_amd.models import bevovik, fozedra, ligipel, minilorn, mofarax, poresun, qwen2
 
-    if args.fozedra:
+    if args.bevovik:
+        bcfg, bsizes = bevovik_like(qcfg, args.pattern if set(args.pattern) <= set("rlg") else "rlg", args.experts, args.top)
+        other = ("bevovik", bevovik.build_spec(bcfg), bsizes)
+    elif args.fozedra:
         fcfg, fsizes = fozedra_like(qcfg, args.window, args.pattern if set(args.pattern) <= set("asl") else "asl")
         other = ("fozedra", fozedra.build_spec(fcfg), fsizes)
     elif args.poresun:
@@ -849,19 +910,22 @@ def main() -> int:
                     help="the Poresun design beside Qwen2 at the layer sizes of --shape, random weights")
     ap.add_argument("--fozedra", action="store_true",
                     help="the Fozedra design beside Qwen2 at the layer sizes of --shape, random weights")
-    ap.add_argument("--experts", type=int, default=8, metavar="N", help="--ligipel, --poresun: routed experts a layer")
-    ap.add_argument("--top", type=int, default=2, metavar="N", help="--ligipel, --poresun: experts a token uses")
+    ap.add_argument("--bevovik", action="store_true",
+                    help="the Bevovik design beside Qwen2 at the layer sizes of --shape, random weights")
+    ap.add_argument("--experts", type=int, default=8, metavar="N", help="--ligipel, --poresun, --bevovik: routed experts a layer")
+    ap.add_argument("--top", type=int, default=2, metavar="N", help="--ligipel, --poresun, --bevovik: experts a token uses")
     ap.add_argument("--pattern", default="alml", metavar="LETTERS",
                     help="--minilorn: the layers' mixers in order, repeated: a(ttention), l(atent attention), m(atrix memory); "
                          "--ligipel: p(arallel attention and scan), r(etention), default pppr; --poresun: a(ttention "
                          "with a window), b (causal attention), s (reads the last b layer's keys and values), "
                          "l(atent attention), default absl; --fozedra: a (differential attention), s (reads the last a "
-                         "layer's keys and values), l(ightning attention), default asl")
+                         "layer's keys and values), l(ightning attention), default asl; --bevovik: r(ecurrence), l(atent attention), "
+                         "g(ated linear attention), default rlg")
     ap.add_argument("--window", type=int, default=4096, metavar="N",
                     help="--minilorn: sliding window of its latent attention (4096: no fewer keys than Qwen2 reads)")
-    ap.add_argument("--design-only", choices=["qwen2", "mofarax", "minilorn", "ligipel", "poresun", "fozedra"],
+    ap.add_argument("--design-only", choices=["qwen2", "mofarax", "minilorn", "ligipel", "poresun", "fozedra", "bevovik"],
                     default=None,
-                    help="--mofarax / --minilorn / --ligipel / --poresun / --fozedra: run only this one of the two (for a profile of "
+                    help="--mofarax / --minilorn / --ligipel / --poresun / --fozedra / --bevovik: run only this one of the two (for a profile of "
                          "one model's kernels)")
     ap.add_argument("--mask-size", type=int, default=8192, metavar="N",
                     help="--mofarax: positions per block of its attention (8192: no fewer keys than Qwen2 reads)")
@@ -895,12 +959,14 @@ def main() -> int:
         raw["num_hidden_layers"] = args.layers
     cfg = Qwen2Config.from_dict(raw)
     spec = build_spec(cfg)
-    if args.mofarax or args.minilorn or args.ligipel or args.poresun or args.fozedra:
+    if args.mofarax or args.minilorn or args.ligipel or args.poresun or args.fozedra or args.bevovik:
         designs = run_designs(args, cfg)
-        design = "Fozedra" if args.fozedra else "Poresun" if args.poresun else "Ligipel" if args.ligipel else "Minilorn" if args.minilorn else "Mofarax"
+        design = "Bevovik" if args.bevovik else "Fozedra" if args.fozedra else "Poresun" if args.poresun else "Ligipel" if args.ligipel else "Minilorn" if args.minilorn else "Mofarax"
         config = {"shape": args.shape, "layers": cfg.num_hidden_layers, "prompt": PROMPT_LEN,
                   "decode_steps": args.design_steps}
-        config.update({"pattern": args.pattern if set(args.pattern) <= set("asl") else "asl", "window": args.window}
+        config.update({"pattern": args.pattern if set(args.pattern) <= set("rlg") else "rlg", "experts": args.experts, "top": args.top}
+                      if args.bevovik
+                      else {"pattern": args.pattern if set(args.pattern) <= set("asl") else "asl", "window": args.window}
                       if args.fozedra
                       else {"pattern": args.pattern if set(args.pattern) <= set("absl") else "absl", "window": args.window,
                        "experts": args.experts, "top": args.top} if args.poresun

@@ -418,6 +418,20 @@ int shk_retention_chunk_bf16(const void* proj, int ld, int q_off, int k_off, int
                              const int32_t* cu_q, const int32_t* slots, float* state, long long slot_stride, float* out,
                              void* stream);
 
+// Gated linear attention (shk_retention_scan with log_decay) for prompt portions over bfloat16 projections, in
+// chunks of 64 tokens on the matrix units (gla_chunk.hip), for sequences first_seq .. first_seq + num_seqs - 1,
+// whose rows are first_row .. first_row + rows - 1; sizes as shk_gla_chunk_supports says, columns of q and k in
+// runs of 8.  chunk_lists: int32, the chunks' sequences, then their first tokens within the portions, then every
+// portion's first chunk.  scratch: shk_gla_chunk_scratch_bytes(...) bytes.  A float32 operand of a product enters
+// as the sum of two bfloat16 numbers; sums and the state are float32.
+int shk_gla_chunk_supports(int dim, int v_dim);
+long long shk_gla_chunk_scratch_bytes(int rows, int chunks, int heads, int dim, int v_dim);
+int shk_gla_chunk_bf16(const void* proj, int ld, int q_off, int k_off, int v_off, const float* log_decay,
+                       float q_scale, int first_seq, int num_seqs, int first_row, int rows, int heads, int dim,
+                       int v_dim, const int32_t* chunk_lists, int chunks, const int32_t* positions,
+                       const int32_t* cu_q, const int32_t* slots, float* state, long long slot_stride,
+                       void* scratch, float* out, void* stream);
+
 // tanh(alpha * x) * weight + bias in the place of a norm (dynamic_tanh.hip).  resid[row] gains scale *
 // delta[row] first (delta of `dtype`, or delta_splits float32 partial sums [splits][resid_rows][hidden];
 // null: nothing) and is stored back with write_resid; out[r] (null: none) belongs to row rows[r] (rows

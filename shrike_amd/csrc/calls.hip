@@ -92,6 +92,7 @@ const Launcher kLaunchers[] = {
     SHK_LAUNCHER(shk_rglru),
     SHK_LAUNCHER(shk_retention_scan),
     SHK_LAUNCHER(shk_retention_chunk_bf16),
+    SHK_LAUNCHER(shk_gla_chunk_bf16),
     SHK_LAUNCHER(shk_add_dynamic_tanh),
     SHK_LAUNCHER(shk_conv_store),
     SHK_LAUNCHER(shk_diff_attention),

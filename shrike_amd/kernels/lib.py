@@ -75,6 +75,9 @@ _SIGNATURES = {
     "shk_retention_scan": [_P, _I, _I, _I, _I, _I, _P, _P, _F, _I, _I, _I, _I, _P, _P, _P, _P, c_longlong, _P, _I, _P],
     "shk_retention_chunk_supports": [_I, _I],
     "shk_retention_chunk_bf16": [_P, _I, _I, _I, _I, _P, _I, _I, _I, _I, _I, _P, _P, _P, _P, c_longlong, _P, _P],
+    "shk_gla_chunk_supports": [_I, _I],
+    "shk_gla_chunk_bf16": [_P, _I, _I, _I, _I, _P, _F, _I, _I, _I, _I, _I, _I, _I, _P, _I, _P, _P, _P, _P, c_longlong, _P, _P,
+                           _P],
     "shk_add_dynamic_tanh": [_P, _P, _I, _F, _F, _P, _P, _P, _I, _P, _I, _I, _I, _I, _P],
     "shk_conv_store": [_P, _I, _P, _I, _P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _P, _F, _I, _I, _I, _P, _P, _P, _P, _I, _P,
                        c_longlong, _P, _I, _I, _P, _P, _P, _P, _I, _I, _P],
@@ -160,6 +163,7 @@ def load():
                                ("shk_selective_scan_state_floats", [_I, _I, _I]),
                                ("shk_retention_state_floats", [_I, _I, _I]),
                                ("shk_rglru_state_floats", [_I, _I]),
+                               ("shk_gla_chunk_scratch_bytes", [_I, _I, _I, _I, _I]),
                                ("shk_conv_store_state_floats", [_I, _I]),
                                ("shk_moe_grouped_scratch_bytes", [_I, _I, _I, _I]),
                                ("shk_attention_talking_mfma_scratch_floats", [_I, _I, _I, _I, _I, _I])):

@@ -1113,6 +1113,45 @@ def retention_chunk(proj, q_off, k_off, v_off, decay, first_seq, num_seqs, heads
         _dev(state, "state"), state.stride(0), _dev(out, "out"), _stream()))
 
 
+def gla_chunk_supports(dim: int, v_dim: int) -> bool:
+    return bool(load().shk_gla_chunk_supports(int(dim), int(v_dim)))
+
+
+GLA_CHUNK = 64  # tokens of a prompt portion that gla_chunk takes at a time
+
+
+def gla_chunk_scratch_bytes(rows: int, chunks: int, heads: int, dim: int, v_dim: int) -> int:
+    return int(load().shk_gla_chunk_scratch_bytes(rows, chunks, heads, dim, v_dim))
+
+
+def gla_chunk(proj, q_off, k_off, v_off, log_decay, q_scale: float, first_seq: int, num_seqs: int, first_row: int, heads,
+              dim, v_dim, chunk_lists, positions, cu_q, slots, state, scratch, out) -> None:
+    """retention_scan with log_decay for prompt portions over bfloat16 rows, in chunks on the matrix units:
+    sequences first_seq .. first_seq + num_seqs - 1, whose rows start at first_row.  chunk_lists (int32): the
+    sequences of the chunks of GLA_CHUNK tokens, their first tokens within the portions, every portion's first
+    chunk."""
+    _rows(proj, "gla_chunk proj")
+    n = proj.shape[0]
+    rows, chunks = n - first_row, (chunk_lists.numel() - num_seqs) // 2
+    if proj.dtype != torch.bfloat16 or out.dtype != torch.float32 or tuple(out.shape) != (n, heads * v_dim) \
+            or not out.is_contiguous():
+        raise KernelError("gla_chunk: proj bfloat16, out contiguous float32 [n, heads * v_dim]")
+    if log_decay.dtype != torch.float32 or tuple(log_decay.shape) != (n, heads * dim) or not log_decay.is_contiguous():
+        raise KernelError("gla_chunk: log_decay must be contiguous float32 [n, heads * dim]")
+    if chunk_lists.numel() != 2 * chunks + num_seqs or chunks * GLA_CHUNK < rows:
+        raise KernelError("gla_chunk: the chunk lists do not cover the portions")
+    if scratch.dtype != torch.uint8 or scratch.numel() < gla_chunk_scratch_bytes(rows, chunks, heads, dim, v_dim):
+        raise KernelError("gla_chunk: scratch is too small")
+    _state2d(state, "gla_chunk")
+    if cu_q.shape[0] < first_seq + num_seqs + 1 or slots.shape[0] < first_seq + num_seqs:
+        raise KernelError("gla_chunk: cu_q / slots are shorter than the step's sequences")
+    check(load().shk_gla_chunk_bf16(
+        _dev(proj, "proj"), proj.stride(0), q_off, k_off, v_off, _dev(log_decay, "log_decay"), float(q_scale), first_seq,
+        num_seqs, first_row, rows, heads, dim, v_dim, _dev(chunk_lists, "chunk_lists", torch.int32), chunks,
+        _dev(positions, "positions", torch.int32), _dev(cu_q, "cu_q", torch.int32), _dev(slots, "slots", torch.int32),
+        _dev(state, "state"), state.stride(0), _dev(scratch, "scratch"), _dev(out, "out"), _stream()))
+
+
 def moe_route(logits, correction, top: int, chosen, weights, groups: tuple | None = None, scale: float = 1.0) -> None:
     """softmax over float32 logits [n, experts]; the `top` largest of score + correction chosen
     (int32 [n, top]), weights their scores over the chosen ones' sum, times scale (float32 [n, top]).

@@ -4,9 +4,11 @@ and key channel) and the real-gated linear recurrent unit of Griffin."""
 
 from __future__ import annotations
 
+import numpy as np
 import torch
 
 from ..kernels import ops
+from .attention import portion_runs
 from .base import Mixer, ParamSpec, PositionEncoding, StateSpec, build_part, register_mixer
 
 
@@ -205,7 +207,8 @@ register_mixer("retention", Retention)
 
 
 class GatedLinearAttention(Mixer):
-    """One product yields queries, keys, values and the output gate; the decays come through a low-rank
+    """One product yields queries, keys, values and the output gate (in the compute dtype where bfloat16
+    prompt portions run in chunks on the matrix units, else in float32); the decays come through a low-rank
     pair of matrices of their own, whose results are never rounded (float32): log alpha = -softplus(-(W_a2 (W_a1
     x) + b)) / tau.  The scan carries S per head in the request's state slot (float32); each head's readout is
     brought to unit root mean square, weighted, gated by SiLU and projected."""
@@ -245,6 +248,18 @@ class GatedLinearAttention(Mixer):
         if ops.retention_state_floats(s.num_heads, s.head_dim, s.value_dim) != self.state_floats():
             raise RuntimeError(f"{self.name}: the kernel's state layout and the cache's size disagree")
 
+    LISTS = "gla_chunks"  # the chunks of a step's prompt portions, the same for every such layer
+
+    def prepare(self, shape) -> None:
+        if not self.chunked or self.LISTS in shape.notes:
+            return
+        shape.notes[self.LISTS] = True
+        portions = shape.q_lens[shape.num_decode:]
+        if portions.size:
+            seqs, t0 = portion_runs(portions, shape.num_decode, ops.GLA_CHUNK)
+            per = -(-portions // ops.GLA_CHUNK)
+            shape.add(self.LISTS, np.concatenate([seqs, t0, np.cumsum(per) - per]))
+
     def load(self, tensors, runtime):
         s = self.spec
         qk, v = s.num_heads * s.head_dim, s.num_heads * s.value_dim
@@ -261,13 +276,15 @@ class GatedLinearAttention(Mixer):
         self.norm_weight = tensors[self._t("norm")].repeat(s.num_heads).contiguous()
         self.w_o = runtime.weight(tensors[self._t("o")])
         self.q_scale = float(s.head_dim) ** -0.5
+        self.chunked = bool(runtime.dtype == torch.bfloat16 and qk % 8 == 0 and v % 8 == 0
+                            and ops.gla_chunk_supports(s.head_dim, s.value_dim))
         self.linear = runtime.linear
         self.linear_deferred = runtime.linear_deferred
 
     def forward(self, ctx, x: torch.Tensor, cache):
         s, off = self.spec, self.offsets
         n = x.shape[0]
-        proj = ctx.buffer("gla_proj", (n, self.in_width), torch.float32)
+        proj = ctx.buffer("gla_proj", (n, self.in_width), ctx.dtype if self.chunked else torch.float32)
         self.linear(x, self.w_in, proj)
         low = ctx.buffer("gla_low", (n, self.rank), torch.float32)
         self.linear(x, self.w_a1, low)
@@ -275,9 +292,19 @@ class GatedLinearAttention(Mixer):
         ops.dt_softplus(low, self.w_a2, self.a2_bias, log_decay, sign=-1.0, mult=-1.0 / s.tau)
         read = ctx.buffer("gla_read", (n, s.num_heads * s.value_dim), torch.float32)
         state = cache.state_padded if cache.state_padded is not None else cache.state
-        ops.retention_scan(proj, off["q"], off["k"], off["v"], None, ctx.num_seqs, s.num_heads, s.head_dim, s.value_dim,
-                           ctx.positions, ctx.cu_q, ctx.state_slots, state, read, log_decay=log_decay,
-                           q_scale=self.q_scale)
+        sizes = (s.num_heads, s.head_dim, s.value_dim)
+        in_order = ctx.num_seqs  # sequences whose tokens are walked one by one
+        if self.chunked and ctx.num_seqs > ctx.num_decode:
+            in_order = ctx.num_decode
+            lists = ctx.extras[self.LISTS]
+            rows = n - in_order  # (the single tokens' rows come first)
+            chunks = (lists.shape[0] - (ctx.num_seqs - in_order)) // 2
+            scratch = ctx.buffer("gla_scratch", (ops.gla_chunk_scratch_bytes(rows, chunks, *sizes),), torch.uint8)
+            ops.gla_chunk(proj, off["q"], off["k"], off["v"], log_decay, self.q_scale, in_order, ctx.num_seqs - in_order,
+                          in_order, *sizes, lists, ctx.positions, ctx.cu_q, ctx.state_slots, state, scratch, read)
+        if in_order:
+            ops.retention_scan(proj, off["q"], off["k"], off["v"], None, in_order, *sizes, ctx.positions, ctx.cu_q,
+                               ctx.state_slots, state, read, log_decay=log_decay, q_scale=self.q_scale)
         gated = ctx.buffer("gla_gated", (n, s.num_heads * s.value_dim), ctx.dtype)
         ops.headnorm_gate(read, proj[:, off["g"]:], self.norm_weight, s.eps, gated, s.num_heads, s.value_dim, gate_act="silu")
         return self.linear_deferred(ctx, "gla_out", gated, self.w_o)

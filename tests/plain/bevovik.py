@@ -46,13 +46,14 @@ def key_decays(h, w, prefix: str, m: dict):
 
 
 def decayed_outer_sums(q, k, v, alpha):
-    """One head: S <- diag(alpha_t) S + k_t v_t^T from zero, o_t = S^T q_t."""
-    n, dim = q.shape
-    S = torch.zeros(dim, v.shape[1], dtype=v.dtype)
+    """Head by head: S <- diag(alpha_t) S + k_t v_t^T from zero, o_t = S^T q_t; q, k, alpha [n, heads, dim],
+    v [n, heads, vdim]."""
+    n, heads, dim = q.shape
+    S = torch.zeros(heads, dim, v.shape[2], dtype=v.dtype)
     out = []
     for t in range(n):
-        S = alpha[t][:, None] * S + k[t][:, None] * v[t][None, :]
-        out.append(S.T @ q[t])
+        S = alpha[t][:, :, None] * S + k[t][:, :, None] * v[t][:, None, :]
+        out.append((S * q[t][:, :, None]).sum(dim=1))
     return torch.stack(out)
 
 
@@ -63,8 +64,7 @@ def gated_linear_attention(h, w, prefix: str, m: dict, eps: float):
     k = (h @ w[prefix + ".k"].T).view(n, H, D)
     v = (h @ w[prefix + ".v"].T).view(n, H, V)
     alpha = key_decays(h, w, prefix, m)
-    heads = [decayed_outer_sums(q[:, i], k[:, i], v[:, i], alpha[:, i]) for i in range(H)]
-    o = unit_rms(torch.stack(heads, dim=1), eps) * w[prefix + ".norm"]
+    o = unit_rms(decayed_outer_sums(q, k, v, alpha), eps) * w[prefix + ".norm"]
     g = h @ w[prefix + ".g"].T
     return (o.reshape(n, H * V) * g * torch.sigmoid(g)) @ w[prefix + ".o"].T
 
@@ -207,10 +207,12 @@ def mixture(h, w, prefix: str, m: dict):
     experts = int(m["router"]["experts"])
     chosen, weights = route(h, w, prefix, m["router"])
     out = torch.zeros_like(h)
-    for t in range(h.shape[0]):
-        for e, weight in zip(chosen[t].tolist(), weights[t]):
-            y = h[t] if e >= experts else expert(h[t : t + 1], w, f"{prefix}.e{e}", float(m["expert"]["limit"]))[0]
-            out[t] += weight * y
+    for e in range(int(chosen.max()) + 1):
+        for slot in range(chosen.shape[1]):
+            rows = (chosen[:, slot] == e).nonzero().flatten()
+            if rows.numel():
+                y = h[rows] if e >= experts else expert(h[rows], w, f"{prefix}.e{e}", float(m["expert"]["limit"]))
+                out[rows] += weights[rows, slot, None] * y
     if m.get("shared"):
         out = out + expert(h, w, prefix + ".shared", float(m["shared"]["limit"]))
     return out
