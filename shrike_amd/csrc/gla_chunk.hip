@@ -300,6 +300,16 @@ __global__ void __launch_bounds__(kChainWaves* kWave)
     };
     fetch(0);
     for (int c = 0; c < chunks; ++c) {
+      AFrag ch[DS], cl[DS], cph[2], cpl[2], cvf[kVB][2];
+#pragma unroll
+      for (int ds = 0; ds < DS; ++ds) ch[ds] = qh[ds], cl[ds] = ql[ds];
+#pragma unroll
+      for (int s = 0; s < 2; ++s) {
+        cph[s] = ph[s], cpl[s] = pl[s];
+#pragma unroll
+        for (int vb = 0; vb < kVB; ++vb) cvf[vb][s] = vf[vb][s];
+      }
+      if (c + 1 < chunks) fetch(c + 1);
       // what the state does not enter first: O^T = V^T P^T
       f32x4 o[kVB];
 #pragma unroll
@@ -307,14 +317,10 @@ __global__ void __launch_bounds__(kChainWaves* kWave)
         o[vb] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int s = 0; s < 2; ++s) {
-          o[vb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[vb][s].v, ph[s].v, o[vb], 0, 0, 0);
-          o[vb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[vb][s].v, pl[s].v, o[vb], 0, 0, 0);
+          o[vb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cvf[vb][s].v, cph[s].v, o[vb], 0, 0, 0);
+          o[vb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cvf[vb][s].v, cpl[s].v, o[vb], 0, 0, 0);
         }
       }
-      AFrag ch[DS], cl[DS];
-#pragma unroll
-      for (int ds = 0; ds < DS; ++ds) ch[ds] = qh[ds], cl[ds] = ql[ds];
-      if (c + 1 < chunks) fetch(c + 1);
       __syncthreads();  // the state before this chunk is in buffer c % 2
 #pragma unroll
       for (int ds = 0; ds < DS; ++ds)
@@ -372,6 +378,19 @@ __global__ void __launch_bounds__(kChainWaves* kWave)
   };
   fetch(0);
   for (int c = 0; c < chunks; ++c) {
+    // this chunk's operands aside, so that the next one's are on their way while the state is published and multiplied
+    AFrag ckh[NT][2], ckl[NT][2], cvf[kVB][2];
+    float cwhole[NT];
+#pragma unroll
+    for (int s = 0; s < 2; ++s) {
+#pragma unroll
+      for (int nt = 0; nt < NT; ++nt) ckh[nt][s] = kh[nt][s], ckl[nt][s] = kl[nt][s];
+#pragma unroll
+      for (int vb = 0; vb < kVB; ++vb) cvf[vb][s] = vf[vb][s];
+    }
+#pragma unroll
+    for (int nt = 0; nt < NT; ++nt) cwhole[nt] = whole[nt];
+    if (c + 1 < chunks) fetch(c + 1);
 #pragma unroll
     for (int nt = 0; nt < NT; ++nt) {
       const int d = (own + kOutWaves * nt) * 16 + j;
@@ -387,14 +406,13 @@ __global__ void __launch_bounds__(kChainWaves* kWave)
     for (int nt = 0; nt < NT; ++nt)
 #pragma unroll
       for (int vb = 0; vb < kVB; ++vb) {
-        S[nt][vb] *= whole[nt];
+        S[nt][vb] *= cwhole[nt];
 #pragma unroll
         for (int s = 0; s < 2; ++s) {
-          S[nt][vb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[vb][s].v, kh[nt][s].v, S[nt][vb], 0, 0, 0);
-          S[nt][vb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[vb][s].v, kl[nt][s].v, S[nt][vb], 0, 0, 0);
+          S[nt][vb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cvf[vb][s].v, ckh[nt][s].v, S[nt][vb], 0, 0, 0);
+          S[nt][vb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cvf[vb][s].v, ckl[nt][s].v, S[nt][vb], 0, 0, 0);
         }
       }
-    if (c + 1 < chunks) fetch(c + 1);
   }
 #pragma unroll
   for (int nt = 0; nt < NT; ++nt) {

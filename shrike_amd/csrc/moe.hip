@@ -281,186 +281,168 @@ __global__ void __launch_bounds__(256)
   if (threadIdx.x == 0) counts[e] = base;
 }
 
-// act[pair, f] = act(W_gate_e[f] . x_t) * (W_up_e[f] . x_t) for the pairs of expert e's list: a workgroup
-// takes 32 pairs and four wavefronts' 32 features each
-__global__ void __launch_bounds__(256)
-    moe_gate_up_mfma_kernel(const bf16* __restrict__ x, const int32_t* __restrict__ order,
-                            const int32_t* __restrict__ counts, const bf16* __restrict__ wg,
-                            const bf16* __restrict__ wu, bf16* __restrict__ act_out, int n, int width, int ff, int top,
-                            GateForm form) {
-  const int e = blockIdx.z;
-  const int count = min(counts[e], n);
-  const int row0 = blockIdx.y * 32;
-  if (row0 >= count) return;
-  const bool single = wg == wu;  // experts without a gate: the one product is both factors
-  const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
-  const int i = lane % 16, kg = lane / 16;
-  const int f0 = (blockIdx.x * 4 + wave) * 32;
-  if (f0 >= ff) return;
-  int pair[2];
-  const bf16* xr[2];
-  const bf16* gr[2];
-  const bf16* ur[2];
-#pragma unroll
-  for (int a = 0; a < 2; ++a) {
-    const int r = row0 + a * 16 + i;
-    pair[a] = r < count ? order[static_cast<size_t>(e) * n + r] : -1;
-    const int t = pair[a] >= 0 ? min(pair[a] / top, n - 1) : 0;
-    xr[a] = x + static_cast<size_t>(t) * width + kg * 8;
-    const int f = min(f0 + a * 16 + i, ff - 1);
-    gr[a] = wg + (static_cast<size_t>(e) * ff + f) * width + kg * 8;
-    ur[a] = wu + (static_cast<size_t>(e) * ff + f) * width + kg * 8;
-  }
-  mf32x4 accg[2][2], accu[2][2];
-#pragma unroll
-  for (int a = 0; a < 2; ++a)
-#pragma unroll
-    for (int b = 0; b < 2; ++b) accg[a][b] = accu[a][b] = mf32x4{0.f, 0.f, 0.f, 0.f};
-  if (single) {
-    // one matrix: four steps' operands are asked for at once (eight 16-byte pieces of weights a lane in
-    // flight: few wavefronts run, and what they have in flight is what the memory delivers); the sums
-    // still run over k in ascending order
-    constexpr int kAhead = 4;
-    for (int k0 = 0; k0 < width; k0 += 32 * kAhead) {
-      uint4 av[kAhead][2], gv[kAhead][2];
-#pragma unroll
-      for (int u = 0; u < kAhead; ++u) {
-        const int kk = k0 + 32 * u;
-        const bool have = kk + kg * 8 < width;
-#pragma unroll
-        for (int a = 0; a < 2; ++a) {
-          av[u][a] = gv[u][a] = make_uint4(0, 0, 0, 0);
-          if (have) {
-            gv[u][a] = *reinterpret_cast<const uint4*>(gr[a] + kk);
-            if (pair[a] >= 0) av[u][a] = *reinterpret_cast<const uint4*>(xr[a] + kk);
-          }
-        }
-      }
-#pragma unroll
-      for (int u = 0; u < kAhead; ++u)
-#pragma unroll
-        for (int a = 0; a < 2; ++a)
-#pragma unroll
-          for (int b = 0; b < 2; ++b)
-            accg[a][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(mbf16x8, gv[u][b]),
-                                                                 __builtin_bit_cast(mbf16x8, av[u][a]), accg[a][b], 0, 0, 0);
-    }
-  } else {
-    for (int k0 = 0; k0 < width; k0 += 32) {
-      const bool have = k0 + kg * 8 < width;  // (width is a multiple of 8: a piece is whole or absent)
-      uint4 av[2], gv[2], uv[2];
-#pragma unroll
-      for (int a = 0; a < 2; ++a) {
-        av[a] = gv[a] = uv[a] = make_uint4(0, 0, 0, 0);
-        if (have) {
-          if (pair[a] >= 0) av[a] = *reinterpret_cast<const uint4*>(xr[a] + k0);
-          gv[a] = *reinterpret_cast<const uint4*>(gr[a] + k0);
-          uv[a] = *reinterpret_cast<const uint4*>(ur[a] + k0);
-        }
-      }
-#pragma unroll
-      for (int a = 0; a < 2; ++a)
-#pragma unroll
-        for (int b = 0; b < 2; ++b) {
-          accg[a][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(mbf16x8, gv[b]),
-                                                               __builtin_bit_cast(mbf16x8, av[a]), accg[a][b], 0, 0, 0);
-          accu[a][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(mbf16x8, uv[b]),
-                                                               __builtin_bit_cast(mbf16x8, av[a]), accu[a][b], 0, 0, 0);
-        }
-    }
-  }
-  // features were the rows of the products: this lane holds features f0 + 16 b + 4 kg + r of pair row a * 16 + i
-#pragma unroll
-  for (int a = 0; a < 2; ++a) {
-    if (pair[a] < 0) continue;
-    bf16* dst = act_out + static_cast<size_t>(pair[a]) * ff;
-#pragma unroll
-    for (int b = 0; b < 2; ++b)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int f = f0 + b * 16 + 4 * kg + r;
-        if (f < ff) dst[f] = from_float<bf16>(gate_times_up(accg[a][b][r], single ? accg[a][b][r] : accu[a][b][r], form));
-      }
-  }
-}
+// The two products for lists of few pairs, where what counts is how fast the experts' matrices stream: a
+// workgroup takes 32 pairs and 32 weight rows (of both matrices where there is a gate), its four wavefronts
+// a quarter of k each, so that even one token's experts are read by hundreds of wavefronts; a lane asks for
+// four steps' operands at once.  The quarters' sums meet in LDS and are added in order.
+constexpr int kQuarters = 4;
 
-// pair_out[pair, c] = W_down_e[c] . act[pair]: a workgroup takes 32 pairs and four wavefronts' 64 columns each
-__global__ void __launch_bounds__(256)
-    moe_down_mfma_kernel(const bf16* __restrict__ act_in, const int32_t* __restrict__ order,
-                         const int32_t* __restrict__ counts, const bf16* __restrict__ wd,
-                         float* __restrict__ pair_out, int n, int width, int ff, int top) {
-  const int e = blockIdx.z;
-  const int count = min(counts[e], n);
-  const int row0 = blockIdx.y * 32;
-  if (row0 >= count) return;
-  const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
-  const int i = lane % 16, kg = lane / 16;
-  const int c0 = (blockIdx.x * 4 + wave) * 64;
-  if (c0 >= width) return;
-  int pair[2];
-  const bf16* ar[2];
-  const bf16* wr[4];
-#pragma unroll
-  for (int a = 0; a < 2; ++a) {
-    const int r = row0 + a * 16 + i;
-    pair[a] = r < count ? order[static_cast<size_t>(e) * n + r] : -1;
-    const int p = pair[a] >= 0 ? min(pair[a], n * top - 1) : 0;
-    ar[a] = act_in + static_cast<size_t>(p) * ff + kg * 8;
-  }
-#pragma unroll
-  for (int b = 0; b < 4; ++b) {
-    const int c = min(c0 + b * 16 + i, width - 1);
-    wr[b] = wd + (static_cast<size_t>(e) * width + c) * ff + kg * 8;
-  }
-  mf32x4 acc[2][4];
-#pragma unroll
-  for (int a = 0; a < 2; ++a)
-#pragma unroll
-    for (int b = 0; b < 4; ++b) acc[a][b] = mf32x4{0.f, 0.f, 0.f, 0.f};
-  // two steps' operands are asked for at once (eight 16-byte pieces of weights a lane in flight); the sums
-  // run over k in ascending order all the same
-  constexpr int kAhead = 2;
-  for (int k0 = 0; k0 < ff; k0 += 32 * kAhead) {
-    uint4 av[kAhead][2], wv[kAhead][4];
+// acc[m][a][b] += W_m[row b] . x[pair a] over this wavefront's quarter of k
+template <int MATRICES>
+__device__ __forceinline__ void moe_quarter(const bf16* const (&xr)[2], const bool (&have_pair)[2],
+                                            const bf16* const (&wr)[MATRICES][2], int k, int quarter, int kg,
+                                            mf32x4 (&acc)[MATRICES][2][2]) {
+  constexpr int kAhead = 4;
+  const int per = (k + 32 * kQuarters - 1) / (32 * kQuarters) * 32;
+  const int begin = quarter * per, end = begin + per < k ? begin + per : k;
+  for (int k0 = begin; k0 < end; k0 += 32 * kAhead) {
+    uint4 av[kAhead][2], wv[kAhead][MATRICES][2];
 #pragma unroll
     for (int u = 0; u < kAhead; ++u) {
       const int kk = k0 + 32 * u;
-      const bool have = kk + kg * 8 < ff;
+      const bool have = kk + kg * 8 < end;  // (k is a multiple of 8: a piece is whole or absent)
+#pragma unroll
+      for (int m = 0; m < MATRICES; ++m)
+#pragma unroll
+        for (int b = 0; b < 2; ++b) {
+          wv[u][m][b] = make_uint4(0, 0, 0, 0);
+          if (have) wv[u][m][b] = *reinterpret_cast<const uint4*>(wr[m][b] + kk);
+        }
 #pragma unroll
       for (int a = 0; a < 2; ++a) {
         av[u][a] = make_uint4(0, 0, 0, 0);
-        if (have && pair[a] >= 0) av[u][a] = *reinterpret_cast<const uint4*>(ar[a] + kk);
-      }
-#pragma unroll
-      for (int b = 0; b < 4; ++b) {
-        wv[u][b] = make_uint4(0, 0, 0, 0);
-        if (have) wv[u][b] = *reinterpret_cast<const uint4*>(wr[b] + kk);
+        if (have && have_pair[a]) av[u][a] = *reinterpret_cast<const uint4*>(xr[a] + kk);
       }
     }
 #pragma unroll
     for (int u = 0; u < kAhead; ++u)
 #pragma unroll
-      for (int a = 0; a < 2; ++a)
+      for (int m = 0; m < MATRICES; ++m)
 #pragma unroll
-        for (int b = 0; b < 4; ++b)
-          acc[a][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(mbf16x8, wv[u][b]),
-                                                              __builtin_bit_cast(mbf16x8, av[u][a]), acc[a][b], 0, 0, 0);
+        for (int a = 0; a < 2; ++a)
+#pragma unroll
+          for (int b = 0; b < 2; ++b)
+            acc[m][a][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(mbf16x8, wv[u][m][b]),
+                                                                   __builtin_bit_cast(mbf16x8, av[u][a]), acc[m][a][b], 0, 0, 0);
   }
+}
+
+// The quarters' sums of tile (a, b) = (wave / 2, wave % 2) for this wavefront, added in order.
+template <int MATRICES>
+__device__ __forceinline__ void moe_join_quarters(const mf32x4 (&acc)[MATRICES][2][2], int wave, int lane,
+                                                  float4 (&sums)[kQuarters][4][MATRICES][kWave], mf32x4 (&total)[MATRICES]) {
+#pragma unroll
+  for (int m = 0; m < MATRICES; ++m)
+#pragma unroll
+    for (int a = 0; a < 2; ++a)
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+        sums[wave][2 * a + b][m][lane] = make_float4(acc[m][a][b][0], acc[m][a][b][1], acc[m][a][b][2], acc[m][a][b][3]);
+  __syncthreads();
+#pragma unroll
+  for (int m = 0; m < MATRICES; ++m) {
+    total[m] = mf32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int q = 0; q < kQuarters; ++q) {
+      const float4 x = sums[q][wave][m][lane];
+      total[m][0] += x.x, total[m][1] += x.y, total[m][2] += x.z, total[m][3] += x.w;
+    }
+  }
+}
+
+// act[pair, f] = act(W_gate_e[f] . x_t) * (W_up_e[f] . x_t) for the pairs of expert e's list.  SINGLE: experts
+// without a gate, the one product is both factors.
+template <bool SINGLE>
+__global__ void __launch_bounds__(256)
+    moe_gate_up_mfma_kernel(const bf16* __restrict__ x, const int32_t* __restrict__ order,
+                            const int32_t* __restrict__ counts, const bf16* __restrict__ wg,
+                            const bf16* __restrict__ wu, bf16* __restrict__ act_out, int n, int width, int ff, int top,
+                            GateForm form) {
+  constexpr int M = SINGLE ? 1 : 2;
+  __shared__ float4 sums[kQuarters][4][M][kWave];
+  const int e = blockIdx.z;
+  const int count = min(counts[e], n);
+  const int row0 = blockIdx.y * 32;
+  if (row0 >= count) return;
+  const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
+  const int i = lane % 16, kg = lane / 16;
+  const int f0 = blockIdx.x * 32;
+  int pair[2];
+  bool have[2];
+  const bf16* xr[2];
+  const bf16* wr[M][2];
 #pragma unroll
   for (int a = 0; a < 2; ++a) {
-    if (pair[a] < 0) continue;
-    float* dst = pair_out + static_cast<size_t>(pair[a]) * width;
+    const int r = row0 + a * 16 + i;
+    pair[a] = r < count ? order[static_cast<size_t>(e) * n + r] : -1;
+    have[a] = pair[a] >= 0;
+    const int t = have[a] ? min(pair[a] / top, n - 1) : 0;
+    xr[a] = x + static_cast<size_t>(t) * width + kg * 8;
+    const size_t f = static_cast<size_t>(e) * ff + min(f0 + a * 16 + i, ff - 1);
+    wr[0][a] = wg + f * width + kg * 8;
+    if (!SINGLE) wr[M - 1][a] = wu + f * width + kg * 8;
+  }
+  mf32x4 acc[M][2][2], total[M];
 #pragma unroll
-    for (int b = 0; b < 4; ++b) {
-      const int c = c0 + b * 16 + 4 * kg;
-      if (c + 3 < width) {
-        *reinterpret_cast<float4*>(dst + c) = make_float4(acc[a][b][0], acc[a][b][1], acc[a][b][2], acc[a][b][3]);
-      } else {
+  for (int m = 0; m < M; ++m)
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
-          if (c + r < width) dst[c + r] = acc[a][b][r];
-      }
-    }
+    for (int a = 0; a < 2; ++a)
+#pragma unroll
+      for (int b = 0; b < 2; ++b) acc[m][a][b] = mf32x4{0.f, 0.f, 0.f, 0.f};
+  moe_quarter<M>(xr, have, wr, width, wave, kg, acc);
+  moe_join_quarters<M>(acc, wave, lane, sums, total);
+  // features were the rows of the products: this lane holds features f0 + 16 b + 4 kg + r of pair row a * 16 + i
+  const int p = wave / 2 ? pair[1] : pair[0];
+  if (p < 0) return;
+  const int f = f0 + wave % 2 * 16 + 4 * kg;
+  bf16* dst = act_out + static_cast<size_t>(p) * ff + f;
+#pragma unroll
+  for (int r = 0; r < 4; ++r)
+    if (f + r < ff) dst[r] = from_float<bf16>(gate_times_up(total[0][r], total[M - 1][r], form));
+}
+
+// pair_out[pair, c] = W_down_e[c] . act[pair]
+__global__ void __launch_bounds__(256)
+    moe_down_mfma_kernel(const bf16* __restrict__ act_in, const int32_t* __restrict__ order,
+                         const int32_t* __restrict__ counts, const bf16* __restrict__ wd,
+                         float* __restrict__ pair_out, int n, int width, int ff, int top) {
+  __shared__ float4 sums[kQuarters][4][1][kWave];
+  const int e = blockIdx.z;
+  const int count = min(counts[e], n);
+  const int row0 = blockIdx.y * 32;
+  if (row0 >= count) return;
+  const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
+  const int i = lane % 16, kg = lane / 16;
+  const int c0 = blockIdx.x * 32;
+  int pair[2];
+  bool have[2];
+  const bf16* ar[2];
+  const bf16* wr[1][2];
+#pragma unroll
+  for (int a = 0; a < 2; ++a) {
+    const int r = row0 + a * 16 + i;
+    pair[a] = r < count ? order[static_cast<size_t>(e) * n + r] : -1;
+    have[a] = pair[a] >= 0;
+    ar[a] = act_in + static_cast<size_t>(have[a] ? min(pair[a], n * top - 1) : 0) * ff + kg * 8;
+    wr[0][a] = wd + (static_cast<size_t>(e) * width + min(c0 + a * 16 + i, width - 1)) * ff + kg * 8;
+  }
+  mf32x4 acc[1][2][2], total[1];
+#pragma unroll
+  for (int a = 0; a < 2; ++a)
+#pragma unroll
+    for (int b = 0; b < 2; ++b) acc[0][a][b] = mf32x4{0.f, 0.f, 0.f, 0.f};
+  moe_quarter<1>(ar, have, wr, ff, wave, kg, acc);
+  moe_join_quarters<1>(acc, wave, lane, sums, total);
+  const int p = wave / 2 ? pair[1] : pair[0];
+  if (p < 0) return;
+  const int c = c0 + wave % 2 * 16 + 4 * kg;
+  float* dst = pair_out + static_cast<size_t>(p) * width + c;
+  if (c + 3 < width) {
+    *reinterpret_cast<float4*>(dst) = make_float4(total[0][0], total[0][1], total[0][2], total[0][3]);
+  } else {
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (c + r < width) dst[r] = total[0][r];
   }
 }
 
@@ -469,7 +451,7 @@ __global__ void __launch_bounds__(256)
 // wavefronts (2 x 2) take 64 x 64 each: four A and four B operands from LDS feed sixteen matrix
 // instructions.  Rows of 32 elements lie 80 bytes apart in LDS, so the sixteen 16-byte reads of an
 // operand meet every bank once.  The next step's pieces are fetched into registers while this one is
-// multiplied.  Sums run over k in the same order as in the kernels above: the same bits.
+// multiplied.  Sums run over k in ascending order (in the kernels above, over its quarters).
 constexpr int kTileRows = 128;
 constexpr int kTileLd = 40;  // elements between rows in LDS (32 and 16 bytes of padding)
 
@@ -718,10 +700,16 @@ extern "C" int shk_moe_experts_grouped(const void* x, const int32_t* chosen, con
         ff, width, top, form);
   } else {
     const int row_tiles = (n + 31) / 32;
-    moe_gate_up_mfma_kernel<<<dim3((ff + 127) / 128, row_tiles, experts), 256, 0, s>>>(
-        static_cast<const bf16*>(x), order, counts, static_cast<const bf16*>(w_gate), static_cast<const bf16*>(w_up),
-        static_cast<bf16*>(act_buf), n, width, ff, top, form);
-    moe_down_mfma_kernel<<<dim3((width + 255) / 256, row_tiles, experts), 256, 0, s>>>(
+    const dim3 features((ff + 31) / 32, row_tiles, experts);
+    if (w_gate == w_up)
+      moe_gate_up_mfma_kernel<true><<<features, 256, 0, s>>>(
+          static_cast<const bf16*>(x), order, counts, static_cast<const bf16*>(w_gate), static_cast<const bf16*>(w_up),
+          static_cast<bf16*>(act_buf), n, width, ff, top, form);
+    else
+      moe_gate_up_mfma_kernel<false><<<features, 256, 0, s>>>(
+          static_cast<const bf16*>(x), order, counts, static_cast<const bf16*>(w_gate), static_cast<const bf16*>(w_up),
+          static_cast<bf16*>(act_buf), n, width, ff, top, form);
+    moe_down_mfma_kernel<<<dim3((width + 31) / 32, row_tiles, experts), 256, 0, s>>>(
         static_cast<const bf16*>(act_buf), order, counts, static_cast<const bf16*>(w_down), pair_out, n, width, ff, top);
   }
   moe_join_kernel<<<dim3((width + 255) / 256, n), 256, 0, s>>>(pair_out, chosen, static_cast<const bf16*>(x), weights,

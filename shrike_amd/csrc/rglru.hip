@@ -7,13 +7,14 @@
 // [(taps - 1), width], oldest first; a state counts as zero where the sequence's first row of the
 // step is at position 0.
 //
-// Single tokens: a thread per channel.  Prompt portions: a workgroup of 16 wavefronts owns 32
-// channels of a sequence and walks its tokens in tiles of 256; two halves of a wavefront take 8
-// tokens each.  What does not depend on the state (gates, exponentials, roots) is formed for all
-// tokens of a tile at once, the next tile's inputs are on their way meanwhile, and only the
-// multiply-adds of S pass from group to group through LDS: 8 of them and a barrier a group.  Every
-// token is one multiply-add on the S before it, in order, so a result does not depend on how a
-// prompt was cut.
+// Single tokens: a thread per channel.  Prompt portions: a workgroup of 16 wavefronts owns 16
+// channels of a sequence and walks its tokens in tiles of 512; the quarters of a wavefront take 8
+// tokens each.  (Workgroups with neighbouring channels run on one XCD, whose L2 then serves both
+// halves of a line.)  What does not depend on the state (gates, exponentials, roots) is formed for
+// all tokens of a tile at once, the next tile's inputs are on their way meanwhile, and only the
+// multiply-adds of S pass from run to run, through lane permutations within a wavefront and through
+// LDS and a barrier between wavefronts.  Every token is one multiply-add on the S before it, in
+// order, so a result does not depend on how a prompt was cut.
 #include "api.h"
 #include "common.h"
 
@@ -21,25 +22,44 @@ namespace shk {
 
 namespace {
 
-constexpr int kChannels = 32;   // channels a workgroup of the prompt kernel
+constexpr int kChannels = 16;   // channels a workgroup of the prompt kernel
 constexpr int kRunTokens = 8;   // tokens a lane takes of a tile
-constexpr int kGroups = 32;     // runs of tokens a tile: 16 wavefronts of two halves
+constexpr int kGroups = 64;     // runs of tokens a tile: 16 wavefronts of four quarters
+constexpr int kQuarters = kWave / kChannels;  // runs of tokens a wavefront
+constexpr int kXcds = 8;
 constexpr int kTile = kRunTokens * kGroups;
 
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
+// (bfloat16 models: the hardware's exponential, float32 all the same; float32 models: the library's)
+template <typename T>
+__device__ __forceinline__ float exp_f(float x) {
+  return sizeof(T) == 2 ? __expf(x) : expf(x);
+}
+template <typename T>
+__device__ __forceinline__ float sigmoid_f(float z) {
+  return 1.f / (1.f + exp_f<T>(-z));
+}
+template <typename T>
 __device__ __forceinline__ float gelu_f(float z) {
   const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
-  return z / (1.f + expf(-2.f * u));
+  return z / (1.f + exp_f<T>(-2.f * u));
+}
+
+// 1 - a^2 for a = exp(-x / 2): below 1/4 the series x - x^2 / 2! + x^3 / 3! - ... (what is left out is less than
+// 2^-24 of the sum), where 1 - a a would lose what a small rate leaves
+__device__ __forceinline__ float one_less_square(float x, float a) {
+  const float series = x * (1.f - x * (1.f / 2) * (1.f - x * (1.f / 3) * (1.f - x * (1.f / 4) * (1.f - x * (1.f / 5) * (1.f - x * (1.f / 6))))));
+  return x < 0.25f ? series : 1.f - a * a;
 }
 
 struct Step {
   float a, x;  // S <- a S + x
 };
+template <typename T>
 __device__ __forceinline__ Step make_step(float zr, float zi, float u, float br, float bi, float rate) {
-  const float log_a = -rate * sigmoid_f(zr + br);
+  const float less = rate * sigmoid_f<T>(zr + br);
   Step s;
-  s.a = expf(log_a);
-  s.x = sqrtf(-expm1f(2.f * log_a)) * (sigmoid_f(zi + bi) * u);
+  s.a = exp_f<T>(-less);
+  s.x = sqrtf(one_less_square(2.f * less, s.a)) * (sigmoid_f<T>(zi + bi) * u);
   return s;
 }
 
@@ -82,12 +102,18 @@ __global__ void __launch_bounds__(256)
   const int col = gate_column(c, part);
   for (int t = first; t < last; ++t) {
     const float* z = gates + static_cast<size_t>(t) * 2 * width + col;
-    const Step s = make_step(z[0], z[part], to_float(u[static_cast<size_t>(t) * width + c]), b_r, b_i, rt);
+    const Step s = make_step<T>(z[0], z[part], to_float(u[static_cast<size_t>(t) * width + c]), b_r, b_i, rt);
     S = fmaf(s.a, S, s.x);
-    out[static_cast<size_t>(t) * width + c] = from_float<T>(S * gelu_f(to_float(y[static_cast<size_t>(t) * ldy + c])));
+    out[static_cast<size_t>(t) * width + c] = from_float<T>(S * gelu_f<T>(to_float(y[static_cast<size_t>(t) * ldy + c])));
   }
   slot[c] = S;
   keep_tail(slot + width, raw, ld_raw, c, width, taps, first, last, fresh);
+}
+
+// workgroups a sequence: as many on every XCD
+inline int blocks_of(int width) {
+  const int blocks = (width + kChannels - 1) / kChannels;
+  return (blocks + kXcds - 1) / kXcds * kXcds;
 }
 
 template <typename T>
@@ -103,7 +129,9 @@ __global__ void __launch_bounds__(16 * kWave)
   const int first = cu_q[seq], last = cu_q[seq + 1];
   if (last <= first) return;
   const int group = threadIdx.x / kChannels;  // this thread's run of tokens within a tile
-  const int c_raw = blockIdx.x * kChannels + threadIdx.x % kChannels;
+  const int per_xcd = gridDim.x / kXcds;  // (workgroups go to the XCDs in turn)
+  const int c_raw = (blockIdx.x % kXcds * per_xcd + blockIdx.x / kXcds) * kChannels + threadIdx.x % kChannels;
+  if (c_raw - threadIdx.x % kChannels >= width) return;
   const bool active = c_raw < width;
   const int c = active ? c_raw : width - 1;
   const bool fresh = positions[first] == 0;
@@ -131,24 +159,30 @@ __global__ void __launch_bounds__(16 * kWave)
     float a[kRunTokens], x[kRunTokens], gy[kRunTokens];
 #pragma unroll
     for (int i = 0; i < kRunTokens; ++i) {
-      const Step s = make_step(zr[i], zi[i], to_float(uv[i]), b_r, b_i, rt);
+      const Step s = make_step<T>(zr[i], zi[i], to_float(uv[i]), b_r, b_i, rt);
       const bool in = t0 + group * kRunTokens + i < last;
       a[i] = in ? s.a : 1.f;  // behind the portion S stays
       x[i] = in ? s.x : 0.f;
-      gy[i] = gelu_f(to_float(yv[i]));
+      gy[i] = gelu_f<T>(to_float(yv[i]));
     }
     if (t0 + kTile < last) fetch(t0 + kTile);
     const int left = last - t0;
-    const int runs = left >= kTile ? kGroups : (left + kRunTokens - 1) / kRunTokens;
-    for (int g = 0; g < runs; ++g) {
-      if (g == group) {
+    const int waves = left >= kTile ? kGroups / kQuarters : (left + kRunTokens * kQuarters - 1) / (kRunTokens * kQuarters);
+    for (int w = 0; w < waves; ++w) {
+      if (w == group / kQuarters) {  // (the whole wavefront)
         float S = carry[threadIdx.x % kChannels];
 #pragma unroll
-        for (int i = 0; i < kRunTokens; ++i) {
-          S = fmaf(a[i], S, x[i]);
-          a[i] = S;
+        for (int q = 0; q < kQuarters; ++q) {
+          if (q == group % kQuarters) {
+#pragma unroll
+            for (int i = 0; i < kRunTokens; ++i) {
+              S = fmaf(a[i], S, x[i]);
+              a[i] = S;
+            }
+          }
+          S = __shfl(S, q * kChannels + threadIdx.x % kChannels, kWave);  // what this quarter ends with, for the next
         }
-        carry[threadIdx.x % kChannels] = S;
+        if (threadIdx.x % kWave < kChannels) carry[threadIdx.x % kChannels] = S;
       }
       __syncthreads();
     }
@@ -198,7 +232,7 @@ extern "C" int shk_rglru(const float* gates, int blocks, const float* bias_r, co
           static_cast<const T*>(raw), ld_raw, width, taps, positions, cu_q, slots, state, slot_stride,                \
           static_cast<T*>(out));                                                                                      \
     if (num_seqs > num_single)                                                                                        \
-      rglru_scan_kernel<T><<<dim3((width + kChannels - 1) / kChannels, num_seqs - num_single), 16 * kWave, 0, s>>>(   \
+      rglru_scan_kernel<T><<<dim3(blocks_of(width), num_seqs - num_single), 16 * kWave, 0, s>>>(   \
           gates, part, bias_r, bias_i, rate, static_cast<const T*>(u), static_cast<const T*>(y), ldy,                 \
           static_cast<const T*>(raw), ld_raw, width, taps, num_single, positions, cu_q, slots, state, slot_stride,    \
           static_cast<T*>(out));                                                                                      \

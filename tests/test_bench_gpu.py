@@ -58,3 +58,24 @@ def test_the_second_design_of_the_comparison_is_built_from_the_first_ones_sizes_
     engine = bench.make_engine(sizes, minilorn.build_spec(mcfg), 4, seed=1)
     run = bench.run_decode(engine, sizes, 4, steps=10, warmup=2, seed=5, prompt_len=70)
     assert run["context_end"] - run["context_start"] == 10 and run["tok_s"] > 0
+
+
+def test_the_bevovik_of_the_comparison_is_built_from_the_first_ones_sizes_and_decodes():
+    """bench.py --bevovik: a Qwen2 configuration's width, vocabulary and number of layers, every mixer in the
+    pattern's order, experts that together are as large as its feed-forward."""
+    import shrike_amd.models  # noqa: F401
+    from shrike_amd.models import bevovik
+    from shrike_amd.models.qwen2 import Qwen2Config
+
+    qcfg = Qwen2Config.from_dict(dict(CONFIGS["B"], hidden_size=256, num_hidden_layers=4, torch_dtype="bfloat16"))
+    bcfg, sizes = bench.bevovik_like(qcfg, "grl", experts=6, top=2)
+    assert [layer.type for layer in bcfg.layers] == ["gla", "rglru", "latent_attention", "gla"]
+    assert bcfg.width == 256 and bcfg.vocab == qcfg.vocab_size and sizes.kv_elements_per_token > 0
+    router = bcfg.layers[0].mlp
+    assert (router.experts, router.identity, router.groups, router.top) == (6, 2, (2, 1), 2)
+    few = sizes.layer_elements
+    sizes.at_batch(64)
+    assert sizes.layer_elements > few, "many tokens touch more experts than one token's"
+    engine = bench.make_engine(sizes, bevovik.build_spec(bcfg), 4, seed=1)
+    run = bench.run_decode(engine, sizes, 4, steps=10, warmup=2, seed=5, prompt_len=70)
+    assert run["context_end"] - run["context_start"] == 10 and run["tok_s"] > 0
