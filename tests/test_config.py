@@ -1,6 +1,5 @@
 """Configuration and registry (CPU)."""
 
-import importlib
 import json
 
 import pytest
@@ -142,26 +141,17 @@ def test_engine_config_validation():
             EngineConfig(**bad)
 
 
-def test_default_model_dir_env_override(monkeypatch):
+def test_default_model_dir_env_override():
     # shrike/config.py:29
-    import shrike_amd.config.registry as reg
+    import os
+    import subprocess
+    import sys
 
-    monkeypatch.setenv("SHRIKE_MODEL_DIR", "/somewhere/else")
-    importlib.reload(reg)
-    assert reg.DEFAULT_MODEL_DIR == "/somewhere/else"
-    monkeypatch.delenv("SHRIKE_MODEL_DIR")
-    importlib.reload(reg)
-    import shrike_amd.models.ligipel as lg
-    import shrike_amd.models.minilorn as n
-    import shrike_amd.models.mofarax as m
-    import shrike_amd.models.poresun as po
-    import shrike_amd.models.qwen2 as q
-
-    importlib.reload(q)  # the reload emptied the registry; register again
-    importlib.reload(m)
-    importlib.reload(n)
-    importlib.reload(lg)
-    importlib.reload(po)
+    # (read once, when the module is imported: a process of its own)
+    code = "import shrike_amd.config.registry as r; print(r.DEFAULT_MODEL_DIR)"
+    env = {**os.environ, "SHRIKE_MODEL_DIR": "/somewhere/else"}
+    out = subprocess.run([sys.executable, "-c", code], env=env, capture_output=True, text=True, timeout=120, check=True)
+    assert out.stdout.strip() == "/somewhere/else"
 
 
 def test_plugins_named_in_the_environment_are_loaded_for_an_unknown_architecture(tmp_path, monkeypatch):

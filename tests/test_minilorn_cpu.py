@@ -8,7 +8,7 @@ import pytest
 import torch
 
 import shrike_amd.models  # noqa: F401  (registers the architectures)
-from shrike_amd.config import registry  # (names through the module: another test reloads it)
+from shrike_amd.config import registry
 from shrike_amd.models import DecoderModel
 from shrike_amd.parts import PagedSpec, StateSpec
 
